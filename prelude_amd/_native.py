@@ -73,7 +73,7 @@ _KERNEL_API = {
     "pa_clamped_gate": (I, [P, I, P, P, I, I, F, F]),
     "pa_relu_squared": (I, [P, I, P, P, c_long]),
     "pa_latent_prep": (I, [P, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, F, c_long]),
-    "pa_rotate_pairs": (I, [P, I, P, P, P, P, I, I, I, I, I, I, I, I]),
+    "pa_rotate_pairs": (I, [P, I, P, P, P, P, I, I, I, I, I, I, I, I, c_long]),
     "pa_head_linear": (I, [P, I, P, P, P, I, I, I, I, c_long, c_long, c_long, c_long]),
     "pa_latent_attn": (I, [P, I, P, P, P, P, I, P, P, P, I, I, I, I, I, I, F]),
     "pa_latent_attn_mfma_supports": (I, [I, I, I]),
@@ -118,6 +118,16 @@ _KERNEL_API = {
     "pa_pair_embed": (I, [P, I, P, P, P, P, P, P, P, P, P, I, I, I, I, c_long, c_long, F]),
     "pa_time_conv_add": (I, [P, I, P, P, P, P, P, P, P, I, I, I, I, I]),
     "pa_stream_add_row": (I, [P, P, P, I, I]),
+    "pa_layer_norm_step": (I, [P, I, P, P, I, c_long, P, P, P, P, P, I, I, F]),
+    "pa_stream_sum": (I, [P, I, P, P, P, P, P, I, I]),
+    "pa_embed_scaled": (I, [P, I, P, P, P, I, I, I, F]),
+    "pa_activate": (I, [P, I, P, c_long, P, c_long, I, I, I, F]),
+    "pa_talking_prepare": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, F]),
+    "pa_gla_decay": (I, [P, I, P, c_long, I, P, P, P, I, I, I, F]),
+    "pa_gla_attn": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, I, I, I, I, I, F, I, I]),
+    "pa_gla_step": (I, [P, I, P, c_long, I, I, I, I, P, P, P, P, P, P, I, I, I, I, I, F, F]),
+    "pa_gla_chunked_workspace": (c_long, [I, I, I, I, I, I]),
+    "pa_gla_attn_chunked": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I]),
     "pa_stream_add_branches": (I, [P, I, P, P, P, c_long]),
     "pa_qkv_rope_prepare": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I]),
     "pa_diff_combine": (I, [P, I, P, P, I, I, I, F, F, F]),

@@ -787,3 +787,133 @@ class NivasunConfig:
                    embed_scale=_get(emb, "scale", float, a, default=1.0), buckets=_positive(pair, "buckets", int, a, pw),
                    mul_prev=mul["mul_prev"], mul_cur=mul["mul_cur"], logit_cap=cap,
                    loop_start=start, loop_stop=stop, loop_times=times, layers=tuple(layers), has_loop=loop is not None)
+
+
+# ---------------------------------------------------------------------------
+@dataclasses.dataclass(frozen=True)
+class PugavikMixerConfig:
+    heads: int
+    dim: int            # query/key dimensions a head (latent attention: the unrotated ones)
+    vdim: int
+    kv_heads: int = 0   # attention
+    window: int = 0     # attention: the query at i sees the key at j with 0 <= i - j < window
+    scale: float = 1.0  # attention, latent attention
+    rot_dims: int = 0   # dimensions that turn, in pairs
+    rot_base: float = 1.0
+    rot_dim: int = 0    # latent attention: rotated query/key dimensions a head (the key's are shared by all heads)
+    kv_rank: int = 0
+    tau: float = 1.0    # gla
+    rank: Optional[int] = None   # gla: inner size of the decays' two-step projection; None: what the tensors have
+
+
+@dataclasses.dataclass(frozen=True)
+class PugavikLayerConfig:
+    type: str
+    mixer: PugavikMixerConfig
+    ff: int             # inner size of the dense feed-forward; 0: the layer has none
+
+
+@dataclasses.dataclass(frozen=True)
+class PugavikConfig:
+    """Pugavik: a decoder whose layers are listed one by one in ``layers``; a stretch of them (``loop``) runs several times in a
+    row on the same tensors, with the embedding added again in front of every pass but the first and a learned vector in
+    front of every pass.  A layer has one layer norm whose output the mixer and the feed-forward both read; both are added
+    to the stream together.  Mixers: ``attention`` (biases, queries and keys normed per head, rotation in pairs, values over
+    their own root mean square, the heads' scores mixed by a matrix, a sliding window, a sink), ``gla`` (gated linear attention
+    with a decay per key channel), ``latent_attention`` (keys and values through a latent with a shared rotated key part).
+    The feed-forward is dense (GELU in its tanh form), or absent.  Every size and constant is read from here; there is no
+    longest position and no end-of-sequence id."""
+    vocab: int
+    width: int
+    norm_eps: float
+    embed_scale: float
+    loop_start: int
+    loop_stop: int
+    loop_times: int             # 1 with start == stop: no loop
+    layers: Tuple[PugavikLayerConfig, ...]
+    has_loop: bool = False      # the configuration has a `loop` (its file then holds a vector per pass, also for an empty stretch)
+
+    ARCH = "Pugavik"
+    MIXERS = ("attention", "gla", "latent_attention")
+
+    @classmethod
+    def _rot(cls, m: Mapping[str, Any], mw: str, dim: int, what: str, optional: bool):
+        a = cls.ARCH
+        rot = _obj(m, "rot", a, mw, optional=optional)
+        if rot is None:
+            return 0, 1.0
+        try:
+            dims = _get(rot, "dims", int, a)
+        except ConfigError as e:
+            raise ConfigError(str(e).replace("`dims`", f"`{mw}rot.dims`")) from None
+        if dims % 2 or dims > dim:
+            raise ConfigError(f"failed to parse {a} config: `{mw}rot.dims` ({dims}) must be even and at most `{what}` ({dim})")
+        return dims, (_positive(rot, "base", float, a, mw + "rot.") if dims else 1.0)
+
+    @classmethod
+    def _mixer(cls, kind: str, m: Mapping[str, Any], mw: str) -> PugavikMixerConfig:
+        a = cls.ARCH
+        heads, dim, vdim = (_positive(m, k, int, a, mw) for k in ("heads", "dim", "vdim"))
+        if kind == "gla":
+            rank = _positive(m, "rank", int, a, mw) if m.get("rank") is not None else None
+            return PugavikMixerConfig(heads, dim, vdim, tau=_positive(m, "tau", float, a, mw), rank=rank)
+        scale = _positive(m, "scale", float, a, mw)
+        if kind == "latent_attention":
+            try:
+                rot_dim = _get(m, "rot_dim", int, a)
+            except ConfigError as e:
+                raise ConfigError(str(e).replace("`rot_dim`", f"`{mw}rot_dim`")) from None
+            dims, base = cls._rot(m, mw, rot_dim, "rot_dim", optional=rot_dim == 0)
+            if dims != rot_dim:
+                raise ConfigError(f"failed to parse {a} config: `{mw}rot.dims` ({dims}) must equal `rot_dim` ({rot_dim}): the rotated "
+                                  f"part turns whole")
+            return PugavikMixerConfig(heads, dim, vdim, scale=scale, rot_dims=dims, rot_base=base, rot_dim=rot_dim,
+                                      kv_rank=_positive(m, "kv_rank", int, a, mw))
+        kv_heads = _positive(m, "kv_heads", int, a, mw)
+        if heads % kv_heads:
+            raise ConfigError(f"failed to parse {a} config: `{mw}heads` ({heads}) is no multiple of `kv_heads` ({kv_heads})")
+        dims, base = cls._rot(m, mw, dim, "dim", optional=True)
+        return PugavikMixerConfig(heads, dim, vdim, kv_heads=kv_heads, scale=scale, rot_dims=dims, rot_base=base,
+                                  window=_positive(_obj(m, "mask", a, mw), "size", int, a, mw + "mask."))
+
+    @classmethod
+    def from_dict(cls, raw: Mapping[str, Any]) -> "PugavikConfig":
+        a = cls.ARCH
+        layers_raw = raw.get("layers")
+        if not isinstance(layers_raw, list) or not layers_raw:
+            raise ConfigError(f"failed to parse {a} config: `layers` must be a non-empty list")
+        layers = []
+        for i, lr in enumerate(layers_raw):
+            w = f"layers[{i}]."
+            if not isinstance(lr, dict):
+                raise ConfigError(f"failed to parse {a} config: `layers[{i}]` must be an object")
+            kind = _get(lr, "type", str, a)
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"failed to parse {a} config: `{w}type` {kind!r} is not one of {list(cls.MIXERS)}")
+            f = _obj(lr, "mlp", a, w, optional=True)
+            ff = 0
+            if f is not None:
+                fk = _get(f, "kind", str, a, default="dense")
+                if fk != "dense":
+                    raise ConfigError(f"failed to parse {a} config: `{w}mlp.kind` {fk!r} is not one of ['dense']")
+                ff = _positive(f, "ff", int, a, w + "mlp.")
+            layers.append(PugavikLayerConfig(kind, cls._mixer(kind, _obj(lr, "mixer", a, w), w + "mixer."), ff))
+        loop = _obj(raw, "loop", a, optional=True)
+        start, stop, times = 0, 0, 1
+        if loop is not None:
+            try:
+                start, stop = _get(loop, "start", int, a), _get(loop, "stop", int, a)
+            except ConfigError as e:
+                raise ConfigError(str(e).replace("`start`", "`loop.start`").replace("`stop`", "`loop.stop`")) from None
+            times = _positive(loop, "times", int, a, "loop.")
+            if not 0 <= start <= stop <= len(layers):
+                raise ConfigError(f"failed to parse {a} config: `loop.start` ({start}) and `loop.stop` ({stop}) must lie in order "
+                                  f"within the {len(layers)} layers")
+        emb = _obj(raw, "embedding", a)
+        try:
+            scale = _get(emb, "scale", float, a)
+        except ConfigError as e:
+            raise ConfigError(str(e).replace("`scale`", "`embedding.scale`")) from None
+        return cls(vocab=_positive(raw, "vocab", int, a, ""), width=_positive(raw, "width", int, a, ""),
+                   norm_eps=_positive(_obj(raw, "norm", a), "eps", float, a, "norm."), embed_scale=scale, loop_start=start,
+                   loop_stop=stop, loop_times=times, layers=tuple(layers), has_loop=loop is not None)

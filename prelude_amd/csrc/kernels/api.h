@@ -227,6 +227,22 @@ int pa_lightning_attn_chunked(void* stream, int dtype, const void* qkv, long ld,
                               const float* decay, float* state, const int* state_slots, const int* cu_q, const int* seq_ids,
                               float* out, float* work, int nlisted, int tokens, int max_len, int heads, int dim, int vdim,
                               int act, int chunk);
+// Gated linear attention: the same with a decay per token, head and key channel, alpha [tokens, heads, dim] 32-bit, and
+// queries times q_scale.  pa_gla_decay: alpha = sigmoid(A2 low + bias)^(1 / tau), A2 [channels, rank] and low [rank] of
+// `dtype`, low at column low_off of a token's row of p; pa_gla_step (the step's sequences of exactly one token) makes its
+// own decays from the same.
+int pa_gla_decay(void* stream, int dtype, const void* p, long ld, int low_off, const void* a2, const float* bias, float* alpha,
+                 int tokens, int channels, int rank, float tau);
+int pa_gla_attn(void* stream, int dtype, const void* qkv, long ld, int q_off, int k_off, int v_off, const float* alpha,
+                float* state, const int* state_slots, const int* cu_q, float* out, int nseq, int tokens, int heads, int dim,
+                int vdim, float q_scale, int max_len, int min_len);
+int pa_gla_step(void* stream, int dtype, const void* qkv, long ld, int q_off, int k_off, int v_off, int low_off, const void* a2,
+                const float* bias, float* state, const int* state_slots, const int* cu_q, float* out, int nseq, int heads, int dim,
+                int vdim, int rank, float tau, float q_scale);
+long pa_gla_chunked_workspace(int nlisted, int tokens, int heads, int dim, int vdim, int chunk);
+int pa_gla_attn_chunked(void* stream, int dtype, const void* qkv, long ld, int q_off, int k_off, int v_off, const float* alpha,
+                        float* state, const int* state_slots, const int* cu_q, const int* seq_ids, float* out, float* work,
+                        int nlisted, int tokens, int max_len, int heads, int dim, int vdim, float q_scale, int chunk);
 
 // ---- attention through a latent (latent.hip) ----
 // in [tokens, q_rank + rank + rot]: cq_out [tokens, q_rank] = RMSNorm(first part) * wq; into the cache row slots[t]
@@ -241,9 +257,9 @@ int pa_latent_prep(void* stream, int dtype, const void* in, const float* wq, con
 int pa_latent_gather(void* stream, int dtype, const void* cache, const int* block_table, int table_stride, const int* seq,
                      const int* pos, void* out, int rows, int rank, int width, int page_size);
 // in [tokens, heads, in_stride] -> out [tokens, heads, out_stride]: `width` elements from in_off to out_off of every
-// head, the first rot_dims of them rotated in pairs
+// head, the first rot_dims of them rotated in pairs; in_token > 0: the input's tokens are that many elements apart
 int pa_rotate_pairs(void* stream, int dtype, const void* in, void* out, const float* inv_freq, const int* positions,
-                    int tokens, int heads, int in_stride, int in_off, int out_stride, int out_off, int width, int rot_dims);
+                    int tokens, int heads, int in_stride, int in_off, int out_stride, int out_off, int width, int rot_dims, long in_token);
 // y[t, h, n] = sum_k x[t, h, k] wt[h, k, n]; strides in elements
 int pa_head_linear(void* stream, int dtype, const void* x, const void* wt, void* y, int tokens, int heads, int K, int N,
                    long xs_t, long xs_h, long ys_t, long ys_h);
@@ -335,6 +351,30 @@ int pa_pair_embed(void* stream, int dtype, const int* ids, const int* positions,
 int pa_time_conv_add(void* stream, int dtype, const void* h, const float* w, float* state, const int* seq_of_token,
                      const int* cu_q, const int* state_slots, void* out, int tokens, int nseq, int channels, int taps,
                      int all_single);
+// ---- layer norm around a 32-bit stream (layer_norm.hip) ----
+// residual += y (a tensor of `dtype`, or `slices` 32-bit partial sums slice_stride elements apart, or neither), then out =
+// layer norm of the row, times w plus b.  With rows: of those rows alone, the residual read only.
+int pa_layer_norm_step(void* stream, int dtype, const void* y, const float* parts, int slices, long slice_stride, float* residual,
+                       const float* w, const float* b, void* out, const int* rows, int nrows, int hidden, float eps);
+// out = x + y + extra + row (y of `dtype` [tokens, hidden], extra likewise in 32-bit, row [hidden]; each may be null); out may be x
+int pa_stream_sum(void* stream, int dtype, const float* x, const void* y, const float* extra, const float* row, float* out,
+                  int tokens, int hidden);
+// out[t] = table[ids[t]] * scale, 32-bit
+int pa_embed_scaled(void* stream, int dtype, const int* ids, const void* table, float* out, int tokens, int hidden, int vocab,
+                    float scale);
+// out = act(x) * scale, rows inside wider ones; act as in pa_silu_mul
+int pa_activate(void* stream, int dtype, const void* x, long x_stride, void* out, long out_stride, int rows, int width, int act,
+                float scale);
+// ---- in front of attention whose heads' scores are mixed (talking_heads.hip) ----
+// p rows -> q_out [tokens, nh, nkv * hd]: queries (bias, norm per head, first `rot` dimensions turned in pairs) mixed by
+// talk [nh, nh] over the key heads side by side; keys likewise -> K [page, offset, nkv * hd]; values (bias; over their own
+// root mean square with value_norm) -> V [page, nkv, vd, offset].  Biases, weights and slots may be null.
+int pa_talking_prepare(void* stream, int dtype, const void* p, long stride, int q_off, int k_off, int v_off, const float* q_bias,
+                       const float* k_bias, const float* v_bias, const float* q_weight, const float* k_weight,
+                       const float* inv_freq, const int* positions, const float* talk, const int* slots, void* q_out,
+                       void* k_cache, void* v_cache, int tokens, int nh, int nkv, int hd, int vd, int rot, int value_norm,
+                       int page_size, float eps);
+
 int pa_stream_add_row(void* stream, float* x, const float* row, int tokens, int hidden);
 int pa_stream_add_branches(void* stream, int dtype, float* x, const void* a, const void* b, long total);
 int pa_qkv_rope_prepare(void* stream, int dtype, const void* p, long stride, int q_off, int k_off, int v_off,

@@ -33,7 +33,8 @@
 namespace pa {
 
 constexpr int kMaskedWaves = 4;
-constexpr int kMaskedMaxDim = 256;
+constexpr int kMaskedMaxDim = 256;     // widest value
+constexpr int kMaskedMaxKey = 4096;    // widest key (the queries lie in LDS)
 
 template <typename T>
 __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
@@ -42,9 +43,10 @@ __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
     const int* __restrict__ positions, T* __restrict__ out, size_t out_stride, int nh, int nkv, int hd, int vd,
     int page_size, int window, int keep_first, float scale, float softcap, const float* __restrict__ slopes,
     const float* __restrict__ sink, const T* __restrict__ gate, size_t gate_stride, float out_scale, int nv) {
-  __shared__ float qs[kMaskedWaves][kMaskedMaxDim];
+  extern __shared__ float qs_all[];            // a query a wavefront
   __shared__ float ps[kMaskedWaves][kWave];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  float* qs = qs_all + (size_t)wave * hd;
   const int t = blockIdx.x;
   const int h = blockIdx.y * kMaskedWaves + wave;
   const bool active = h < nh;  // every wave of the block shares the token, hence the trip counts below
@@ -59,13 +61,15 @@ __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
   const int first_window_chunk = lo / kWave > kept_chunks ? lo / kWave : kept_chunks;
   const int last_chunk = hi / kWave;
   const int kvh = active ? h / (nh / nkv) : 0;
-  const int vh = kvh % nv;   // fewer value heads than key heads: key head k goes with value head k mod nv
+  // fewer value heads than key heads: key head k goes with value head k mod nv; more: the query heads are dealt out to
+  // the value heads as they are to the key heads
+  const int vh = nv <= nkv ? kvh % nv : (active ? h / (nh / nv) : 0);
   const int* table = block_table + (size_t)seq * table_stride;
   const float slope = (slopes && active) ? slopes[h] : 0.f;
 
   if (active) {
     const T* qr = q + ((size_t)t * nh + h) * hd;
-    for (int d = lane; d < hd; d += kWave) qs[wave][d] = to_f32(qr[d]);
+    for (int d = lane; d < hd; d += kWave) qs[d] = to_f32(qr[d]);
   }
   __syncthreads();
 
@@ -81,7 +85,7 @@ __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
       const int page = table[c / page_size];
       const T* kr = k_cache + (((size_t)page * nkv + kvh) * page_size + (c % page_size)) * hd;
       float dot = 0.f;
-      for (int d = 0; d < hd; ++d) dot = fmaf(qs[wave][d], to_f32(kr[d]), dot);
+      for (int d = 0; d < hd; ++d) dot = fmaf(qs[d], to_f32(kr[d]), dot);
       s = dot * scale;
       if (softcap != 0.f) s = softcap * tanhf(s / softcap);
       s -= slope * (float)(pos - c);
@@ -441,18 +445,19 @@ extern "C" int pa_attn_masked(void* stream, int dtype, const void* q, const void
                               const int* context_lens, int nseq, int max_q_len, int nv) {
   if (tokens == 0) return 0;
   if (nv <= 0) nv = nkv;
-  PA_REQUIRE(nkv % nv == 0, "attn_masked: %d key heads are not a multiple of %d value heads", nkv, nv);
+  PA_REQUIRE(nkv % nv == 0 || (nv % nkv == 0 && nh % nv == 0), "attn_masked: %d key heads and %d value heads for %d query heads",
+             nkv, nv, nh);
   PA_REQUIRE(tokens > 0 && nh > 0 && nkv > 0 && page_size > 0 && table_stride > 0,
              "attn_masked: bad sizes tokens=%d nh=%d nkv=%d page=%d table_stride=%d", tokens, nh, nkv, page_size, table_stride);
   PA_REQUIRE(nh % nkv == 0, "attn_masked: %d query heads are not a multiple of %d KV heads", nh, nkv);
-  PA_REQUIRE(hd > 0 && hd <= kMaskedMaxDim && vd > 0 && vd <= kMaskedMaxDim,
-             "attn_masked: key width %d or value width %d is outside 1..%d", hd, vd, kMaskedMaxDim);
+  PA_REQUIRE(hd > 0 && hd <= kMaskedMaxKey && vd > 0 && vd <= kMaskedMaxDim,
+             "attn_masked: key width %d is outside 1..%d or value width %d outside 1..%d", hd, kMaskedMaxKey, vd, kMaskedMaxDim);
   PA_REQUIRE(window >= 0 && keep_first >= 0, "attn_masked: window %d or kept first tokens %d negative", window, keep_first);
   PA_REQUIRE(softcap >= 0.f, "attn_masked: a score cap of %g is negative (0 means none)", (double)softcap);
   PA_REQUIRE(out_stride >= (long)nh * vd && (!gate || gate_stride >= nh), "attn_masked: output stride %ld or gate stride %ld "
              "too small for %d heads of %d", out_stride, gate_stride, nh, vd);
   hipStream_t st = (hipStream_t)stream;
-  if (dtype == kBF16 && pa_attn_masked_mfma_supports(hd, vd, page_size) && cu_q && context_lens && nseq > 0 && max_q_len > 0) {
+  if (dtype == kBF16 && nv <= nkv && pa_attn_masked_mfma_supports(hd, vd, page_size) && cu_q && context_lens && nseq > 0 && max_q_len > 0) {
     const int group = nh / nkv;
     // two heads a wavefront where the group is even: four leave a head of 128 no registers and measured slower
     const int gt = group % 2 == 0 ? 2 : 1;
@@ -483,13 +488,22 @@ extern "C" int pa_attn_masked(void* stream, int dtype, const void* q, const void
     return check_launch("attn_masked (matrix cores)");
   }
   dim3 grid(tokens, (nh + kMaskedWaves - 1) / kMaskedWaves);
+  const size_t lds = (size_t)kMaskedWaves * hd * sizeof(float);
+  if (lds > 65536 - sizeof(float) * kMaskedWaves * kWave) {
+    static const hipError_t allowed[2] = {
+        hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_masked_kernel<float>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                            kMaskedWaves * kMaskedMaxKey * (int)sizeof(float)),
+        hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_masked_kernel<bf16>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                            kMaskedWaves * kMaskedMaxKey * (int)sizeof(float))};
+    PA_REQUIRE(allowed[0] == hipSuccess && allowed[1] == hipSuccess, "attn_masked: %zu bytes of LDS refused", lds);
+  }
   if (dtype == kF32) {
-    hipLaunchKernelGGL(attn_masked_kernel<float>, grid, dim3(kMaskedWaves * kWave), 0, st, (const float*)q,
+    hipLaunchKernelGGL(attn_masked_kernel<float>, grid, dim3(kMaskedWaves * kWave), lds, st, (const float*)q,
                        (const float*)k_cache, (const float*)v_cache, block_table, table_stride, seq_of_token, positions,
                        (float*)out, (size_t)out_stride, nh, nkv, hd, vd, page_size, window, keep_first, scale, softcap, slopes,
                        sink, (const float*)gate, (size_t)gate_stride, out_scale, nv);
   } else if (dtype == kBF16) {
-    hipLaunchKernelGGL(attn_masked_kernel<bf16>, grid, dim3(kMaskedWaves * kWave), 0, st, (const bf16*)q,
+    hipLaunchKernelGGL(attn_masked_kernel<bf16>, grid, dim3(kMaskedWaves * kWave), lds, st, (const bf16*)q,
                        (const bf16*)k_cache, (const bf16*)v_cache, block_table, table_stride, seq_of_token, positions,
                        (bf16*)out, (size_t)out_stride, nh, nkv, hd, vd, page_size, window, keep_first, scale, softcap, slopes,
                        sink, (const bf16*)gate, (size_t)gate_stride, out_scale, nv);

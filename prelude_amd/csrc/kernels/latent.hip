@@ -5,7 +5,7 @@
 // itself, the weighted sum of cached latents (rank elements a head) is taken through the value map afterwards.
 // All heads read the same keys: one "KV head" of width rank + rot whose value is its own first `rank` elements.
 //
-//   pa_latent_prep    the merged down projection's row [q_rank | rank | rot]: RMS norm of the query latent (out),
+//   pa_latent_prep    the merged down projection's row [q_rank | rank | rot]: RMS norm of the query latent (out; q_rank 0: none),
 //                     RMS norm of c and rotation of the shared key part (into the paged cache; c a second time
 //                     transposed, where the cache keeps that copy for the matrix-core kernel)
 //   pa_rotate_pairs   rotation of a part of every head's vector by position, pairs (2i, 2i+1)
@@ -96,11 +96,11 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const T* __restrict__ 
 }
 
 // ---- rotation of a part of every head ---------------------------------------
-// in [T, heads, in_stride] -> out [T, heads, out_stride]: elements in_off .. in_off + width of a head go to
+// in [T, heads, in_stride] (tokens in_token apart) -> out [T, heads, out_stride]: elements in_off .. in_off + width of a head go to
 // out_off .., the first rot_dims of them rotated in pairs.
 template <typename T>
 __global__ void rotate_pairs_kernel(const T* __restrict__ in, T* __restrict__ out, const float* __restrict__ inv_freq,
-                                    const int* __restrict__ positions, int heads, int in_stride, int in_off,
+                                    const int* __restrict__ positions, int heads, long in_token, int in_stride, int in_off,
                                     int out_stride, int out_off, int width, int rot_dims) {
   const int t = blockIdx.x;
   const float p = (float)positions[t];
@@ -108,7 +108,7 @@ __global__ void rotate_pairs_kernel(const T* __restrict__ in, T* __restrict__ ou
   const int per_head = half + (width - rot_dims);
   for (int e = threadIdx.x; e < heads * per_head; e += blockDim.x) {
     const int h = e / per_head, i = e % per_head;
-    const T* src = in + ((size_t)t * heads + h) * in_stride + in_off;
+    const T* src = in + (size_t)t * in_token + (size_t)h * in_stride + in_off;
     T* dst = out + ((size_t)t * heads + h) * out_stride + out_off;
     if (i < half) {
       float s, c;
@@ -280,7 +280,7 @@ extern "C" int pa_latent_prep(void* stream, int dtype, const void* in, const flo
   if (tokens == 0) return 0;
   if (in_stride <= 0) in_stride = q_rank + rank + rot;
   PA_REQUIRE(in_stride >= q_rank + rank + rot, "latent_prep: a row stride of %ld is less than the row", in_stride);
-  PA_REQUIRE(tokens > 0 && q_rank > 0 && rank > 0 && rot >= 0, "latent_prep: bad sizes tokens=%d q_rank=%d rank=%d rot=%d",
+  PA_REQUIRE(tokens > 0 && q_rank >= 0 && (q_rank > 0 || !cq_out) && rank > 0 && rot >= 0, "latent_prep: bad sizes tokens=%d q_rank=%d rank=%d rot=%d",
              tokens, q_rank, rank, rot);
   PA_REQUIRE(rot_dims >= 0 && rot_dims <= rot && rot_dims % 2 == 0, "latent_prep: %d rotated of %d is not an even part", rot_dims, rot);
   PA_REQUIRE(!slots || cache, "latent_prep: slots without a cache");
@@ -306,15 +306,17 @@ extern "C" int pa_latent_gather(void* stream, int dtype, const void* cache, cons
 
 extern "C" int pa_rotate_pairs(void* stream, int dtype, const void* in, void* out, const float* inv_freq,
                                const int* positions, int tokens, int heads, int in_stride, int in_off, int out_stride,
-                               int out_off, int width, int rot_dims) {
+                               int out_off, int width, int rot_dims, long in_token) {
+  if (in_token <= 0) in_token = (long)heads * in_stride;
   if (tokens == 0 || width == 0) return 0;
   PA_REQUIRE(tokens > 0 && heads > 0 && width > 0 && rot_dims >= 0 && rot_dims <= width && rot_dims % 2 == 0,
              "rotate_pairs: bad sizes tokens=%d heads=%d width=%d rotated=%d", tokens, heads, width, rot_dims);
+  PA_REQUIRE(in_token >= (long)heads * in_stride, "rotate_pairs: tokens %ld apart overlap", in_token);
   PA_REQUIRE(in_off >= 0 && out_off >= 0 && in_off + width <= in_stride && out_off + width <= out_stride,
              "rotate_pairs: a part of %d at %d / %d does not fit heads of %d / %d", width, in_off, out_off, in_stride, out_stride);
   PA_BY_TYPE(dtype, "rotate_pairs",
              hipLaunchKernelGGL(rotate_pairs_kernel<T>, dim3(tokens), dim3(256), 0, (hipStream_t)stream, (const T*)in, (T*)out,
-                                inv_freq, positions, heads, in_stride, in_off, out_stride, out_off, width, rot_dims));
+                                inv_freq, positions, heads, in_token, in_stride, in_off, out_stride, out_off, width, rot_dims));
   return check_launch("rotate_pairs");
 }
 

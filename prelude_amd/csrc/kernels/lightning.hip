@@ -25,6 +25,15 @@
 // over the chunks of a sequence in order turns the U into the S_b and leaves the final state in the slot, (3) every
 // chunk adds the second term.  All three keep to 32-bit and to non-negative powers of a.  Sequences of at most one
 // chunk are left to pa_lightning_attn.
+//
+// pa_gla_*: gated linear attention, the same recurrence with a decay per token, head and key channel,
+//
+//   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,   o_t = q_scale S_t^T q_t,   alpha = sigmoid(A2 low + bias)^(1 / tau)
+//
+// `low` [rank] a token inside the merged projection.  pa_gla_decay makes alpha [tokens, heads, dim] in 32-bit for
+// the portions; pa_gla_step (single tokens) makes its own on the way in.  The chunked form multiplies the state on from
+// token to token in its third pass (S_b decayed, nothing added), so only products of decays appear, never quotients:
+// any decay from 0 to 1 is exact to rounding.
 #include "common.h"
 #include "api.h"
 
@@ -59,12 +68,14 @@ __device__ __forceinline__ size_t la_chunk_index(int row0, int chunk, int z, int
 // `min_len` are left alone.
 // kLaLocal / kLaApply: grid (column tiles, heads, listed sequences x max_chunks); sequences of at most one chunk and
 // chunks past a sequence's end leave at once.
-template <typename T, int R, int NC, int MODE>
+// VEC: `decay` is [tokens, heads, dim], one a token and key channel, queries are multiplied by q_scale on their way in,
+// and kLaLocal leaves every chunk's product of decays in chunk_decay [chunk, heads, dim].
+template <typename T, int R, int NC, int MODE, bool VEC>
 __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
     const T* __restrict__ qkv, long ld, int q_off, int k_off, int v_off, const float* __restrict__ decay,
     float* __restrict__ state, const int* __restrict__ state_slots, const int* __restrict__ cu_q,
     const int* __restrict__ seq_ids, float* __restrict__ out, float* __restrict__ work, int heads, int dim, int vdim, int act,
-    int max_len, int chunk, int max_chunks, int min_len) {
+    int max_len, int chunk, int max_chunks, int min_len, float q_scale, float* __restrict__ chunk_decay) {
   constexpr int kCols = kLaLanes * NC;
   // a quarter's rows lie R + 4 floats apart: the four 16-byte reads of a wavefront (one a quarter) then fall into
   // different banks (R is a multiple of 8, so R floats apart they would all fall into the same four)
@@ -73,6 +84,7 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
   __shared__ __align__(16) float ks[MODE == kLaApply ? 1 : kLaTokens][4 * kQuarter];
   __shared__ float vs[MODE == kLaApply ? 1 : kLaTokens][kCols];
   __shared__ float pw[MODE == kLaApply ? kLaMaxChunk : 1];
+  __shared__ __align__(16) float as[VEC ? kLaTokens : 1][4 * kQuarter];
   const int w = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int dp = lane / 16;                      // which quarter of the rows
   const int cl = 16 * w + lane % 16;             // column within a run of 64
@@ -97,10 +109,11 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
     row0 += j * chunk;
     row1 = row1 < row0 + chunk ? row1 : row0 + chunk;
   }
-  const float a = decay[h];
-  if (MODE == kLaApply) {
+  const float a = VEC ? 1.f : decay[h];
+  if (MODE == kLaApply && !VEC) {
     for (int i = threadIdx.x; i < chunk; i += kLaThreads) pw[i] = powf(a, (float)(i + 1));
   }
+  float total = 1.f;   // VEC, kLaLocal: the chunk's product of decays of channel threadIdx.x
   int col[NC];
   bool live[NC];
   float S[NC][R];
@@ -128,7 +141,19 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
   constexpr int kPerToken = (MODE == kLaApply ? 4 * R : 8 * R + kCols);
   constexpr int kRaw = (kLaTokens * kPerToken + kLaThreads - 1) / kLaThreads;
   T raw[kRaw];
+  constexpr int kRawDecay = VEC ? (kLaTokens * 4 * R + kLaThreads - 1) / kLaThreads : 1;
+  float raw_decay[kRawDecay];
   auto fetch = [&](int t0) {
+    if (VEC) {
+#pragma unroll
+      for (int i = 0; i < kRawDecay; ++i) {
+        const int e = threadIdx.x + kLaThreads * i;
+        const int t = e / (4 * R), d = e % (4 * R);
+        const int tt = t0 + t < row1 ? t0 + t : row1 - 1;
+        const float v = decay[((size_t)tt * heads + h) * dim + (d < dim ? d : dim - 1)];
+        raw_decay[i] = (t0 + t < row1 && d < dim) ? v : 1.f;
+      }
+    }
 #pragma unroll
     for (int i = 0; i < kRaw; ++i) {
       const int e = threadIdx.x + kLaThreads * i;
@@ -146,6 +171,14 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
     }
   };
   auto stage = [&]() {
+    if (VEC) {
+#pragma unroll
+      for (int i = 0; i < kRawDecay; ++i) {
+        const int e = threadIdx.x + kLaThreads * i;
+        const int t = e / (4 * R), d = e % (4 * R);
+        if (t < kLaTokens) as[t][(d / R) * kQuarter + d % R] = raw_decay[i];
+      }
+    }
 #pragma unroll
     for (int i = 0; i < kRaw; ++i) {
       const int e = threadIdx.x + kLaThreads * i;
@@ -153,7 +186,7 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
       if (t >= kLaTokens) continue;
       const float v = la_act(to_f32(raw[i]), act);
       if (x < 4 * R) {
-        qs[t][(x / R) * kQuarter + x % R] = v;
+        qs[t][(x / R) * kQuarter + x % R] = VEC ? v * q_scale : v;
       } else if (MODE != kLaApply) {
         if (x < 8 * R) ks[t][((x - 4 * R) / R) * kQuarter + (x - 4 * R) % R] = v;
         else vs[t][x - 8 * R] = v;
@@ -167,6 +200,9 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
     stage();
     __syncthreads();
     if (t0 + kLaTokens < row1) fetch(t0 + kLaTokens);
+    if (VEC && MODE == kLaLocal && blockIdx.x == 0 && (int)threadIdx.x < dim) {
+      for (int t = 0; t < n; ++t) total *= as[t][(threadIdx.x / R) * kQuarter + threadIdx.x % R];
+    }
     // The block's tokens in groups whose results leave together.  The third pass adds to what the stream holds: it
     // asks for a whole block's places before the walk (its state is fixed, so it has the registers); the passes
     // that carry the state along take four tokens at a time, which keeps two wavefronts on a SIMD.
@@ -197,11 +233,14 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
             const f32x4 q4 = *reinterpret_cast<const f32x4*>(&qs[t][dp * kQuarter + r]);
             f32x4 k4 = f32x4{0.f, 0.f, 0.f, 0.f};
             if (MODE != kLaApply) k4 = *reinterpret_cast<const f32x4*>(&ks[t][dp * kQuarter + r]);
+            f32x4 a4 = f32x4{a, a, a, a};
+            if (VEC) a4 = *reinterpret_cast<const f32x4*>(&as[t][dp * kQuarter + r]);
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
 #pragma unroll
               for (int c = 0; c < NC; ++c) {
-                if (MODE != kLaApply) S[c][r + e] = fmaf(a, S[c][r + e], k4[e] * v[c]);
+                if (MODE != kLaApply) S[c][r + e] = fmaf(a4[e], S[c][r + e], k4[e] * v[c]);
+                else if (VEC) S[c][r + e] *= a4[e];
                 acc[c] = fmaf(S[c][r + e], q4[e], acc[c]);
               }
             }
@@ -209,7 +248,7 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
 #pragma unroll
           for (int c = 0; c < NC; ++c) {
             const float sum = la_sum_rows(acc[c]);
-            res[u][c] = MODE == kLaApply ? res[u][c] + pw[t0 + t - row0] * sum : sum;
+            res[u][c] = MODE == kLaApply ? res[u][c] + (VEC ? sum : pw[t0 + t - row0] * sum) : sum;
           }
         }
       }
@@ -222,6 +261,8 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
       }
     }
   }
+  if (VEC && MODE == kLaLocal && blockIdx.x == 0 && (int)threadIdx.x < dim)
+    chunk_decay[(la_chunk_index(cu_q[seq], chunk, z, j) * heads + h) * dim + threadIdx.x] = total;
   if (MODE != kLaApply) {
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
@@ -234,17 +275,52 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
   }
 }
 
+// alpha = sigmoid(z)^(1 / tau), z = w . low + bias: log sigmoid(z) = min(z, 0) - log(1 + e^-|z|), which loses nothing at either end.
+__device__ __forceinline__ float gla_alpha(float z, float inv_tau) {
+  return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);
+}
+// One channel's row of A2 against a token's low-rank vector in LDS, in ascending order.
+template <typename T>
+__device__ __forceinline__ float gla_dot(const T* __restrict__ w, const float* low, int rank) {
+  float acc = 0.f;
+  if (sizeof(T) == 2 && rank % 8 == 0) {
+    for (int i = 0; i < rank; i += 8) {
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(w + i);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc = fmaf((float)v[e], low[i + e], acc);
+    }
+  } else {
+    for (int i = 0; i < rank; ++i) acc = fmaf(to_f32(w[i]), low[i], acc);
+  }
+  return acc;
+}
+
+// alpha [tokens, channels].  Grid (tokens, runs of 256 channels); LDS: the token's low-rank vector.
+template <typename T>
+__global__ __launch_bounds__(256) void gla_decay_kernel(const T* __restrict__ p, long ld, int low_off, const T* __restrict__ a2,
+                                                        const float* __restrict__ bias, float* __restrict__ alpha, int channels,
+                                                        int rank, float inv_tau) {
+  extern __shared__ float low[];
+  const size_t t = blockIdx.x;
+  for (int i = threadIdx.x; i < rank; i += 256) low[i] = to_f32(p[t * ld + low_off + i]);
+  __syncthreads();
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c < channels) alpha[t * channels + c] = gla_alpha(gla_dot(a2 + (size_t)c * rank, low, rank) + bias[c], inv_tau);
+}
+
 // Sequences of exactly one token (a decode step): the same sums as the kernel above gives for them, bit for bit, in a
 // kernel small enough that a step's many launches do not wait for its code.  Grid (tiles of 64 columns, heads,
 // sequences); a wavefront owns a quarter of the rows (the quarters of the kernel above), a lane a column: a row's 64
 // columns are one run of memory.  All of a lane's rows of S are asked for at once, updated and stored; the quarters'
 // dot products meet in LDS and are added (0 + 1) + (2 + 3).
-template <typename T, int R>
+// VEC: the decays are gla_alpha of the token's low-rank vector (`decay` is the bias there).
+template <typename T, int R, bool VEC>
 __global__ __launch_bounds__(kLaThreads) void lightning_step_kernel(
     const T* __restrict__ qkv, long ld, int q_off, int k_off, int v_off, const float* __restrict__ decay,
     float* __restrict__ state, const int* __restrict__ state_slots, const int* __restrict__ cu_q, float* __restrict__ out,
-    int heads, int dim, int vdim, int act) {
-  __shared__ float qs[4 * R], ks[4 * R];
+    int heads, int dim, int vdim, int act, float q_scale, int low_off, const T* __restrict__ a2, int rank, float inv_tau) {
+  extern __shared__ float low[];   // VEC: the token's low-rank vector
+  __shared__ float qs[4 * R], ks[4 * R], as[VEC ? 4 * R : 1];
   __shared__ float part[4][kLaLanes];
   const int w = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int h = blockIdx.y, seq = blockIdx.z;
@@ -263,17 +339,26 @@ __global__ __launch_bounds__(kLaThreads) void lightning_step_kernel(
   const T* src = qkv + (size_t)row * ld;
   if ((int)threadIdx.x < 4 * R) {
     const int d = (int)threadIdx.x < dim ? threadIdx.x : dim - 1;
-    qs[threadIdx.x] = la_act(to_f32(src[q_off + (size_t)h * dim + d]), act);
+    const float qv = la_act(to_f32(src[q_off + (size_t)h * dim + d]), act);
+    qs[threadIdx.x] = VEC ? qv * q_scale : qv;
     ks[threadIdx.x] = la_act(to_f32(src[k_off + (size_t)h * dim + d]), act);
   }
   const float v = la_act(to_f32(src[v_off + (size_t)h * vdim + (live ? col : vdim - 1)]), act);
-  const float a = decay[h];
+  const float a = VEC ? 1.f : decay[h];
+  if (VEC) {
+    for (int i = threadIdx.x; i < rank; i += kLaThreads) low[i] = to_f32(src[low_off + i]);
+    __syncthreads();
+    if ((int)threadIdx.x < 4 * R) {
+      const int c = h * dim + ((int)threadIdx.x < dim ? (int)threadIdx.x : dim - 1);
+      as[threadIdx.x] = gla_alpha(gla_dot(a2 + (size_t)c * rank, low, rank) + decay[c], inv_tau);
+    }
+  }
   __syncthreads();
   float acc = 0.f;
 #pragma unroll
   for (int r = 0; r < R; ++r) {
     const int d = w * R + r;
-    s[r] = fmaf(a, s[r], ks[d] * v);
+    s[r] = fmaf(VEC ? as[d] : a, s[r], ks[d] * v);
     if (d < dim) acc = fmaf(s[r], qs[d], acc);
   }
 #pragma unroll
@@ -287,11 +372,13 @@ __global__ __launch_bounds__(kLaThreads) void lightning_step_kernel(
 }
 
 // The chunks of one listed sequence in order: work[chunk] holds U coming in and the state before the chunk going
-// out; the state slot gives the start and receives the end.  A thread an element of a head's state.
+// out; the state slot gives the start and receives the end.  A thread an element of a head's state.  VEC: `decay` holds
+// every chunk's product of decays, [chunk, heads, dim].
+template <bool VEC>
 __global__ __launch_bounds__(256) void lightning_scan_kernel(const float* __restrict__ decay, float* __restrict__ state,
                                                             const int* __restrict__ state_slots, const int* __restrict__ cu_q,
                                                             const int* __restrict__ seq_ids, float* __restrict__ work,
-                                                            int heads, int per_head, int chunk) {
+                                                            int heads, int per_head, int chunk, int vdim) {
   const int z = blockIdx.z, h = blockIdx.y;
   const int seq = seq_ids[z];
   const int row0 = cu_q[seq], len = cu_q[seq + 1] - row0;
@@ -299,8 +386,9 @@ __global__ __launch_bounds__(256) void lightning_scan_kernel(const float* __rest
   if (slot < 0 || len <= chunk) return;
   const int e = blockIdx.x * 256 + threadIdx.x;
   if (e >= per_head) return;
-  const float a = decay[h];
-  const float a_chunk = powf(a, (float)chunk);
+  const float a = VEC ? 1.f : decay[h];
+  const float a_chunk = VEC ? 1.f : powf(a, (float)chunk);
+  const int dim = per_head / vdim;
   float* sp = state + ((size_t)slot * heads + h) * per_head + e;
   float S = *sp;
   const int chunks = (len + chunk - 1) / chunk;
@@ -309,16 +397,17 @@ __global__ __launch_bounds__(256) void lightning_scan_kernel(const float* __rest
     const float U = *wp;
     *wp = S;
     const int n = len - j * chunk;
-    S = fmaf(n >= chunk ? a_chunk : powf(a, (float)n), S, U);
+    if (VEC) S = fmaf(decay[(la_chunk_index(row0, chunk, z, j) * heads + h) * dim + e / vdim], S, U);
+    else S = fmaf(n >= chunk ? a_chunk : powf(a, (float)n), S, U);
   }
   *sp = S;
 }
 
-template <typename T, int MODE>
+template <typename T, int MODE, bool VEC = false>
 static void launch_lightning(hipStream_t st, int zdim, const T* qkv, long ld, int q_off, int k_off, int v_off,
                              const float* decay, float* state, const int* state_slots, const int* cu_q, const int* seq_ids,
                              float* out, float* work, int heads, int dim, int vdim, int act, int max_len, int chunk,
-                             int max_chunks, int min_len = 0) {
+                             int max_chunks, int min_len = 0, float q_scale = 1.f, float* chunk_decay = nullptr) {
   // two columns a lane where the state is wide enough and its rows leave the registers for them
   // ... and there are workgroups enough without halving the columns of each (a step of few single tokens wants the
   // workgroups)
@@ -326,8 +415,9 @@ static void launch_lightning(hipStream_t st, int zdim, const T* qkv, long ld, in
   const int cols = two ? 2 * kLaLanes : kLaLanes;
   dim3 grid((vdim + cols - 1) / cols, heads, zdim);
 #define PA_LA(R, NC)                                                                                                       \
-  hipLaunchKernelGGL((lightning_attn_kernel<T, R, NC, MODE>), grid, dim3(kLaThreads), 0, st, qkv, ld, q_off, k_off, v_off, \
-                     decay, state, state_slots, cu_q, seq_ids, out, work, heads, dim, vdim, act, max_len, chunk, max_chunks, min_len)
+  hipLaunchKernelGGL((lightning_attn_kernel<T, R, NC, MODE, VEC>), grid, dim3(kLaThreads), 0, st, qkv, ld, q_off, k_off, v_off, \
+                     decay, state, state_slots, cu_q, seq_ids, out, work, heads, dim, vdim, act, max_len, chunk, max_chunks, min_len, \
+                     q_scale, chunk_decay)
   if (dim <= 32) { if (two) PA_LA(8, 2); else PA_LA(8, 1); }
   else if (dim <= 64) { if (two) PA_LA(16, 2); else PA_LA(16, 1); }
   else if (dim <= 128) { if (two) PA_LA(32, 2); else PA_LA(32, 1); }
@@ -380,8 +470,8 @@ extern "C" int pa_lightning_step(void* stream, int dtype, const void* qkv, long 
   hipStream_t st = (hipStream_t)stream;
   dim3 grid((vdim + kLaLanes - 1) / kLaLanes, heads, nseq);
 #define PA_LS(T, R)                                                                                                       \
-  hipLaunchKernelGGL((lightning_step_kernel<T, R>), grid, dim3(kLaThreads), 0, st, (const T*)qkv, ld, q_off, k_off, v_off, \
-                     decay, state, state_slots, cu_q, out, heads, dim, vdim, act)
+  hipLaunchKernelGGL((lightning_step_kernel<T, R, false>), grid, dim3(kLaThreads), 0, st, (const T*)qkv, ld, q_off, k_off,  \
+                     v_off, decay, state, state_slots, cu_q, out, heads, dim, vdim, act, 1.f, 0, (const T*)nullptr, 0, 1.f)
 #define PA_LS_R(T)                    \
   do {                                \
     if (dim <= 32) PA_LS(T, 8);       \
@@ -425,8 +515,8 @@ extern "C" int pa_lightning_attn_chunked(void* stream, int dtype, const void* qk
   launch_lightning<T, MODE>(st, nlisted * max_chunks, (const T*)qkv, ld, q_off, k_off, v_off, decay, state, state_slots, cu_q, seq_ids, out, \
                             work, heads, dim, vdim, act, 0, chunk, max_chunks)
 #define PA_LA_SCAN()                                                                                                      \
-  hipLaunchKernelGGL(lightning_scan_kernel, scan_grid, dim3(256), 0, st, decay, state, state_slots, cu_q, seq_ids, work,   \
-                     heads, per_head, chunk)
+  hipLaunchKernelGGL(lightning_scan_kernel<false>, scan_grid, dim3(256), 0, st, decay, state, state_slots, cu_q, seq_ids, work,   \
+                     heads, per_head, chunk, vdim)
   if (dtype == kF32) {
     PA_LA_PASS(float, kLaLocal);
     PA_LA_SCAN();
@@ -441,4 +531,119 @@ extern "C" int pa_lightning_attn_chunked(void* stream, int dtype, const void* qk
 #undef PA_LA_PASS
 #undef PA_LA_SCAN
   return check_launch("lightning_attn_chunked");
+}
+
+// ---- gated linear attention ------------------------------------------------------------------------------------------
+static int gla_low_check(const char* what, long ld, int low_off, int rank) {
+  PA_REQUIRE(rank > 0 && rank <= 8192 && low_off >= 0 && low_off + (long)rank <= ld, "%s: a low-rank vector of %d at column %d of a row of %ld",
+             what, rank, low_off, ld);
+  return 0;
+}
+
+extern "C" int pa_gla_decay(void* stream, int dtype, const void* p, long ld, int low_off, const void* a2, const float* bias,
+                            float* alpha, int tokens, int channels, int rank, float tau) {
+  if (tokens == 0) return 0;
+  PA_REQUIRE(tokens > 0 && channels > 0 && tau > 0.f && (channels + 255) / 256 <= 65535, "gla_decay: bad sizes tokens=%d channels=%d tau=%g",
+             tokens, channels, (double)tau);
+  if (int rc = gla_low_check("gla_decay", ld, low_off, rank)) return rc;
+  dim3 grid(tokens, (channels + 255) / 256);
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == kF32)
+    hipLaunchKernelGGL(gla_decay_kernel<float>, grid, dim3(256), rank * sizeof(float), st, (const float*)p, ld, low_off,
+                       (const float*)a2, bias, alpha, channels, rank, 1.f / tau);
+  else if (dtype == kBF16)
+    hipLaunchKernelGGL(gla_decay_kernel<bf16>, grid, dim3(256), rank * sizeof(float), st, (const bf16*)p, ld, low_off,
+                       (const bf16*)a2, bias, alpha, channels, rank, 1.f / tau);
+  else
+    return pa::fail("gla_decay: unknown element type code %d", dtype);
+  return check_launch("gla_decay");
+}
+
+// Sequences of max_len tokens at most (max_len > 0) and min_len at least, token by token.
+extern "C" int pa_gla_attn(void* stream, int dtype, const void* qkv, long ld, int q_off, int k_off, int v_off, const float* alpha,
+                           float* state, const int* state_slots, const int* cu_q, float* out, int nseq, int tokens, int heads,
+                           int dim, int vdim, float q_scale, int max_len, int min_len) {
+  if (nseq == 0 || tokens == 0) return 0;
+  if (int rc = lightning_check("gla_attn", nseq, tokens, heads, dim, vdim, ld, q_off, k_off, v_off, 0)) return rc;
+  PA_REQUIRE(nseq <= 65535, "gla_attn: %d sequences exceed the grid", nseq);
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == kF32)
+    launch_lightning<float, kLaWhole, true>(st, nseq, (const float*)qkv, ld, q_off, k_off, v_off, alpha, state, state_slots, cu_q,
+                                            nullptr, out, nullptr, heads, dim, vdim, 0, max_len, 0, 1, min_len, q_scale);
+  else if (dtype == kBF16)
+    launch_lightning<bf16, kLaWhole, true>(st, nseq, (const bf16*)qkv, ld, q_off, k_off, v_off, alpha, state, state_slots, cu_q,
+                                           nullptr, out, nullptr, heads, dim, vdim, 0, max_len, 0, 1, min_len, q_scale);
+  else
+    return pa::fail("gla_attn: unknown element type code %d", dtype);
+  return check_launch("gla_attn");
+}
+
+extern "C" int pa_gla_step(void* stream, int dtype, const void* qkv, long ld, int q_off, int k_off, int v_off, int low_off,
+                           const void* a2, const float* bias, float* state, const int* state_slots, const int* cu_q, float* out,
+                           int nseq, int heads, int dim, int vdim, int rank, float tau, float q_scale) {
+  if (nseq == 0) return 0;
+  if (int rc = lightning_check("gla_step", nseq, nseq, heads, dim, vdim, ld, q_off, k_off, v_off, 0)) return rc;
+  if (int rc = gla_low_check("gla_step", ld, low_off, rank)) return rc;
+  PA_REQUIRE(nseq <= 65535 && tau > 0.f, "gla_step: %d sequences or tau %g", nseq, (double)tau);
+  hipStream_t st = (hipStream_t)stream;
+  dim3 grid((vdim + kLaLanes - 1) / kLaLanes, heads, nseq);
+#define PA_GS(T, R)                                                                                                          \
+  hipLaunchKernelGGL((lightning_step_kernel<T, R, true>), grid, dim3(kLaThreads), rank * sizeof(float), st, (const T*)qkv, ld, \
+                     q_off, k_off, v_off, bias, state, state_slots, cu_q, out, heads, dim, vdim, 0, q_scale, low_off,          \
+                     (const T*)a2, rank, 1.f / tau)
+#define PA_GS_R(T)                    \
+  do {                                \
+    if (dim <= 32) PA_GS(T, 8);       \
+    else if (dim <= 64) PA_GS(T, 16); \
+    else if (dim <= 128) PA_GS(T, 32); \
+    else PA_GS(T, 64);                \
+  } while (0)
+  if (dtype == kF32)
+    PA_GS_R(float);
+  else if (dtype == kBF16)
+    PA_GS_R(bf16);
+  else
+    return pa::fail("gla_step: unknown element type code %d", dtype);
+#undef PA_GS_R
+#undef PA_GS
+  return check_launch("gla_step");
+}
+
+// 32-bit words of workspace: the chunks' states, then their products of decays
+extern "C" long pa_gla_chunked_workspace(int nlisted, int tokens, int heads, int dim, int vdim, int chunk) {
+  if (chunk <= 0) return 0;
+  return ((long)tokens / chunk + nlisted) * heads * dim * (vdim + 1L);
+}
+
+extern "C" int pa_gla_attn_chunked(void* stream, int dtype, const void* qkv, long ld, int q_off, int k_off, int v_off,
+                                   const float* alpha, float* state, const int* state_slots, const int* cu_q, const int* seq_ids,
+                                   float* out, float* work, int nlisted, int tokens, int max_len, int heads, int dim, int vdim,
+                                   float q_scale, int chunk) {
+  if (nlisted == 0 || tokens == 0 || max_len <= chunk) return 0;
+  if (int rc = lightning_check("gla_attn_chunked", nlisted, tokens, heads, dim, vdim, ld, q_off, k_off, v_off, 0)) return rc;
+  PA_REQUIRE(chunk >= kLaTokens && chunk % kLaTokens == 0 && chunk <= kLaMaxChunk,
+             "gla_attn_chunked: chunks of %d tokens are not a multiple of %d up to %d", chunk, kLaTokens, kLaMaxChunk);
+  PA_REQUIRE(seq_ids && work, "gla_attn_chunked: no list of sequences or no workspace");
+  const int max_chunks = (max_len + chunk - 1) / chunk;
+  PA_REQUIRE((long)nlisted * max_chunks <= 65535, "gla_attn_chunked: %d sequences x %d chunks exceed the grid", nlisted, max_chunks);
+  hipStream_t st = (hipStream_t)stream;
+  const int per_head = dim * vdim;
+  float* chunk_decay = work + ((long)tokens / chunk + nlisted) * heads * (long)per_head;
+  dim3 scan_grid((per_head + 255) / 256, heads, nlisted);
+#define PA_GLA_PASS(T, MODE)                                                                                                  \
+  launch_lightning<T, MODE, true>(st, nlisted * max_chunks, (const T*)qkv, ld, q_off, k_off, v_off, alpha, state, state_slots,  \
+                                  cu_q, seq_ids, out, work, heads, dim, vdim, 0, 0, chunk, max_chunks, 0, q_scale, chunk_decay)
+#define PA_GLA(T)                                                                                                             \
+  do {                                                                                                                        \
+    PA_GLA_PASS(T, kLaLocal);                                                                                                 \
+    hipLaunchKernelGGL(lightning_scan_kernel<true>, scan_grid, dim3(256), 0, st, chunk_decay, state, state_slots, cu_q, seq_ids, \
+                       work, heads, per_head, chunk, vdim);                                                                   \
+    PA_GLA_PASS(T, kLaApply);                                                                                                 \
+  } while (0)
+  if (dtype == kF32) PA_GLA(float);
+  else if (dtype == kBF16) PA_GLA(bf16);
+  else return pa::fail("gla_attn_chunked: unknown element type code %d", dtype);
+#undef PA_GLA
+#undef PA_GLA_PASS
+  return check_launch("gla_attn_chunked");
 }

@@ -70,6 +70,7 @@ class CausalLM:
             self.embedding_cache = len(self.cache_slots)
             self.cache_slots.append(CacheSlot(-1, ecs))
         self.stream_rows: Optional[torch.Tensor] = None
+        self._adds_embedding = any(r.add_embedding for r in spec.order)
         for i, r in enumerate(spec.order):
             mixer = getattr(self.blocks[r.layer], "mixer", None)
             cs = mixer.cache_spec() if mixer is not None else None
@@ -143,7 +144,7 @@ class CausalLM:
         """Kernel launches of one step, about: every run's block by its parts' own counts, and the embedding, the
         final norm and the head."""
         total = self.embedding.LAUNCHES + self.final_norm.LAUNCHES + self.head.LAUNCHES
-        total += sum(1 for r in self.spec.order if r.stream_row is not None)
+        total += sum(1 for r in self.spec.order if r.stream_row is not None or r.add_embedding)
         for r in self.spec.order:
             b = self.blocks[r.layer]
             total += b.launches() if hasattr(b, "launches") else 1
@@ -171,17 +172,25 @@ class CausalLM:
         return any(getattr(p, "ATOMIC_PREFILL", False) for p, _ in self._parts)
 
     # ---- forward ------------------------------------------------------------
-    def _add_stream_row(self, hidden, residual, row: int):
-        """Adds row ``row`` of the model's stream rows to the stream, in 32-bit and in place.  The stream is what a block
-        that hands it on left (``hidden`` None, a 32-bit residual), or, in front of the first run, the embedding."""
+    def _add_to_stream(self, hidden, residual, row: Optional[int], embedded=None):
+        """Adds the embedding's output ``embedded`` (or nothing) and row ``row`` of the model's stream rows (None: nothing) to
+        the stream, in 32-bit.  The stream is what a block that hands it on left (``hidden`` None, a 32-bit residual, changed
+        in place), or what waits and the residual it waits for (added as well), or, in front of the first run, the
+        embedding (left as it is where a later run adds it again)."""
         from ..ops import kernels as K
+        vec = None if row is None else self.stream_rows[row]
         if residual is None:
             hidden = K.as_tensor(hidden)
             stream = hidden if hidden.dtype == torch.float32 else K.to_f32(hidden)
-            return K.stream_add_row_(stream, self.stream_rows[row]), None
-        if hidden is not None or residual.dtype != torch.float32:
-            raise PartError("a row is added to a 32-bit stream that travels alone between blocks")
-        K.stream_add_row_(residual, self.stream_rows[row])
+            if self._adds_embedding:
+                return None, K.stream_sum(stream, extra=embedded, row=vec)
+            return K.stream_add_row_(stream, vec), None
+        if residual.dtype != torch.float32:
+            raise PartError("rows and embeddings are added to a 32-bit stream")
+        if hidden is None and embedded is None:
+            K.stream_add_row_(residual, vec)
+        else:
+            K.stream_sum(residual, None if hidden is None else K.as_tensor(hidden), embedded, vec, out=residual)
         return None, residual
 
     def forward(self, step, caches) -> torch.Tensor:
@@ -194,11 +203,17 @@ class CausalLM:
                                             cache=None if self.embedding_cache is None else caches[self.embedding_cache])
         else:
             hidden = self.embedding.forward(step.token_ids)
-        residual = None
+        residual = embedded = None
         step.compute_dtype = self.dtype
+        if self._adds_embedding:
+            from ..ops import kernels as K
+            embedded = hidden = K.to_f32(K.as_tensor(hidden))
+            first = self.spec.order[0]
+            if first.stream_row is None and not first.add_embedding:
+                hidden, residual = None, K.stream_sum(embedded)   # the stream changes in place, the embedding stays
         for i, r in enumerate(self.spec.order):
-            if r.stream_row is not None:
-                hidden, residual = self._add_stream_row(hidden, residual, r.stream_row)
+            if r.stream_row is not None or r.add_embedding:
+                hidden, residual = self._add_to_stream(hidden, residual, r.stream_row, embedded if r.add_embedding else None)
             ci = self.run_cache[i]
             cache = None if ci is None else (tuple(caches[c] for c in ci) if isinstance(ci, tuple) else caches[ci])
             hidden, residual = self.blocks[r.layer].forward(hidden, residual, step, cache,

@@ -34,10 +34,13 @@ class RunSpec:
     run (by its index in ``order``) whose cache it reads without writing.
     ``stream_row``: row of the model's ``stream_rows`` tensor that is added to the stream right in front of this run
     (a learned vector per pass of a stretch of layers that runs several times, say); None: nothing.
+    ``add_embedding``: the embedding's output (the stream as it was in front of the first run) is added to the stream right
+    in front of this run, before the row.
     """
     layer: int
     reads_cache_of: Optional[int] = None
     stream_row: Optional[int] = None
+    add_embedding: bool = False
 
 
 @dataclasses.dataclass

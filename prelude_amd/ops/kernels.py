@@ -1240,10 +1240,11 @@ def relu_squared(x: torch.Tensor) -> torch.Tensor:
 
 # ---------------------------------------------------------------------------
 # Attention through a latent
-def latent_prep(down: torch.Tensor, q_weight: torch.Tensor, c_weight: torch.Tensor, inv_freq: Optional[torch.Tensor],
+def latent_prep(down: torch.Tensor, q_weight: Optional[torch.Tensor], c_weight: torch.Tensor, inv_freq: Optional[torch.Tensor],
                 positions: torch.Tensor, slots: Optional[torch.Tensor], cache: Optional[torch.Tensor], q_rank: int,
-                rank: int, rot: int, rot_dims: int, eps: float, cache_t: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """The merged down projection [T, q_rank + rank + rot]: returns the normed query latent [T, q_rank]; writes the
+                rank: int, rot: int, rot_dims: int, eps: float, cache_t: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """The merged down projection [T, q_rank + rank + rot]: returns the normed query latent [T, q_rank] (None for a ``q_rank``
+    of 0); writes the
     normed latent and the rotated shared key part of every token into ``cache`` [pages, page, rank + rot] at ``slots``,
     and the latent once more into ``cache_t`` [pages, rank, page] where the cache keeps that copy."""
     _dev(q_weight, c_weight, inv_freq, positions, slots, cache, cache_t)   # ``down`` may be rows of a wider tensor
@@ -1254,7 +1255,7 @@ def latent_prep(down: torch.Tensor, q_weight: torch.Tensor, c_weight: torch.Tens
     _f32(inv_freq, "rotary frequencies")
     _i32(positions, "positions")
     t = down.shape[0]
-    if down.dim() != 2 or down.shape[1] != q_rank + rank + rot or down.stride(1) != 1 or q_weight.shape != (q_rank,) or \
+    if down.dim() != 2 or down.shape[1] != q_rank + rank + rot or down.stride(1) != 1 or (q_rank and q_weight.shape != (q_rank,)) or \
             c_weight.shape != (rank,):
         raise NativeError(f"latent_prep: input {tuple(down.shape)} for parts {q_rank} + {rank} + {rot}")
     if positions.shape != (t,) or (rot_dims and (inv_freq is None or inv_freq.shape != (rot_dims // 2,))):
@@ -1265,7 +1266,7 @@ def latent_prep(down: torch.Tensor, q_weight: torch.Tensor, c_weight: torch.Tens
             raise NativeError(f"latent_prep: cache must be [pages, page, {rank + rot}] of {down.dtype}")
         if cache_t is not None and (cache_t.dtype != cache.dtype or tuple(cache_t.shape) != (cache.shape[0], rank, cache.shape[1])):
             raise NativeError(f"latent_prep: the transposed copy must be [pages, {rank}, page] of {cache.dtype}")
-    cq = torch.empty((t, q_rank), dtype=down.dtype, device=down.device)
+    cq = torch.empty((t, q_rank), dtype=down.dtype, device=down.device) if q_rank else None
     caching = slots is not None
     check(kernels().pa_latent_prep(_stream(), _code(down), down.data_ptr(), _ptr(q_weight), _ptr(c_weight), _ptr(inv_freq),
                                    _ptr(positions), _ptr(slots), _ptr(cq), _ptr(cache) if caching else None,
@@ -1274,11 +1275,18 @@ def latent_prep(down: torch.Tensor, q_weight: torch.Tensor, c_weight: torch.Tens
     return cq
 
 
+def _heads_of_rows(x: torch.Tensor, what: str) -> None:
+    """x [T, heads, a] whose tokens' heads lie side by side, the tokens any distance apart."""
+    if not x.is_cuda or x.dim() != 3 or x.stride(2) != 1 or x.stride(1) != x.shape[2] or (x.shape[0] > 1 and x.stride(0) < x.shape[1] * x.shape[2]):
+        raise NativeError(f"{what}: {tuple(x.shape)} with strides {x.stride()} is not a row of heads a token")
+
+
 def rotate_pairs(x: torch.Tensor, out: torch.Tensor, inv_freq: Optional[torch.Tensor], positions: torch.Tensor, in_off: int,
                  out_off: int, width: int, rot_dims: int) -> None:
-    """x [T, heads, a] -> out [T, heads, b]: ``width`` elements from ``in_off`` of every head to ``out_off``, the first
-    ``rot_dims`` of them rotated in pairs (2i, 2i+1) by position * inv_freq[i]."""
-    _dev(x, out, inv_freq, positions)
+    """x [T, heads, a] (a token's heads may lie inside a wider row) -> out [T, heads, b]: ``width`` elements from ``in_off``
+    of every head to ``out_off``, the first ``rot_dims`` of them rotated in pairs (2i, 2i+1) by position * inv_freq[i]."""
+    _dev(out, inv_freq, positions)
+    _heads_of_rows(x, "rotate_pairs")
     _f32(inv_freq, "rotary frequencies")
     _i32(positions, "positions")
     if x.dim() != 3 or out.dim() != 3 or x.shape[:2] != out.shape[:2] or x.dtype != out.dtype or positions.shape != (x.shape[0],):
@@ -1286,7 +1294,7 @@ def rotate_pairs(x: torch.Tensor, out: torch.Tensor, inv_freq: Optional[torch.Te
     if rot_dims and (inv_freq is None or inv_freq.shape != (rot_dims // 2,)):
         raise NativeError("rotate_pairs: rotary frequencies do not match the rotated width")
     check(kernels().pa_rotate_pairs(_stream(), _code(x), _ptr(x), _ptr(out), _ptr(inv_freq), _ptr(positions), x.shape[0],
-                                    x.shape[1], x.shape[2], int(in_off), out.shape[2], int(out_off), int(width), int(rot_dims)))
+                                    x.shape[1], x.shape[2], int(in_off), out.shape[2], int(out_off), int(width), int(rot_dims), x.stride(0)))
 
 
 class GroupedWeight:
@@ -1307,17 +1315,19 @@ class GroupedWeight:
 
 
 def head_linear(x: torch.Tensor, w: GroupedWeight, out: torch.Tensor, x_off: int = 0, out_off: int = 0) -> None:
-    """out[t, h, out_off : out_off + n] = W[h] x[t, h, x_off : x_off + k] for x [T, heads, a], out [T, heads, b] and a
-    weight per head ``w`` [heads, n, k]."""
+    """out[t, h, out_off : out_off + n] = W[h] x[t, h, x_off : x_off + k] for x [T, heads, a], out [T, heads, b] (a token's
+    heads may lie inside a wider row in both) and a weight per head ``w`` [heads, n, k]."""
     k, n = w.k, w.n
     wt = w.nk if w.nk is not None else w.kn
-    _dev(x, wt, out)
+    _dev(wt)
+    _heads_of_rows(x, "head_linear")
+    _heads_of_rows(out, "head_linear")
     if (x.dim() != 3 or out.dim() != 3 or x.shape[:2] != out.shape[:2] or w.groups != x.shape[1]
             or not (x.dtype == w.dtype == out.dtype) or x_off + k > x.shape[2] or out_off + n > out.shape[2]):
         raise NativeError(f"head_linear: x {tuple(x.shape)} / w [{w.groups}, {n}, {k}] / out {tuple(out.shape)}")
     el = x.element_size()
-    strides = (x.shape[1] * x.shape[2], x.shape[2], out.shape[1] * out.shape[2], out.shape[2])
-    if w.nk is not None and x.shape[2] % 8 == 0 and x_off % 8 == 0:
+    strides = (x.stride(0), x.shape[2], out.stride(0), out.shape[2])
+    if w.nk is not None and x.shape[2] % 8 == 0 and x_off % 8 == 0 and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0:
         check(kernels().pa_head_linear_mfma(_stream(), x.data_ptr() + x_off * el, _ptr(wt), out.data_ptr() + out_off * el,
                                             x.shape[0], x.shape[1], k, n, *strides))
         return
@@ -1724,6 +1734,10 @@ def qkv_prepare(p: torch.Tensor, q_off: int, k_off: int, v_off: int, q_weight: O
     return q
 
 
+MASKED_MAX_KEY, MASKED_MAX_VALUE = 4096, 256   # widest key and value of the kernel on the vector units
+TALKING_MAX_LDS = 16384                        # 32-bit words of LDS: heads * (head width + heads)
+
+
 def attention_masked_mfma_supported(hd: int, vd: int, page_size: int) -> bool:
     """Whether ``attention_masked`` runs these widths on the matrix cores (bfloat16)."""
     return bool(kernels().pa_attn_masked_mfma_supports(int(hd), int(vd), int(page_size)))
@@ -1748,8 +1762,9 @@ def attention_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         raise NativeError(f"attention_masked: q {tuple(q.shape)} / caches")
     t, nh, hd = q.shape
     pages, nkv, page, khd = k_cache.shape
-    nv, vd = v_cache.shape[1], v_cache.shape[2]   # fewer value heads than key heads: key head k goes with value head k mod nv
-    if khd != hd or tuple(v_cache.shape) != (pages, nv, vd, page) or nkv % nv or k_cache.dtype != q.dtype or v_cache.dtype != q.dtype:
+    # fewer value heads than key heads: key head k goes with value head k mod nv; more: the query heads are dealt out to them
+    nv, vd = v_cache.shape[1], v_cache.shape[2]
+    if khd != hd or tuple(v_cache.shape) != (pages, nv, vd, page) or (nkv % nv and (nv % nkv or nh % nv)) or k_cache.dtype != q.dtype or v_cache.dtype != q.dtype:
         raise NativeError(f"attention_masked: caches {tuple(k_cache.shape)} / {tuple(v_cache.shape)} for q {tuple(q.shape)} {q.dtype}")
     for name, v in (("slopes", slopes), ("sink", sink)):
         if v is not None:
@@ -1976,3 +1991,158 @@ def cap_logits_(x: torch.Tensor, cap: float) -> torch.Tensor:
         raise NativeError("cap_logits: the logits are not contiguous")
     check(kernels().pa_cap_logits(_stream(), _ptr(x), x.numel(), float(cap)))
     return x
+
+
+# ---------------------------------------------------------------------------
+# Layer norm around a 32-bit stream; what such a stream takes between layers
+def layer_norm_step(x, residual: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, eps: float, out_dtype: torch.dtype,
+                    rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """residual += x (a tensor [T, H], ``SliceSums``, or None: nothing), then the layer norm of the 32-bit ``residual``
+    [T, H] times ``weight`` plus ``bias``, in ``out_dtype``.  With ``rows`` (int32 [R]): of those rows of the sum alone, and the
+    residual is read only."""
+    parts, y = (x.parts, None) if isinstance(x, SliceSums) else (None, x)
+    _dev(y, parts, residual, weight, bias, rows)
+    for t, name in ((residual, "residual"), (weight, "norm weight"), (bias, "norm bias")):
+        _f32(t, name)
+    if residual.dim() != 2:
+        raise NativeError(f"layer_norm_step: the stream {tuple(residual.shape)} is not [T, H]")
+    m, h = residual.shape
+    if tuple(weight.shape) != (h,) or tuple(bias.shape) != (h,) or (x is not None and (tuple(x.shape) != (m, h) or x.dtype != out_dtype)):
+        raise NativeError(f"layer_norm_step: branch {None if x is None else (tuple(x.shape), x.dtype)} / weight {tuple(weight.shape)} "
+                          f"beside a stream {tuple(residual.shape)} and an output of {out_dtype}")
+    n = m
+    if rows is not None:
+        _i32(rows, "rows")
+        n = rows.shape[0]
+    out = torch.empty((n, h), dtype=out_dtype, device=residual.device)
+    check(kernels().pa_layer_norm_step(_stream(), _CODES[out_dtype], _ptr(y), _ptr(parts), 0 if parts is None else parts.shape[0],
+                                       m * h, _ptr(residual), _ptr(weight), _ptr(bias), _ptr(out), _ptr(rows), n, h, float(eps)))
+    return out
+
+
+def stream_sum(x: torch.Tensor, y: Optional[torch.Tensor] = None, extra: Optional[torch.Tensor] = None,
+               row: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x + y + extra + row in 32-bit, x and ``extra`` float32 [T, H], ``y`` [T, H] of the engine's type, ``row`` float32 [H];
+    into ``out`` (may be x) or a fresh tensor."""
+    _dev(x, y, extra, row, out)
+    for t, name in ((x, "stream"), (extra, "extra"), (row, "row"), (out, "out")):
+        _f32(t, name)
+    if x.dim() != 2 or any(t is not None and t.shape != x.shape for t in (y, extra, out)) or (row is not None and tuple(row.shape) != (x.shape[1],)):
+        raise NativeError(f"stream_sum: the operands do not match a stream {tuple(x.shape)}")
+    if out is None:
+        out = torch.empty_like(x)
+    check(kernels().pa_stream_sum(_stream(), 0 if y is None else _code(y), _ptr(x), _ptr(y), _ptr(extra), _ptr(row), _ptr(out),
+                                  x.shape[0], x.shape[1]))
+    return out
+
+
+def embed_scaled(ids: torch.Tensor, table: torch.Tensor, scale: float) -> torch.Tensor:
+    """table[ids] * scale as float32 [T, H]."""
+    _dev(ids, table)
+    _i32(ids, "ids")
+    if ids.dim() != 1 or table.dim() != 2:
+        raise NativeError(f"embed_scaled: ids {tuple(ids.shape)} / table {tuple(table.shape)}")
+    out = torch.empty((ids.shape[0], table.shape[1]), dtype=torch.float32, device=table.device)
+    check(kernels().pa_embed_scaled(_stream(), _code(table), _ptr(ids), _ptr(table), _ptr(out), ids.shape[0], table.shape[1],
+                                    table.shape[0], float(scale)))
+    return out
+
+
+def activate(x: torch.Tensor, activation: str, out: Optional[torch.Tensor] = None, scale: float = 1.0) -> torch.Tensor:
+    """act(x) * scale, element by element in 32-bit; x and ``out`` [T, N], rows may lie inside wider tensors."""
+    act = gate_activation_code(activation)
+    if out is None:
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+    for t in (x, out):
+        if not t.is_cuda or t.dim() != 2 or t.stride(1) != 1 or t.shape != x.shape or t.dtype != x.dtype:
+            raise NativeError(f"activate: x {tuple(x.shape)} {x.dtype} / out {tuple(out.shape)} {out.dtype}")
+    if x.shape[0]:
+        check(kernels().pa_activate(_stream(), _code(x), x.data_ptr(), x.stride(0), out.data_ptr(), out.stride(0), x.shape[0],
+                                    x.shape[1], act, float(scale)))
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Attention whose heads' scores are mixed
+def talking_prepare(p: torch.Tensor, q_off: int, k_off: int, v_off: int, biases, q_weight: Optional[torch.Tensor],
+                    k_weight: Optional[torch.Tensor], inv_freq: Optional[torch.Tensor], positions: torch.Tensor, talk: torch.Tensor,
+                    slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, nh: int, nkv: int, hd: int, vd: int, rot: int,
+                    value_norm: bool, eps: float) -> torch.Tensor:
+    """From the merged projection ``p`` [T, width]: queries mixed by ``talk`` (float32 [nh, nh]) over the key heads side by
+    side, [T, nh, nkv * hd]; keys into K [pages, 1, page, nkv * hd] and values into V [pages, nkv, vd, page] at ``slots``.
+    ``biases``: (q, k, v) float32 or None; ``q_weight`` / ``k_weight`` float32 [hd]: every head over its own root mean square
+    times it; the first ``rot`` dimensions turned in pairs by position * inv_freq[i]; ``value_norm``: every value head over
+    its own root mean square.  All of it in 32-bit, rounded once."""
+    bq, bk, bv = biases if biases is not None else (None, None, None)
+    _dev(bq, bk, bv, q_weight, k_weight, inv_freq, positions, talk, slots, k_cache, v_cache)
+    for t, name in ((bq, "bias"), (bk, "bias"), (bv, "bias"), (q_weight, "query norm weight"), (k_weight, "key norm weight"),
+                    (inv_freq, "rotary frequencies"), (talk, "mixing matrix")):
+        _f32(t, name)
+    _i32(positions, "positions")
+    _i32(slots, "slots")
+    t = p.shape[0]
+    if not p.is_cuda or p.dim() != 2 or p.stride(1) != 1 or positions.shape != (t,) or slots.shape != (t,):
+        raise NativeError(f"talking_prepare: projection {tuple(p.shape)} with strides {p.stride()}, or positions or slots of another size")
+    page = k_cache.shape[2]
+    if k_cache.dtype != p.dtype or v_cache.dtype != p.dtype or tuple(k_cache.shape[1:]) != (1, page, nkv * hd) or \
+            tuple(v_cache.shape) != (k_cache.shape[0], nkv, vd, page):
+        raise NativeError(f"talking_prepare: caches {tuple(k_cache.shape)} / {tuple(v_cache.shape)} for {nkv} heads of {hd} and {vd}")
+    for v, size, name in ((bq, nh * hd, "bias"), (bk, nkv * hd, "bias"), (bv, nkv * vd, "bias"), (q_weight, hd, "norm weight"),
+                          (k_weight, hd, "norm weight")):
+        if v is not None and tuple(v.shape) != (size,):
+            raise NativeError(f"talking_prepare: {name} {tuple(v.shape)} is not [{size}]")
+    if tuple(talk.shape) != (nh, nh) or (rot and (inv_freq is None or tuple(inv_freq.shape) != (rot // 2,))):
+        raise NativeError(f"talking_prepare: mixing matrix {tuple(talk.shape)} or frequencies do not match")
+    q = torch.empty((t, nh, nkv * hd), dtype=p.dtype, device=p.device)
+    if t:
+        check(kernels().pa_talking_prepare(_stream(), _code(p), p.data_ptr(), p.stride(0), int(q_off), int(k_off), int(v_off), _ptr(bq),
+                                           _ptr(bk), _ptr(bv), _ptr(q_weight), _ptr(k_weight), _ptr(inv_freq), _ptr(positions),
+                                           _ptr(talk), _ptr(slots), _ptr(q), _ptr(k_cache), _ptr(v_cache), t, nh, nkv, hd, vd,
+                                           int(rot), 1 if value_norm else 0, page, float(eps)))
+    return q
+
+
+# ---------------------------------------------------------------------------
+# Gated linear attention
+def gated_linear_attention(p: torch.Tensor, q_off: int, k_off: int, v_off: int, low_off: int, a2: torch.Tensor, a2_bias: torch.Tensor,
+                           tau: float, state: torch.Tensor, step, heads: int, dim: int, vdim: int,
+                           chunk: Optional[int] = None) -> torch.Tensor:
+    """Per head S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t dim^(-1/2), a decay per key channel
+    alpha = sigmoid(a2 low + a2_bias)^(1 / tau).
+
+    ``p`` [T, width] (rows may lie inside a wider tensor): a token's queries and keys [heads, dim], values [heads, vdim] and low-rank vector
+    [rank] start at the given columns; ``a2`` [heads * dim, rank] of the engine's type, ``a2_bias`` float32; state float32
+    [slots, heads, dim, vdim], read and left by the step's sequences.  Returns float32 [T, heads, vdim].
+
+    ``chunk``: as in ``lightning_attention``."""
+    _dev(a2, a2_bias, state)
+    _f32(a2_bias, "decay bias")
+    _f32(state, "state")
+    t, rank = p.shape[0], a2.shape[1]
+    if not p.is_cuda or p.dim() != 2 or p.stride(1) != 1 or a2.dtype != p.dtype or tuple(a2.shape) != (heads * dim, rank) or \
+            tuple(a2_bias.shape) != (heads * dim,) or state.dim() != 4 or tuple(state.shape[1:]) != (heads, dim, vdim) or \
+            max(q_off, k_off) + heads * dim > p.shape[1] or v_off + heads * vdim > p.shape[1] or low_off + rank > p.shape[1]:
+        raise NativeError(f"gated_linear_attention: p {tuple(p.shape)} / a2 {tuple(a2.shape)} / state {tuple(state.shape)} for {heads} heads "
+                          f"of {dim} and {vdim}")
+    if chunk is None:
+        chunk = LIGHTNING_CHUNK if p.dtype == torch.bfloat16 else 0
+    q_scale = float(dim) ** -0.5
+    chunked = chunk > 0 and step.n_prefill > 0 and step.max_prefill_q > chunk
+    out = torch.empty((t, heads, vdim), dtype=torch.float32, device=p.device)
+    cols = (_code(p), p.data_ptr(), p.stride(0), int(q_off), int(k_off), int(v_off))
+    where = (_ptr(state), _ptr(step.state_slots), _ptr(step.cu_q))
+    singles = getattr(step, "n_decode", 0) > 0
+    if singles:
+        check(kernels().pa_gla_step(_stream(), *cols, int(low_off), _ptr(a2), _ptr(a2_bias), *where, _ptr(out), step.num_seqs, heads, dim,
+                                    vdim, rank, float(tau), q_scale))
+    if step.n_prefill > 0 or not singles:
+        alpha = torch.empty((t, heads * dim), dtype=torch.float32, device=p.device)
+        check(kernels().pa_gla_decay(_stream(), *cols[:3], int(low_off), _ptr(a2), _ptr(a2_bias), _ptr(alpha), t, heads * dim, rank, float(tau)))
+        check(kernels().pa_gla_attn(_stream(), *cols, _ptr(alpha), *where, _ptr(out), step.num_seqs, t, heads, dim, vdim, q_scale,
+                                    int(chunk) if chunked else 0, 2 if singles else 0))
+        if chunked:
+            words = kernels().pa_gla_chunked_workspace(step.n_prefill, t, heads, dim, vdim, int(chunk))
+            work = torch.empty((max(words, 1),), dtype=torch.float32, device=p.device)
+            check(kernels().pa_gla_attn_chunked(_stream(), *cols, _ptr(alpha), *where, _ptr(step.prefill_seqs), _ptr(out), _ptr(work),
+                                                step.n_prefill, t, int(step.max_prefill_q), heads, dim, vdim, q_scale, int(chunk)))
+    return out

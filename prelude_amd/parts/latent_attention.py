@@ -1,7 +1,7 @@
 """Attention through a latent, with a learned sink in the softmax.
 
-Queries come through a latent of their own: c_q = RMSNorm(W_dq h) * g_q, q = W_uq c_q, laid out head by head
-as [dim unrotated | rot rotated].  One down projection gives rank + rot numbers a token: the first rank,
+Queries come through a latent of their own: c_q = RMSNorm(W_dq h) * g_q, q = W_uq c_q (or straight from h, q = W_q h, with
+``q_rank`` 0), laid out head by head as [dim unrotated | rot rotated].  One down projection gives rank + rot numbers a token: the first rank,
 RMS-normed, are the latent c, the rest one rotated key part shared by all heads.  Head h's unrotated key is
 W_uk[h] c and its value W_uv[h] c, so only c and the rotated part are cached (``LatentCacheSpec``), and both maps
 move to the query side:
@@ -77,11 +77,14 @@ class LatentAttention(Mixer):
                  q_rank: int, norm_eps: float, scale: Optional[float] = None, position: Optional[str] = None,
                  rotary_dim: Optional[int] = None, sink: bool = False, window: int = 0, output_gate: bool = False):
         for name, v in (("hidden_size", hidden_size), ("num_heads", num_heads), ("head_dim", head_dim),
-                        ("value_dim", value_dim), ("kv_rank", kv_rank), ("q_rank", q_rank)):
+                        ("value_dim", value_dim), ("kv_rank", kv_rank)):
             if int(v) <= 0:
                 raise PartError(f"latent_attention: {name} {v} must be positive")
         self.hidden_size, self.num_heads, self.head_dim = int(hidden_size), int(num_heads), int(head_dim)
-        self.rot_dim, self.value_dim, self.kv_rank, self.q_rank = int(rot_dim), int(value_dim), int(kv_rank), int(q_rank)
+        self.rot_dim, self.value_dim, self.kv_rank = int(rot_dim), int(value_dim), int(kv_rank)
+        self.q_rank = int(q_rank or 0)   # 0: the queries are a product of the mixer's input (tensor ``q``)
+        if self.q_rank < 0:
+            raise PartError(f"latent_attention: q_rank {q_rank} is negative")
         self.norm_eps, self.window, self.sink = float(norm_eps), int(window or 0), bool(sink)
         # the heads' outputs side by side times sigmoid(W_g x), element by element (tensor ``g`` [heads * value_dim,
         # hidden]); the gate reads the mixer's input, as the projections do
@@ -112,9 +115,10 @@ class LatentAttention(Mixer):
 
     def tensors(self):
         h, nh, d, r, v = self.hidden_size, self.num_heads, self.head_dim, self.rot_dim, self.value_dim
-        t = {"dq": TensorReq((self.q_rank, h), MATRIX), "dq.norm": TensorReq((self.q_rank,), NORM),
-             "uq": TensorReq((nh * (d + r), self.q_rank), MATRIX),
-             "dkv": TensorReq((self.kv_rank + r, h), MATRIX), "dkv.norm": TensorReq((self.kv_rank,), NORM),
+        t = {"q": TensorReq((nh * (d + r), h), MATRIX)} if not self.q_rank else \
+            {"dq": TensorReq((self.q_rank, h), MATRIX), "dq.norm": TensorReq((self.q_rank,), NORM),
+             "uq": TensorReq((nh * (d + r), self.q_rank), MATRIX)}
+        t |= {"dkv": TensorReq((self.kv_rank + r, h), MATRIX), "dkv.norm": TensorReq((self.kv_rank,), NORM),
              "uk": TensorReq((nh * d, self.kv_rank), MATRIX), "uv": TensorReq((nh * v, self.kv_rank), MATRIX),
              "o": TensorReq((h, nh * v), MATRIX)}
         if self.sink:
@@ -123,22 +127,36 @@ class LatentAttention(Mixer):
             t["g"] = TensorReq((nh * v, h), MATRIX)
         return t
 
-    def load(self, tensors, dtype, device):
+    @property
+    def mixed_size(self) -> int:
+        return self.num_heads * self.value_dim
+
+    @property
+    def query_columns(self) -> int:
+        """Columns of the product of the mixer's input that the queries take: their latent, or the queries themselves."""
+        return self.q_rank or self.num_heads * (self.head_dim + self.rot_dim)
+
+    def input_rows(self, tensors) -> torch.Tensor:
+        """The rows of the product of its input this mixer wants, [query latent or queries | kv_rank | rot | gate]; keeps its
+        other tensors."""
         nh, d, v, rank = self.num_heads, self.head_dim, self.value_dim, self.kv_rank
-        # one product for both down projections: [q_rank | kv_rank | rot] rows
-        down = [tensors["dq"], tensors["dkv"]] + ([tensors["g"]] if self.output_gate else [])   # the gate's rows ride along
-        self.w_down = K.prepare_weight(torch.cat(down, dim=0).contiguous())
-        self.w_uq = K.prepare_weight(tensors["uq"])
-        self.w_o = K.prepare_weight(tensors["o"])
+        if self.q_rank:
+            self.w_uq, self.q_norm = K.prepare_weight(tensors["uq"]), tensors["dq.norm"]
         # the per-head maps as [head, out, in]: W_uk[h] is [d, rank] as stored and is applied transposed (out rank,
         # in d); W_uv[h] is [v, rank] and is applied as it is
         self.uk_t = K.GroupedWeight(tensors["uk"].reshape(nh, d, rank).transpose(1, 2))
         self.uv_t = K.GroupedWeight(tensors["uv"].reshape(nh, v, rank))
-        self.q_norm, self.c_norm = tensors["dq.norm"], tensors["dkv.norm"]
+        self.c_norm = tensors["dkv.norm"]
         self.sinks = tensors["sink"] if self.sink else None
-        if self.rot_dim == 0 and not self.sink and dtype == torch.bfloat16:
+        if self.rot_dim == 0 and not self.sink and tensors["uk"].dtype == torch.bfloat16:
             # for the expanded form: every head's keys, then every head's values, from a latent by one product
             self.w_ukv = K.prepare_weight(torch.cat([tensors["uk"], tensors["uv"]], dim=0).contiguous())
+        rows = [tensors["dq" if self.q_rank else "q"], tensors["dkv"]] + ([tensors["g"]] if self.output_gate else [])
+        return torch.cat(rows, dim=0)
+
+    def load(self, tensors, dtype, device):
+        self.w_down = K.prepare_weight(self.input_rows(tensors).contiguous())
+        self.w_o = K.prepare_weight(tensors["o"])
 
     def _expands(self, x, step, cache, write_cache) -> bool:
         if not (self.w_ukv is not None and write_cache and x.dtype == torch.bfloat16 and getattr(step, "graph", None) is None
@@ -151,7 +169,7 @@ class LatentAttention(Mixer):
         rows = sum(min(s + n, n + (self.window or s + n) + page) for s, n in zip(step.starts, step.q_lens))
         return rows <= 4 * step.num_tokens
 
-    def _expanded(self, q, step, cache, g):
+    def _expanded(self, q, step, cache, g, out=None):
         """The heads' outputs side by side [T, heads * value_dim] from keys and values made of the visible latents."""
         nh, d, v, rank = self.num_heads, self.head_dim, self.value_dim, self.kv_rank
         page = cache.latent.shape[1]
@@ -162,34 +180,37 @@ class LatentAttention(Mixer):
         v_tmp = torch.zeros((plan.pages, nh, v, page), dtype=q.dtype, device=q.device)
         K.qkv_rope_prepare(kv, 0, 0, nh * d, None, plan.pos, plan.slots, k_tmp, v_tmp, 0, nh, nh, d, v, 0, False)
         return K.attention_masked(q.contiguous(), k_tmp, v_tmp, types.SimpleNamespace(block_table=plan.table), step, self.window, 0,
-                                  self.scale)
+                                  self.scale, out=out)
 
-    def forward(self, x, step, cache, write_cache=True):
+    def mix(self, x, p, off, step, cache, write_cache, out=None, out_scale=1.0):
+        """From the product ``p`` of its input (its columns start at ``off``) to the heads' outputs side by side
+        [T, heads * value_dim], into ``out`` when given."""
+        if out_scale != 1.0 or (out is not None and self.output_gate):
+            raise PartError("latent_attention: beside other branches it has neither a scale nor an output gate")
         nh, d, r, v, rank = self.num_heads, self.head_dim, self.rot_dim, self.value_dim, self.kv_rank
         g = step.kv[cache.group]
         freq = self.rope.inv_freq if self.rope is not None else None
-        down = K.linear(x, self.w_down)
-        gate = None
-        if self.output_gate:
-            gate = down[:, self.q_rank + rank + r:]
-            down = down[:, : self.q_rank + rank + r]
-        cq = K.latent_prep(down, self.q_norm, self.c_norm, freq, step.positions, g.slots if write_cache else None,
+        # what the norm and the cache write read: the query latent (if there is one) and the latent beside it
+        first = off if self.q_rank else off + self.query_columns
+        at = off + self.query_columns + rank + r
+        cq = K.latent_prep(p[:, first: at], self.q_norm, self.c_norm, freq, step.positions, g.slots if write_cache else None,
                            cache.latent if write_cache else None, self.q_rank, rank, r, self.rotary_dim, self.norm_eps,
                            cache_t=cache.latent_t if write_cache else None)
-        q = K.linear(cq, self.w_uq).view(-1, nh, d + r)
+        if self.q_rank:
+            q = K.linear(cq, self.w_uq).view(-1, nh, d + r)
+        else:
+            q = p[:, off: off + nh * (d + r)].unflatten(1, (nh, d + r))
         if self._expands(x, step, cache, write_cache):
-            o = self._expanded(q, step, cache, g)
-            if gate is not None:
-                o = K.sigmoid_gate(o, gate)
-            return K.linear(o, self.w_o, slices_ok=True)
-        ql = torch.empty((q.shape[0], nh, rank + r), dtype=q.dtype, device=q.device)
-        K.head_linear(q, self.uk_t, ql)                                             # the key map, on the query side
-        if r:
-            K.rotate_pairs(q, ql, freq, step.positions, d, rank, r, self.rotary_dim)
-        ol = K.latent_attention(ql, cache.latent, self.sinks, g, step, rank, self.window, self.scale, cache_t=cache.latent_t)
-        o = torch.empty((q.shape[0], nh, v), dtype=q.dtype, device=q.device)
-        K.head_linear(ol, self.uv_t, o)                                            # the value map, after the sum
-        o = o.view(-1, nh * v)
-        if gate is not None:
-            o = K.sigmoid_gate(o, gate)
-        return K.linear(o, self.w_o, slices_ok=True)
+            o = self._expanded(q, step, cache, g, out)
+        else:
+            ql = torch.empty((q.shape[0], nh, rank + r), dtype=q.dtype, device=q.device)
+            K.head_linear(q, self.uk_t, ql)                                         # the key map, on the query side
+            if r:
+                K.rotate_pairs(q, ql, freq, step.positions, d, rank, r, self.rotary_dim)
+            ol = K.latent_attention(ql, cache.latent, self.sinks, g, step, rank, self.window, self.scale, cache_t=cache.latent_t)
+            o = torch.empty((q.shape[0], nh * v), dtype=q.dtype, device=q.device) if out is None else out
+            K.head_linear(ol, self.uv_t, o.unflatten(1, (nh, v)))                   # the value map, after the sum
+        return K.sigmoid_gate(o, p[:, at: at + nh * v]) if self.output_gate else o
+
+    def forward(self, x, step, cache, write_cache=True):
+        return K.linear(self.mix(x, K.linear(x, self.w_down), 0, step, cache, write_cache), self.w_o, slices_ok=True)

@@ -6,6 +6,8 @@ head logits = W h with W [vocab, hidden], the embedding matrix itself when tied
 """
 from __future__ import annotations
 
+from typing import Optional
+
 import torch
 
 from ..ops import kernels as K
@@ -16,8 +18,10 @@ from .base import MATRIX, Part, PartError, StateSpec, TensorReq, register_part
 class TokenEmbedding(Part):
     GRAPH_SAFE_PORTIONS = True   # launches follow the step's shape alone; tokens, positions and pages are read on the device
 
-    def __init__(self, vocab_size: int, hidden_size: int):
+    def __init__(self, vocab_size: int, hidden_size: int, scale: Optional[float] = None):
+        """``scale``: the rows leave as table[token] * scale in 32-bit, as the stream; None: as they are stored."""
         self.vocab_size, self.hidden_size = int(vocab_size), int(hidden_size)
+        self.scale = None if scale is None else float(scale)
         self.weight = None
 
     def tensors(self):
@@ -27,6 +31,8 @@ class TokenEmbedding(Part):
         self.weight = tensors["weight"]
 
     def forward(self, token_ids: torch.Tensor) -> torch.Tensor:
+        if self.scale is not None:
+            return K.embed_scaled(token_ids, self.weight, self.scale)
         return K.embed_gather(token_ids, self.weight)
 
 

@@ -128,3 +128,38 @@ class PolyNormMLP(FeedForward):
     def forward(self, x):
         z = K.linear(x, self.up)
         return K.linear(K.poly_norm(z, self.coeff, self.eps, bias=self.up_bias), self.down, self.down_bias)
+
+
+@register_part("ffn", "plain_mlp")
+class PlainMLP(FeedForward):
+    """down(act(up(x))): two products and an activation between them, no gate and no biases.  It can stand beside a mixer
+    that reads the same input (``parallel_mixers``): its first product's rows then ride in that one's product, and its
+    second adds up with the mixer's output projection."""
+    LAUNCHES = 3
+    GRAPH_SAFE_PORTIONS = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "gelu_tanh"):
+        if activation not in K.GATE_ACTIVATIONS:
+            raise PartError(f"plain_mlp: activation {activation!r} is not one of {sorted(K.GATE_ACTIVATIONS)}")
+        self.hidden_size, self.intermediate_size, self.activation = int(hidden_size), int(intermediate_size), activation
+        self.up = self.down = None
+
+    @property
+    def mixed_size(self) -> int:
+        return self.intermediate_size
+
+    def tensors(self):
+        h, i = self.hidden_size, self.intermediate_size
+        return {"up": TensorReq((i, h), MATRIX), "o": TensorReq((h, i), MATRIX)}
+
+    def input_rows(self, tensors) -> torch.Tensor:
+        return tensors["up"]
+
+    def load(self, tensors, dtype, device):
+        self.up, self.down = K.prepare_weight(tensors["up"]), K.prepare_weight(tensors["o"])
+
+    def mix(self, x, p, off, step, cache, write_cache, out=None, out_scale=1.0):
+        return K.activate(p[:, off: off + self.intermediate_size], self.activation, out, out_scale)
+
+    def forward(self, x):
+        return K.linear(K.activate(K.linear(x, self.up), self.activation), self.down, slices_ok=True)

@@ -1,4 +1,4 @@
-"""RMSNorm, alone, fused with the residual add in front of it, or on a branch's output with the add behind it.
+"""RMSNorm, alone, fused with the residual add in front of it, or on a branch's output with the add behind it; layer norm.
 
 y = x * rsqrt(mean(x^2) + eps) * w in 32-bit
 (crates/prelude-core/src/models/commons/linear.rs:435-501); with a residual:
@@ -133,3 +133,41 @@ class GroupRMSNorm(Norm):
             return K.group_norm_step(self._stream(residual), self.groups, self.eps, y=K.as_tensor(y), w_add=self.weight,
                                      w_out=then.weight, out_dtype=out_dtype)
         return super().forward_branch_then(y, residual, then, out_dtype)
+
+
+@register_part("norm", "layer_norm")
+class LayerNorm(Norm):
+    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * weight + bias around a 32-bit stream: the branch's output that waits is added
+    to the stream and the new row normed in one launch; the normed output is of the engine's type."""
+    GRAPH_SAFE_PORTIONS = True
+    TAKES_SLICE_SUMS = True
+
+    def __init__(self, size: int, eps: float):
+        self.size, self.eps = int(size), float(eps)
+        self.weight = self.bias = self.dtype = None
+
+    def tensors(self):
+        return {"weight": TensorReq((self.size,), NORM), "bias": TensorReq((self.size,), VECTOR)}
+
+    def load(self, tensors, dtype, device):
+        self.weight, self.bias, self.dtype = tensors["weight"], tensors["bias"], dtype
+
+    @staticmethod
+    def _stream(residual):
+        if residual is None or residual.dtype != torch.float32:
+            raise PartError("layer_norm: works around a 32-bit stream")
+        return residual
+
+    def forward_residual(self, x, residual):
+        """residual None: the stream starts as x in 32-bit.  x None: nothing waits to be added."""
+        if residual is None:
+            x, residual = None, K.to_f32(K.as_tensor(x))
+        return residual, K.layer_norm_step(x, self._stream(residual), self.weight, self.bias, self.eps, self.dtype)
+
+    def forward_stream(self, residual, out_dtype):
+        return K.layer_norm_step(None, self._stream(residual), self.weight, self.bias, self.eps, out_dtype)
+
+    def forward_rows(self, x, residual, rows, out_dtype=None):
+        if residual is None:
+            x, residual = None, K.to_f32(K.as_tensor(x))
+        return K.layer_norm_step(x, self._stream(residual), self.weight, self.bias, self.eps, out_dtype or self.dtype, rows=rows)

@@ -1,7 +1,7 @@
-"""Mixers side by side: several mixers read the same input, and the layer's mixer output is the sum of theirs, each
-times a constant.
+"""Branches side by side: several mixers (or a mixer and a feed-forward) read the same input, and the layer's mixer output
+is the sum of theirs, each times a constant.
 
-A member is any mixer that offers ``input_rows(tensors)`` (the rows of the product of its input it wants),
+A member is any mixer or feed-forward that offers ``input_rows(tensors)`` (the rows of the product of its input it wants),
 ``mix(x, p, off, step, cache, write_cache, out, out_scale)`` (from that product to what its output projection reads,
 written into a slice of a shared row) and ``mixed_size``, and names its output projection ``o``.  The members' input
 rows are one product, and their output projections one product over the members' outputs side by side (each already
@@ -23,14 +23,14 @@ class ParallelMixers(Mixer):
     GRAPH_SAFE_PORTIONS = True
 
     def __init__(self, hidden_size: int, members: Sequence[Mapping[str, Any]]):
-        """``members``: per member ``{"kind": ..., "params": {...}, "scale": c}``; a member's tensors are named
-        ``"<index>.<its local name>"``."""
+        """``members``: per member ``{"kind": ..., "params": {...}, "scale": c, "category": "mixer" | "ffn"}`` (scale 1 and a
+        mixer where they go unsaid); a member's tensors are named ``"<index>.<its local name>"``."""
         if not members:
             raise PartError("parallel_mixers: no members")
         self.hidden_size = int(hidden_size)
         self.members, self.scales = [], []
         for m in members:
-            part = build_part("mixer", m["kind"], m["params"])
+            part = build_part(m.get("category", "mixer"), m["kind"], m["params"])
             for need in ("input_rows", "mix", "mixed_size"):
                 if not hasattr(part, need):
                     raise PartError(f"parallel_mixers: a {m['kind']} offers no `{need}` and cannot stand beside others")
@@ -39,7 +39,7 @@ class ParallelMixers(Mixer):
         self.GRAPH_SAFE = all(p.GRAPH_SAFE for p in self.members)
         self.GRAPH_SAFE_PORTIONS = all(p.GRAPH_SAFE_PORTIONS for p in self.members)
         self.LAUNCHES = sum(p.LAUNCHES for p in self.members) - 2 * (len(self.members) - 1)
-        self.ATOMIC_PREFILL = any(p.ATOMIC_PREFILL for p in self.members)
+        self.ATOMIC_PREFILL = any(getattr(p, "ATOMIC_PREFILL", False) for p in self.members)
         self.w_in = self.w_o = None
         self.in_offsets, self.out_offsets = [], []
 
@@ -47,8 +47,13 @@ class ParallelMixers(Mixer):
         for p in self.members:
             p.bind(shared)
 
+    @staticmethod
+    def _keeps(part):
+        """What a member keeps between steps: a spec, or None (a feed-forward keeps nothing)."""
+        return part.cache_spec() if hasattr(part, "cache_spec") else None
+
     def cache_spec(self):
-        return tuple(cs for cs in (p.cache_spec() for p in self.members) if cs is not None)
+        return tuple(cs for cs in (self._keeps(p) for p in self.members) if cs is not None)
 
     def tensors(self):
         return {f"{i}.{name}": req for i, p in enumerate(self.members) for name, req in p.tensors().items()}
@@ -75,7 +80,7 @@ class ParallelMixers(Mixer):
         mixed = torch.empty((x.shape[0], self.total_out), dtype=x.dtype, device=x.device)
         caches = iter(cache if isinstance(cache, tuple) else (cache,))
         for part, scale, off, ooff in zip(self.members, self.scales, self.in_offsets, self.out_offsets):
-            c = next(caches) if part.cache_spec() is not None else None
+            c = next(caches) if self._keeps(part) is not None else None
             out = mixed[:, ooff: ooff + part.mixed_size]
             part.mix(x, p, off, step, c, write_cache, out, scale)
         return K.linear(mixed, self.w_o, slices_ok=True)
