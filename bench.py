@@ -196,6 +196,42 @@ def nivasun_record(args):
     return arch_record(args, "nivasun", (("nivasun", nivasun_shape(layers)), ("fazopel_beside", fazopel_beside_nivasun(runs))))
 
 
+# ``--arch pugavik``: a decoder of the Pugavik design at layer sizes of a real model of that kind: eight layers in periods of
+# four (attention through latents with a shared rotated key part; attention whose heads' scores are mixed, under a window
+# of 1,024; gated linear attention; latents again), a dense feed-forward beside every mixer on the same norm, the four
+# layers in the middle run twice (twelve runs) -- beside the closest existing design at equal size, a Fazopel decoder of
+# twelve layers with plain attention in the attentions' places, linear attention with a fixed decay in the recurrences', and
+# dense feed-forwards of the same size
+def pugavik_shape(layers=8, width=2048, vocab=65536):
+    dense = dict(kind="dense", ff=8192)
+    latent = dict(heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, scale=192 ** -0.5, rot=dict(base=10000.0, dims=64))
+    mixed = dict(heads=16, kv_heads=4, dim=64, vdim=128, scale=64 ** -0.5, mask=dict(size=1024), rot=dict(base=1000000.0, dims=64))
+    gla = dict(heads=16, dim=128, vdim=128, tau=16.0, rank=16)
+    period = (("latent_attention", latent), ("attention", mixed), ("gla", gla), ("latent_attention", latent))
+    start = min(2, layers)
+    return dict(architecture="Pugavik", vocab=vocab, width=width, norm=dict(eps=1e-5), embedding=dict(scale=width ** 0.5),
+                layers=[dict(type=period[i % 4][0], mixer=period[i % 4][1], mlp=dense) for i in range(layers)],
+                loop=dict(start=start, stop=max(start, layers - 2), times=2))
+
+
+def fazopel_beside_pugavik(layers=8):
+    from prelude_amd.config.model_config import PugavikConfig
+    from prelude_amd.models.pugavik import run_order
+    own = pugavik_shape(layers)
+    raw = fazopel_shape(4)
+    lightning, attention = raw["layers"][0]["mixer"], raw["layers"][3]["mixer"]
+    order = [own["layers"][i]["type"] for i, _ in run_order(PugavikConfig.from_dict(own))]
+    raw["layers"] = [dict(type="lightning" if t == "gla" else "attention", mixer=lightning if t == "gla" else attention,
+                          mlp=dict(kind="dense", ff=8192)) for t in order]
+    return raw
+
+
+def pugavik_record(args):
+    """Prefill and decode throughput of the Pugavik shape and of a dense Fazopel shape beside it, same points."""
+    layers = args.layers or 8
+    return arch_record(args, "pugavik", (("pugavik", pugavik_shape(layers)), ("fazopel_beside", fazopel_beside_pugavik(layers))))
+
+
 def build_engine(raw, dtype, cache_tokens, seed=0, page_size=16, **cfg_overrides):
     """The engine in its random-weights mode: the product's own loader, tensors drawn on the device."""
     from prelude_amd.config import EngineConfig
@@ -431,8 +467,8 @@ def main() -> int:
     ap.add_argument("--layers", type=int, default=None, help="fewer layers than the configuration has (named in config)")
     ap.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
     ap.add_argument("--shape", default="4b", choices=sorted(SHAPES), help="layer sizes: Qwen3-4B (the default run), 0.6B, 8B or 32B")
-    ap.add_argument("--arch", default="qwen3", choices=["qwen3", "libodra", "fazopel", "tedalix", "nivasun"],
-                    help="libodra, fazopel, tedalix, nivasun: prefill and decode of that design at a real model's layer sizes beside the closest other "
+    ap.add_argument("--arch", default="qwen3", choices=["qwen3", "libodra", "fazopel", "tedalix", "nivasun", "pugavik"],
+                    help="libodra, fazopel, tedalix, nivasun, pugavik: prefill and decode of that design at a real model's layer sizes beside the closest other "
                          "decoder of equal size, as one record (the default run and its record are Qwen3's)")
     ap.add_argument("--prefill-tokens", type=int, default=2048)
     ap.add_argument("--no-points", action="store_true", help="skip the points at other batches and lengths")
@@ -467,6 +503,9 @@ def main() -> int:
         return 0
     if args.arch == "nivasun":
         print(json.dumps(nivasun_record(args)), flush=True)
+        return 0
+    if args.arch == "pugavik":
+        print(json.dumps(pugavik_record(args)), flush=True)
         return 0
     raw = dict(SHAPES[args.shape])
     name = f"Qwen3-{args.shape.upper()} shape"

@@ -118,6 +118,12 @@ _KERNEL_API = {
     "pa_pair_embed": (I, [P, I, P, P, P, P, P, P, P, P, P, I, I, I, I, c_long, c_long, F]),
     "pa_time_conv_add": (I, [P, I, P, P, P, P, P, P, P, I, I, I, I, I]),
     "pa_stream_add_row": (I, [P, P, P, I, I]),
+    "pa_latent_expand": (I, [P, I, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, I]),
+    "pa_latent_queries": (I, [P, I, P, c_long, P, P, P, I, I, I, I, I]),
+    "pa_attn_wide_supports": (I, [I, I, I]),
+    "pa_attn_wide": (I, [P, P, P, P, P, I, P, P, P, P, c_long, I, I, I, I, I, I, I, I, I, F, P]),
+    "pa_attn_shared_workspace": (c_long, [I, I, I, I]),
+    "pa_attn_shared": (I, [P, P, P, P, P, I, P, P, P, P, c_long, P, I, I, I, I, I, I, I, F, P, I, I]),
     "pa_layer_norm_step": (I, [P, I, P, P, I, c_long, P, P, P, P, P, I, I, F]),
     "pa_stream_sum": (I, [P, I, P, P, P, P, P, I, I]),
     "pa_embed_scaled": (I, [P, I, P, P, P, I, I, I, F]),

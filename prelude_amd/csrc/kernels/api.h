@@ -260,6 +260,14 @@ int pa_latent_gather(void* stream, int dtype, const void* cache, const int* bloc
 // head, the first rot_dims of them rotated in pairs; in_token > 0: the input's tokens are that many elements apart
 int pa_rotate_pairs(void* stream, int dtype, const void* in, void* out, const float* inv_freq, const int* positions,
                     int tokens, int heads, int in_stride, int in_off, int out_stride, int out_off, int width, int rot_dims, long in_token);
+// kv [rows, heads * (d + v)] made of the latents of the cached positions (seq[i], pos[i]) -> K [page, heads, offset, d + rot]
+// (its last rot elements from the cached vector) and V [page, heads, v, offset] at slots[i]
+int pa_latent_expand(void* stream, int dtype, const void* kv, const void* cache, const int* block_table, int table_stride,
+                     const int* seq, const int* pos, const int* slots, void* k_out, void* v_out, int rows, int heads, int d, int v,
+                     int rank, int rot, int page_size);
+// q [tokens, heads, d + rot] (tokens in_token apart) -> out, packed, the first rot_dims of every head's last rot turned in pairs
+int pa_latent_queries(void* stream, int dtype, const void* q, long in_token, void* out, const float* inv_freq,
+                      const int* positions, int tokens, int heads, int d, int rot, int rot_dims);
 // y[t, h, n] = sum_k x[t, h, k] wt[h, k, n]; strides in elements
 int pa_head_linear(void* stream, int dtype, const void* x, const void* wt, void* y, int tokens, int heads, int K, int N,
                    long xs_t, long xs_h, long ys_t, long ys_h);
@@ -351,6 +359,20 @@ int pa_pair_embed(void* stream, int dtype, const int* ids, const int* positions,
 int pa_time_conv_add(void* stream, int dtype, const void* h, const float* w, float* state, const int* seq_of_token,
                      const int* cu_q, const int* state_slots, void* out, int tokens, int nseq, int channels, int taps,
                      int all_single);
+// ---- attention on the matrix cores for keys and values of any widths (attention_wide.hip), bfloat16 ----
+// q [tokens, nh, kd], K [page, nkv, offset, kd], V [page, nv, vd, offset]; nv <= nkv: key head k goes with value head k mod nv,
+// else the query heads are dealt out to the value heads in runs.  kd a multiple of 8 up to 512, vd of 4 up to 256, pages of a
+// power of two from 8 on.  pa_attn_wide: the listed sequences' portions; pa_attn_shared: single tokens, all heads over one
+// key head, in splits of split_keys keys (work: pa_attn_shared_workspace words).
+int pa_attn_wide_supports(int kd, int vd, int page_size);
+int pa_attn_wide(void* stream, const void* q, const void* kc, const void* vc, const int* block_table, int table_stride,
+                 const int* seq_ids, const int* cu_q, const int* context_lens, void* out, long out_stride, int nseq, int max_q_len,
+                 int nh, int nkv, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink);
+long pa_attn_shared_workspace(int nseq, int nh, int vd, int max_splits);
+int pa_attn_shared(void* stream, const void* q, const void* kc, const void* vc, const int* block_table, int table_stride,
+                   const int* seq_ids, const int* cu_q, const int* context_lens, void* out, long out_stride, float* work, int nseq,
+                   int nh, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink, int split_keys,
+                   int max_splits);
 // ---- layer norm around a 32-bit stream (layer_norm.hip) ----
 // residual += y (a tensor of `dtype`, or `slices` 32-bit partial sums slice_stride elements apart, or neither), then out =
 // layer norm of the row, times w plus b.  With rows: of those rows alone, the residual read only.

@@ -9,6 +9,8 @@
 //                     RMS norm of c and rotation of the shared key part (into the paged cache; c a second time
 //                     transposed, where the cache keeps that copy for the matrix-core kernel)
 //   pa_rotate_pairs   rotation of a part of every head's vector by position, pairs (2i, 2i+1)
+//   pa_latent_expand  every head's keys (with the shared rotated part) and values, made from the latents by one product, into
+//                     temporary pages; pa_latent_queries: the queries for them, their rotated part turned
 //   pa_head_linear    y[t, h, :] = W[h] x[t, h, :], a product per head
 //   pa_latent_attn    causal softmax attention over the latent cache with a learned sink per head in the
 //                     denominator; 32-bit arithmetic on the vector ALU, any sizes: the true 32-bit path and
@@ -119,6 +121,105 @@ __global__ void rotate_pairs_kernel(const T* __restrict__ in, T* __restrict__ ou
     } else {
       const int d = rot_dims + (i - half);
       dst[d] = src[d];
+    }
+  }
+}
+
+// ---- the expanded form: every head's own keys and values ----
+// kv [rows, heads * d + heads * v] (all heads' keys, then all heads' values) of cached positions -> temporary pages
+// K [page, heads, offset, d + rot], V [page, heads, v, offset]; the last rot elements of every key are the cached vector's
+// rotated part (from `cache` at the position's own page).  Rows follow each other in runs of `page_size`-aligned slots: eight
+// consecutive rows whose slots are consecutive and start at a multiple of eight leave their values in one piece.
+// Grid (rows / 8, heads).
+template <typename T>
+__global__ __launch_bounds__(128) void latent_expand_kernel(const T* __restrict__ kv, const T* __restrict__ cache,
+                                                            const int* __restrict__ block_table, int table_stride,
+                                                            const int* __restrict__ seq, const int* __restrict__ pos,
+                                                            const int* __restrict__ slots, T* __restrict__ k_out,
+                                                            T* __restrict__ v_out, int rows, int heads, int d, int v, int rank,
+                                                            int rot, int page_size) {
+  typedef T vec8 __attribute__((ext_vector_type(8)));
+  const int i0 = blockIdx.x * 8, h = blockIdx.y;
+  const int n = rows - i0 < 8 ? rows - i0 : 8;
+  const size_t width = (size_t)heads * (d + v);
+  const int dk = d + rot;
+  __shared__ int slot[8];
+  __shared__ const T* kr[8];
+  if ((int)threadIdx.x < n) {
+    const int i = i0 + threadIdx.x;
+    slot[threadIdx.x] = slots[i];
+    const int p = pos[i];
+    kr[threadIdx.x] = cache + ((size_t)block_table[(size_t)seq[i] * table_stride + p / page_size] * page_size + p % page_size) * (rank + rot) + rank;
+  }
+  __syncthreads();
+  auto key_row = [&](int r) { return k_out + (((size_t)(slot[r] / page_size) * heads + h) * page_size + slot[r] % page_size) * dk; };
+  if (d % 8 == 0 && rot % 8 == 0 && rank % 8 == 0) {        // 16-byte pieces
+    const int pieces = dk / 8;
+    for (int e = threadIdx.x; e < n * pieces; e += blockDim.x) {
+      const int r = e / pieces, j = 8 * (e % pieces);
+      const T* src = j < d ? kv + (size_t)(i0 + r) * width + (size_t)h * d + j : kr[r] + (j - d);
+      *reinterpret_cast<vec8*>(key_row(r) + j) = *reinterpret_cast<const vec8*>(src);
+    }
+  } else {
+    for (int e = threadIdx.x; e < n * dk; e += blockDim.x) {
+      const int r = e / dk, j = e % dk;
+      key_row(r)[j] = j < d ? kv[(size_t)(i0 + r) * width + (size_t)h * d + j] : kr[r][j - d];
+    }
+  }
+  const T* vsrc = kv + (size_t)i0 * width + (size_t)heads * d + (size_t)h * v;
+  bool run = n == 8 && slot[0] % 8 == 0;
+  for (int r = 1; r < n; ++r) run = run && slot[r] == slot[0] + r;   // page_size is a multiple of 8: one page
+  if (run) {
+    T* dst = v_out + (((size_t)(slot[0] / page_size) * heads + h) * v) * page_size + slot[0] % page_size;
+    for (int j = threadIdx.x; j < v; j += blockDim.x) {
+      vec8 x;
+#pragma unroll
+      for (int r = 0; r < 8; ++r) x[r] = vsrc[(size_t)r * width + j];
+      *reinterpret_cast<vec8*>(dst + (size_t)j * page_size) = x;
+    }
+  } else {
+    for (int e = threadIdx.x; e < n * v; e += blockDim.x) {
+      const int r = e / v, j = e % v;
+      v_out[(((size_t)(slot[r] / page_size) * heads + h) * v + j) * page_size + slot[r] % page_size] = vsrc[(size_t)r * width + j];
+    }
+  }
+}
+
+// q [T, heads, d + rot] (tokens in_token apart) -> out [T, heads, d + rot]: the first d elements of every head as they are,
+// the rest with its first rot_dims turned in pairs by position.  A workgroup a token.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_queries_kernel(const T* __restrict__ q, long in_token, T* __restrict__ out,
+                                                             const float* __restrict__ inv_freq, const int* __restrict__ positions,
+                                                             int heads, int d, int rot, int rot_dims) {
+  typedef T vec8 __attribute__((ext_vector_type(8)));
+  const int t = blockIdx.x, dk = d + rot;
+  const T* src = q + (size_t)t * in_token;
+  T* dst = out + (size_t)t * heads * dk;
+  const float p = (float)positions[t];
+  const int half = rot_dims / 2;
+  for (int e = threadIdx.x; e < heads * half; e += blockDim.x) {
+    const int at = (e / half) * dk + d + 2 * (e % half);
+    float s, c;
+    sincosf(p * inv_freq[e % half], &s, &c);
+    const float u = to_f32(src[at]), v = to_f32(src[at + 1]);
+    dst[at] = from_f32<T>(u * c - v * s);
+    dst[at + 1] = from_f32<T>(v * c + u * s);
+  }
+  const int rest = rot - rot_dims;
+  for (int e = threadIdx.x; e < heads * rest; e += blockDim.x) {
+    const int at = (e / rest) * dk + d + rot_dims + e % rest;
+    dst[at] = src[at];
+  }
+  if (d % 8 == 0 && dk % 8 == 0 && in_token % 8 == 0 && (reinterpret_cast<uintptr_t>(q) & 15) == 0) {
+    const int pieces = d / 8;
+    for (int e = threadIdx.x; e < heads * pieces; e += blockDim.x) {
+      const int at = (e / pieces) * dk + 8 * (e % pieces);
+      *reinterpret_cast<vec8*>(dst + at) = *reinterpret_cast<const vec8*>(src + at);
+    }
+  } else {
+    for (int e = threadIdx.x; e < heads * d; e += blockDim.x) {
+      const int at = (e / d) * dk + e % d;
+      dst[at] = src[at];
     }
   }
 }
@@ -302,6 +403,32 @@ extern "C" int pa_latent_gather(void* stream, int dtype, const void* cache, cons
              hipLaunchKernelGGL(latent_gather_kernel<T>, dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, (const T*)cache,
                                 block_table, table_stride, seq, pos, (T*)out, rows, rank, width, page_size));
   return check_launch("latent_gather");
+}
+
+extern "C" int pa_latent_expand(void* stream, int dtype, const void* kv, const void* cache, const int* block_table, int table_stride,
+                                const int* seq, const int* pos, const int* slots, void* k_out, void* v_out, int rows, int heads,
+                                int d, int v, int rank, int rot, int page_size) {
+  if (rows == 0) return 0;
+  PA_REQUIRE(rows > 0 && heads > 0 && heads <= 65535 && d > 0 && v > 0 && rank > 0 && rot >= 0 && table_stride > 0, "latent_expand: bad "
+             "sizes rows=%d heads=%d d=%d v=%d rank=%d rot=%d", rows, heads, d, v, rank, rot);
+  PA_REQUIRE(page_size > 0 && page_size % 8 == 0, "latent_expand: pages of %d tokens are no multiple of 8", page_size);
+  PA_BY_TYPE(dtype, "latent_expand",
+             hipLaunchKernelGGL(latent_expand_kernel<T>, dim3((rows + 7) / 8, heads), dim3(128), 0, (hipStream_t)stream, (const T*)kv,
+                                (const T*)cache, block_table, table_stride, seq, pos, slots, (T*)k_out, (T*)v_out, rows, heads, d, v,
+                                rank, rot, page_size));
+  return check_launch("latent_expand");
+}
+
+extern "C" int pa_latent_queries(void* stream, int dtype, const void* q, long in_token, void* out, const float* inv_freq,
+                                 const int* positions, int tokens, int heads, int d, int rot, int rot_dims) {
+  if (tokens == 0) return 0;
+  PA_REQUIRE(tokens > 0 && heads > 0 && d > 0 && rot >= 0 && rot_dims >= 0 && rot_dims <= rot && rot_dims % 2 == 0 &&
+             in_token >= (long)heads * (d + rot) && positions && (rot_dims == 0 || inv_freq),
+             "latent_queries: bad sizes tokens=%d heads=%d d=%d rot=%d of which %d turn", tokens, heads, d, rot, rot_dims);
+  PA_BY_TYPE(dtype, "latent_queries",
+             hipLaunchKernelGGL(latent_queries_kernel<T>, dim3(tokens), dim3(256), 0, (hipStream_t)stream, (const T*)q, in_token, (T*)out,
+                                inv_freq, positions, heads, d, rot, rot_dims));
+  return check_launch("latent_queries");
 }
 
 extern "C" int pa_rotate_pairs(void* stream, int dtype, const void* in, void* out, const float* inv_freq,

@@ -17,8 +17,11 @@ namespace pa {
 
 constexpr int kTalkThreads = 256;
 constexpr int kTalkWaves = kTalkThreads / kWave;
+constexpr int kTalkMaxHead = 256;                 // widest key or value head
+constexpr int kTalkPer = kTalkMaxHead / kWave;    // elements of a head a lane holds
 
-// A workgroup a token.  LDS: the normed, rotated queries [nh, hd] and the mixing matrix [nh, nh].
+// A workgroup a (token, key head c): the queries of the heads that read c, key head c and value head c; then the columns c of
+// every head's mixed query.  LDS: those queries, normed and rotated [nh / nkv, hd], and their columns of the mixing matrix.
 template <typename T>
 __global__ __launch_bounds__(kTalkThreads) void talking_prepare_kernel(
     const T* __restrict__ p, size_t stride, int q_off, int k_off, int v_off, const float* __restrict__ q_bias,
@@ -27,74 +30,81 @@ __global__ __launch_bounds__(kTalkThreads) void talking_prepare_kernel(
     const float* __restrict__ talk, const int* __restrict__ slots, T* __restrict__ q_out, T* __restrict__ k_cache,
     T* __restrict__ v_cache, int nh, int nkv, int hd, int vd, int rot, int value_norm, int page_size, float eps) {
   extern __shared__ float qs[];
-  float* ts = qs + nh * hd;
+  const int group = nh / nkv, kd = nkv * hd;
+  float* ts = qs + group * hd;                    // [group][nh]
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const size_t t = blockIdx.x;
+  const int c = blockIdx.y;
   const T* row = p + t * stride;
   const int slot = slots ? slots[t] : -1;
   const float pos = (float)positions[t];
   const size_t page = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot % page_size : 0;
-  for (int i = threadIdx.x; i < nh * nh; i += kTalkThreads) ts[i] = talk[i];
-  for (int u = wave; u < nh + 2 * nkv; u += kTalkWaves) {   // a wavefront a head
-    if (u >= nh && slot < 0) break;
-    if (u >= nh + nkv) {                                    // a value head
-      const int c = u - nh - nkv;
-      const T* src = row + v_off + (size_t)c * vd;
-      const float* b = v_bias ? v_bias + (size_t)c * vd : nullptr;
-      float inv = 1.f;
-      if (value_norm) {
-        float ss = 0.f;
-        for (int i = lane; i < vd; i += kWave) {
-          const float v = to_f32(src[i]) + (b ? b[i] : 0.f);
-          ss += v * v;
+  for (int i = threadIdx.x; i < group * nh; i += kTalkThreads) ts[i] = talk[(size_t)(i % nh) * nh + c * group + i / nh];
+  for (int u = wave; u < group + 2; u += kTalkWaves) {      // a wavefront a head; a lane holds two neighbouring elements at a time
+    if (u >= group && slot < 0) break;
+    const bool is_q = u < group, is_v = u == group + 1;
+    const int h = is_q ? c * group + u : c;
+    const int width = is_v ? vd : hd;
+    const T* src = row + (is_q ? q_off : is_v ? v_off : k_off) + (size_t)h * width;
+    const float* bias = is_q ? q_bias : is_v ? v_bias : k_bias;
+    const float* w = is_q ? q_weight : is_v ? nullptr : k_weight;
+    float x[kTalkPer];
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < kTalkPer / 2; ++e)
+#pragma unroll
+      for (int b = 0; b < 2; ++b) {
+        const int i = 2 * (lane + kWave * e) + b;
+        float v = 0.f;
+        if (i < width) {
+          v = to_f32(src[i]);
+          if (bias) v += bias[(size_t)h * width + i];
         }
-        inv = 1.0f / sqrtf(wave_sum(ss) / (float)vd + eps);
-      }
-      T* dst = v_cache + ((page * nkv + c) * vd) * page_size + off;
-      for (int i = lane; i < vd; i += kWave) dst[(size_t)i * page_size] = from_f32<T>((to_f32(src[i]) + (b ? b[i] : 0.f)) * inv);
-      continue;
-    }
-    const bool is_q = u < nh;
-    const int h = is_q ? u : u - nh;
-    const T* src = row + (is_q ? q_off : k_off) + (size_t)h * hd;
-    const float* bias = is_q ? q_bias : k_bias;
-    const float* b = bias ? bias + (size_t)h * hd : nullptr;
-    const float* w = is_q ? q_weight : k_weight;
-    float inv = 1.f;
-    if (w) {
-      float ss = 0.f;
-      for (int i = lane; i < hd; i += kWave) {
-        const float v = to_f32(src[i]) + (b ? b[i] : 0.f);
+        x[2 * e + b] = v;
         ss += v * v;
       }
-      inv = 1.0f / sqrtf(wave_sum(ss) / (float)hd + eps);
+    const bool normed = is_v ? value_norm != 0 : w != nullptr;
+    const float inv = normed ? 1.0f / sqrtf(wave_sum(ss) / (float)width + eps) : 1.0f;
+#pragma unroll
+    for (int e = 0; e < kTalkPer / 2; ++e) {
+      const int i = 2 * (lane + kWave * e);
+      if (i >= width) continue;
+      const bool two = i + 1 < width;
+      float u0 = x[2 * e] * inv, u1 = x[2 * e + 1] * inv;
+      if (w) {
+        u0 *= w[i];
+        if (two) u1 *= w[i + 1];
+      }
+      if (is_v) {
+        T* dst = v_cache + ((page * nkv + c) * vd + i) * page_size + off;
+        dst[0] = from_f32<T>(u0);
+        if (two) dst[page_size] = from_f32<T>(u1);
+        continue;
+      }
+      if (i < rot) {                                        // rot is even: the pair turns whole
+        float sn, cs;
+        sincosf(pos * inv_freq[i / 2], &sn, &cs);
+        const float v0 = u0 * cs - u1 * sn;
+        u1 = u1 * cs + u0 * sn;
+        u0 = v0;
+      }
+      if (is_q) {
+        qs[u * hd + i] = u0;
+        if (two) qs[u * hd + i + 1] = u1;
+      } else {
+        T* dst = k_cache + (page * page_size + off) * (size_t)kd + (size_t)c * hd + i;
+        dst[0] = from_f32<T>(u0);
+        if (two) dst[1] = from_f32<T>(u1);
+      }
     }
-    auto value = [&](int i) {
-      const float v = (to_f32(src[i]) + (b ? b[i] : 0.f)) * inv;
-      return w ? v * w[i] : v;
-    };
-    T* kdst = is_q ? nullptr : k_cache + (page * page_size + off) * ((size_t)nkv * hd) + (size_t)h * hd;
-    auto put = [&](int i, float v) {
-      if (is_q) qs[h * hd + i] = v;
-      else kdst[i] = from_f32<T>(v);
-    };
-    for (int i = lane; i < rot / 2; i += kWave) {           // a lane a pair
-      float s, c;
-      sincosf(pos * inv_freq[i], &s, &c);
-      const float x = value(2 * i), y = value(2 * i + 1);
-      put(2 * i, x * c - y * s);
-      put(2 * i + 1, y * c + x * s);
-    }
-    for (int i = rot + lane; i < hd; i += kWave) put(i, value(i));
   }
   __syncthreads();
-  const int group = nh / nkv, kd = nkv * hd;
-  T* dst = q_out + t * (size_t)nh * kd;
-  for (int i = threadIdx.x; i < nh * kd; i += kTalkThreads) {
-    const int h = i / kd, c = (i % kd) / hd, d = i % hd;
+  T* dst = q_out + t * (size_t)nh * kd + (size_t)c * hd;
+  for (int i = threadIdx.x; i < nh * hd; i += kTalkThreads) {
+    const int h = i / hd, d = i % hd;
     float acc = 0.f;
-    for (int g = 0; g < group; ++g) acc = fmaf(ts[h * nh + c * group + g], qs[(c * group + g) * hd + d], acc);
-    dst[i] = from_f32<T>(acc);
+    for (int g = 0; g < group; ++g) acc = fmaf(ts[g * nh + h], qs[g * hd + d], acc);
+    dst[(size_t)h * kd + d] = from_f32<T>(acc);
   }
 }
 
@@ -115,11 +125,12 @@ extern "C" int pa_talking_prepare(void* stream, int dtype, const void* p, long s
   PA_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && q_off + (long)nh * hd <= stride && k_off + (long)nkv * hd <= stride &&
              v_off + (long)nkv * vd <= stride, "talking_prepare: the columns do not fit the row of %ld", stride);
   PA_REQUIRE(!slots || (k_cache && v_cache && page_size > 0), "talking_prepare: slots without caches");
-  const size_t lds = ((size_t)nh * hd + (size_t)nh * nh) * sizeof(float);
+  PA_REQUIRE(hd <= kTalkMaxHead && vd <= kTalkMaxHead, "talking_prepare: heads of %d or values of %d are wider than %d", hd, vd, kTalkMaxHead);
+  const size_t lds = (size_t)(nh / nkv) * (hd + nh) * sizeof(float);
   PA_REQUIRE(lds <= 65536, "talking_prepare: %d heads of %d take %zu bytes of LDS, more than 65536", nh, hd, lds);
   hipStream_t st = (hipStream_t)stream;
 #define PA_TALK(T)                                                                                                              \
-  hipLaunchKernelGGL(talking_prepare_kernel<T>, dim3(tokens), dim3(kTalkThreads), lds, st, (const T*)p, (size_t)stride, q_off,   \
+  hipLaunchKernelGGL(talking_prepare_kernel<T>, dim3(tokens, nkv), dim3(kTalkThreads), lds, st, (const T*)p, (size_t)stride, q_off,   \
                      k_off, v_off, q_bias, k_bias, v_bias, q_weight, k_weight, inv_freq, positions, talk, slots, (T*)q_out,      \
                      (T*)k_cache, (T*)v_cache, nh, nkv, hd, vd, rot, value_norm, page_size, eps)
   if (dtype == kF32) PA_TALK(float);

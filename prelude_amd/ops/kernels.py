@@ -1735,7 +1735,7 @@ def qkv_prepare(p: torch.Tensor, q_off: int, k_off: int, v_off: int, q_weight: O
 
 
 MASKED_MAX_KEY, MASKED_MAX_VALUE = 4096, 256   # widest key and value of the kernel on the vector units
-TALKING_MAX_LDS = 16384                        # 32-bit words of LDS: heads * (head width + heads)
+TALKING_MAX_LDS, TALKING_MAX_HEAD = 16384, 256 # 32-bit words of LDS: a key head's query heads * (head width + heads); widest head
 
 
 def attention_masked_mfma_supported(hd: int, vd: int, page_size: int) -> bool:
@@ -2100,6 +2100,102 @@ def talking_prepare(p: torch.Tensor, q_off: int, k_off: int, v_off: int, biases,
                                            _ptr(talk), _ptr(slots), _ptr(q), _ptr(k_cache), _ptr(v_cache), t, nh, nkv, hd, vd,
                                            int(rot), 1 if value_norm else 0, page, float(eps)))
     return q
+
+
+def attention_wide_supported(kd: int, vd: int, page_size: int) -> bool:
+    """Whether ``attention_wide`` takes these widths and pages (bfloat16)."""
+    return bool(kernels().pa_attn_wide_supports(int(kd), int(vd), int(page_size)))
+
+
+SHARED_SPLIT_KEYS = (128, 256, 512, 1024, 2048, 4096)   # keys a split of a single token's context, all heads over one key head
+SHARED_SPLIT_WORKGROUPS = 1024                          # the shortest split whose launch stays within this many workgroups
+
+
+def shared_split_plan(n_seqs: int, heads: int, max_context: int, window: int, page_size: int):
+    """(keys a split, most splits a sequence) for a step of ``n_seqs`` single tokens whose contexts are at most
+    ``max_context`` tokens.  It follows the context rounded up (``decode_context_bound``), so that a step run directly and
+    one replayed from a graph are cut alike."""
+    bound = decode_context_bound(max_context, page_size)
+    tiles = -(-int(heads) // 16)
+
+    def splits(keys):
+        span = min(bound, window) if window else bound
+        return -(-span // keys) + (1 if window and bound > window else 0)
+    keys = next((k for k in SHARED_SPLIT_KEYS if n_seqs * tiles * splits(k) <= SHARED_SPLIT_WORKGROUPS), SHARED_SPLIT_KEYS[-1])
+    return keys, splits(keys)
+
+
+def attention_wide(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, group, step, window: int, scale: float,
+                   sink: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Paged causal attention of one step on the matrix cores for key and value widths of any size (``attention_wide_supported``),
+    bfloat16: q [T, nh, kd], K [pages, nkv, page, kd], V [pages, nv, vd, page] (value heads as in ``attention_masked``), a window
+    (0: none), a sink per head.  Portions are tiles of tokens; where all heads read one key head, single tokens have a kernel
+    that reads every key once for all heads.  Returns (or fills ``out``, whose rows may lie inside a wider tensor) [T, nh * vd]."""
+    _dev(q, k_cache, v_cache, sink, group.block_table)
+    t, nh, kd = q.shape
+    pages, nkv, page, _ = k_cache.shape
+    nv, vd = v_cache.shape[1], v_cache.shape[2]
+    if q.dtype != torch.bfloat16 or k_cache.dtype != q.dtype or v_cache.dtype != q.dtype or k_cache.shape[3] != kd or \
+            tuple(v_cache.shape) != (pages, nv, vd, page):
+        raise NativeError(f"attention_wide: q {tuple(q.shape)} {q.dtype} / caches {tuple(k_cache.shape)} / {tuple(v_cache.shape)}")
+    if sink is not None:
+        _check_sinks(sink, nh)
+    if out is None:
+        out = torch.empty((t, nh * vd), dtype=q.dtype, device=q.device)
+    elif out.dtype != q.dtype or tuple(out.shape) != (t, nh * vd) or out.stride(1) != 1:
+        raise NativeError(f"attention_wide: out {tuple(out.shape)} {out.dtype}")
+    args = (_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(group.block_table), group.block_table.shape[1])
+    if step.n_decode:
+        every = step.n_prefill == 0 and step.n_decode == step.num_seqs
+        ids = None if every else _ptr(step.decode_seqs)
+        if nkv == 1:
+            keys, splits = shared_split_plan(step.n_decode, nh, step.max_decode_context, window, page)
+            work = torch.empty(int(kernels().pa_attn_shared_workspace(step.n_decode, nh, vd, splits)), dtype=torch.float32, device=q.device)
+            check(kernels().pa_attn_shared(_stream(), *args, ids, _ptr(step.cu_q), _ptr(step.context_lens), out.data_ptr(), out.stride(0),
+                                           _ptr(work), step.n_decode, nh, nv, kd, vd, page, int(window), float(scale), _ptr(sink), keys,
+                                           splits))
+        else:
+            check(kernels().pa_attn_wide(_stream(), *args, ids, _ptr(step.cu_q), _ptr(step.context_lens), out.data_ptr(), out.stride(0),
+                                         step.n_decode, 1, nh, nkv, nv, kd, vd, page, int(window), float(scale), _ptr(sink)))
+    if step.n_prefill:
+        check(kernels().pa_attn_wide(_stream(), *args, _ptr(step.prefill_seqs), _ptr(step.cu_q), _ptr(step.context_lens), out.data_ptr(),
+                                     out.stride(0), step.n_prefill, int(step.max_prefill_q), nh, nkv, nv, kd, vd, page, int(window),
+                                     float(scale), _ptr(sink)))
+    return out
+
+
+def latent_expand(kv: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, seq: torch.Tensor, pos: torch.Tensor,
+                  slots: torch.Tensor, k_out: torch.Tensor, v_out: torch.Tensor, heads: int, d: int, v: int, rank: int) -> None:
+    """``kv`` [N, heads * d + heads * v] (every head's keys, then every head's values, of the cached positions (seq, pos)) into the
+    pages ``k_out`` [pages, heads, page, d + rot] and ``v_out`` [pages, heads, v, page] at ``slots``; a key's last rot elements
+    are the cached vector's (``cache`` [pages, page, rank + rot])."""
+    _dev(kv, cache, block_table, seq, pos, slots, k_out, v_out)
+    for t, name in ((block_table, "block_table"), (seq, "sequences"), (pos, "positions"), (slots, "slots")):
+        _i32(t, name)
+    page, rot = cache.shape[1], cache.shape[2] - rank
+    if tuple(kv.shape) != (seq.shape[0], heads * (d + v)) or k_out.shape[1:] != (heads, page, d + rot) or \
+            tuple(v_out.shape) != (k_out.shape[0], heads, v, page) or not (kv.dtype == cache.dtype == k_out.dtype == v_out.dtype) or \
+            pos.shape != seq.shape or slots.shape != seq.shape:
+        raise NativeError(f"latent_expand: kv {tuple(kv.shape)} / pages {tuple(k_out.shape)} / {tuple(v_out.shape)}")
+    check(kernels().pa_latent_expand(_stream(), _code(kv), _ptr(kv), _ptr(cache), _ptr(block_table), block_table.shape[1], _ptr(seq),
+                                     _ptr(pos), _ptr(slots), _ptr(k_out), _ptr(v_out), kv.shape[0], heads, d, v, rank, rot, page))
+
+
+def latent_queries(q: torch.Tensor, inv_freq: Optional[torch.Tensor], positions: torch.Tensor, d: int, rot_dims: int) -> torch.Tensor:
+    """q [T, heads, d + rot] (a token's heads may lie inside a wider row) packed, with the first ``rot_dims`` of every head's
+    last rot elements turned in pairs by position."""
+    _heads_of_rows(q, "latent_queries")
+    _dev(inv_freq, positions)
+    _f32(inv_freq, "rotary frequencies")
+    _i32(positions, "positions")
+    t, heads, dk = q.shape
+    if rot_dims and (inv_freq is None or tuple(inv_freq.shape) != (rot_dims // 2,)):
+        raise NativeError("latent_queries: rotary frequencies do not match the rotated width")
+    out = torch.empty((t, heads, dk), dtype=q.dtype, device=q.device)
+    if t:
+        check(kernels().pa_latent_queries(_stream(), _code(q), q.data_ptr(), q.stride(0), _ptr(out), _ptr(inv_freq), _ptr(positions), t,
+                                          heads, int(d), dk - int(d), int(rot_dims)))
+    return out
 
 
 # ---------------------------------------------------------------------------

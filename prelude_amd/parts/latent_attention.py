@@ -64,8 +64,8 @@ def window_plan(step, window: int, page: int, device) -> types.SimpleNamespace:
 class LatentAttention(Mixer):
     LAUNCHES = 8   # down projections, prep, query up, absorb, rotation, attention, value up, output
     GRAPH_SAFE_PORTIONS = True   # launches follow the step's shape alone (the expanded form below runs in direct steps only)
-    # A step that brings this many tokens or more (and is run directly, in bfloat16, by a mixer without a rotated part
-    # whose head sizes the matrix-core attention takes) attends in the expanded form: the keys and values of every
+    # A step that brings this many tokens or more (and is run directly, in bfloat16, with head sizes the matrix-core
+    # attention takes) attends in the expanded form: the keys and values of every
     # head are made from the latents its sequences can see, by one product, into temporary pages, and the queries
     # attend to them as they stand.  The form above moves both maps to the query side and pays rank + rot
     # multiplications a (query, key, head) where this one pays head_dim and value_dim; what it costs instead is the
@@ -148,7 +148,7 @@ class LatentAttention(Mixer):
         self.uv_t = K.GroupedWeight(tensors["uv"].reshape(nh, v, rank))
         self.c_norm = tensors["dkv.norm"]
         self.sinks = tensors["sink"] if self.sink else None
-        if self.rot_dim == 0 and not self.sink and tensors["uk"].dtype == torch.bfloat16:
+        if tensors["uk"].dtype == torch.bfloat16:
             # for the expanded form: every head's keys, then every head's values, from a latent by one product
             self.w_ukv = K.prepare_weight(torch.cat([tensors["uk"], tensors["uv"]], dim=0).contiguous())
         rows = [tensors["dq" if self.q_rank else "q"], tensors["dkv"]] + ([tensors["g"]] if self.output_gate else [])
@@ -158,10 +158,11 @@ class LatentAttention(Mixer):
         self.w_down = K.prepare_weight(self.input_rows(tensors).contiguous())
         self.w_o = K.prepare_weight(tensors["o"])
 
-    def _expands(self, x, step, cache, write_cache) -> bool:
+    def _expands(self, x, step, cache, write_cache, out) -> bool:
         if not (self.w_ukv is not None and write_cache and x.dtype == torch.bfloat16 and getattr(step, "graph", None) is None
                 and step.n_prefill > 0 and step.num_tokens >= self.EXPAND_FROM_TOKENS and len(step.starts) == step.num_seqs
-                and K.attention_masked_mfma_supported(self.head_dim, self.value_dim, cache.latent.shape[1])):
+                and self.scale > 0 and K.attention_wide_supported(self.head_dim + self.rot_dim, self.value_dim, cache.latent.shape[1])
+                and (out is None or (out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0))):
             return False
         # not where the latents to expand outnumber the step's tokens several times (many single tokens, each with a
         # window behind it, beside a short portion)
@@ -171,16 +172,19 @@ class LatentAttention(Mixer):
 
     def _expanded(self, q, step, cache, g, out=None):
         """The heads' outputs side by side [T, heads * value_dim] from keys and values made of the visible latents."""
-        nh, d, v, rank = self.num_heads, self.head_dim, self.value_dim, self.kv_rank
+        nh, d, r, v, rank = self.num_heads, self.head_dim, self.rot_dim, self.value_dim, self.kv_rank
         page = cache.latent.shape[1]
         plan = window_plan(step, self.window, page, q.device)
         kv = K.linear(K.latent_gather(cache.latent, g.block_table, plan.seq, plan.pos, rank), self.w_ukv)
-        # zeroed: the places of a sequence's last page behind its last token are multiplied by weights of zero
-        k_tmp = torch.zeros((plan.pages, nh, page, d), dtype=q.dtype, device=q.device)
+        # values zeroed: the places of a sequence's last page behind its last token are multiplied by weights of zero (the
+        # keys' scores are masked whatever they are)
+        k_tmp = torch.empty((plan.pages, nh, page, d + r), dtype=q.dtype, device=q.device)
         v_tmp = torch.zeros((plan.pages, nh, v, page), dtype=q.dtype, device=q.device)
-        K.qkv_rope_prepare(kv, 0, 0, nh * d, None, plan.pos, plan.slots, k_tmp, v_tmp, 0, nh, nh, d, v, 0, False)
-        return K.attention_masked(q.contiguous(), k_tmp, v_tmp, types.SimpleNamespace(block_table=plan.table), step, self.window, 0,
-                                  self.scale, out=out)
+        K.latent_expand(kv, cache.latent, g.block_table, plan.seq, plan.pos, plan.slots, k_tmp, v_tmp, nh, d, v, rank)
+        if r or not q.is_contiguous():
+            q = K.latent_queries(q, self.rope.inv_freq if self.rope is not None else None, step.positions, d, self.rotary_dim)
+        return K.attention_wide(q, k_tmp, v_tmp, types.SimpleNamespace(block_table=plan.table), step, self.window, self.scale,
+                                sink=self.sinks, out=out)
 
     def mix(self, x, p, off, step, cache, write_cache, out=None, out_scale=1.0):
         """From the product ``p`` of its input (its columns start at ``off``) to the heads' outputs side by side
@@ -200,7 +204,7 @@ class LatentAttention(Mixer):
             q = K.linear(cq, self.w_uq).view(-1, nh, d + r)
         else:
             q = p[:, off: off + nh * (d + r)].unflatten(1, (nh, d + r))
-        if self._expands(x, step, cache, write_cache):
+        if self._expands(x, step, cache, write_cache, out):
             o = self._expanded(q, step, cache, g, out)
         else:
             ql = torch.empty((q.shape[0], nh, rank + r), dtype=q.dtype, device=q.device)

@@ -24,7 +24,7 @@ from .base import MATRIX, NORM, VECTOR, Mixer, PartError, TensorReq, register_pa
 
 @register_part("mixer", "talking_heads_attention")
 class TalkingHeadsAttention(Mixer):
-    LAUNCHES = 4   # merged projection, norms + rotation + mixing + cache write, attention, output projection
+    LAUNCHES = 5   # merged projection, norms + rotation + mixing + cache write, attention, its merge, output projection
     GRAPH_SAFE_PORTIONS = True
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, scale: float,
@@ -35,7 +35,7 @@ class TalkingHeadsAttention(Mixer):
         if head_dim < 1 or num_kv_heads * head_dim > K.MASKED_MAX_KEY or not 1 <= value_dim <= K.MASKED_MAX_VALUE:
             raise PartError(f"talking_heads_attention: {num_kv_heads} keys of {head_dim} side by side (at most {K.MASKED_MAX_KEY}) or a "
                             f"value width of {value_dim} (at most {K.MASKED_MAX_VALUE}) is outside what the kernels take")
-        if num_heads * (head_dim + num_heads) > K.TALKING_MAX_LDS:
+        if num_heads // num_kv_heads * (head_dim + num_heads) > K.TALKING_MAX_LDS or max(head_dim, value_dim) > K.TALKING_MAX_HEAD:
             raise PartError(f"talking_heads_attention: {num_heads} heads of {head_dim} do not fit the kernel that mixes them")
         if sink not in (None, "learned"):
             raise PartError(f"talking_heads_attention: sink {sink!r} is not one of None, 'learned'")
@@ -99,6 +99,10 @@ class TalkingHeadsAttention(Mixer):
         self.w_in = K.prepare_weight(self.input_rows(tensors).contiguous())
         self.w_o = K.prepare_weight(tensors["o"])
 
+    def on_matrix_cores(self, q, cache, out) -> bool:
+        return (q.dtype == torch.bfloat16 and self.scale > 0 and K.attention_wide_supported(self.nk, self.value_dim, cache.k.shape[2])
+                and (out is None or (out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0)))
+
     def mix(self, x, p, off, step, cache, write_cache, out=None, out_scale=1.0):
         """From the product ``p`` of its input (its columns start at ``off``) to the heads' outputs side by side
         [T, heads * value_dim], times ``out_scale``, into ``out`` when given."""
@@ -109,6 +113,8 @@ class TalkingHeadsAttention(Mixer):
                               self.rope.inv_freq if self.rope is not None else None, step.positions, self.talk, g.slots, cache.k,
                               cache.v, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim, self.rotary_dim,
                               self.value_norm, self.norm_eps)
+        if self.on_matrix_cores(q, cache, out) and out_scale == 1.0:
+            return K.attention_wide(q, cache.k, cache.v, g, step, self.window, self.scale, sink=self.sinks, out=out)
         return K.attention_masked(q, cache.k, cache.v, g, step, self.window, 0, self.scale, sink=self.sinks, out=out,
                                   out_scale=out_scale)
 
