@@ -3,8 +3,8 @@
 // `nv` value heads (fewer value heads than key heads: key head k goes with value head k mod nv; more: the query heads are
 // dealt out to them in runs as to the key heads), an optional window and an optional sink per head.  bfloat16 storage,
 // 32-bit scores, sums and softmax.  The inner arithmetic and its operand layout are those of attention_mfma_core.h; the
-// kernels are compiled for bounds of the widths, and chunks beyond the actual ones are skipped by branches that are the
-// same for the whole launch.
+// kernels are compiled for bounds of the widths; what lies between a width and its bound takes part in the products as
+// zeros (a branch around it would end a basic block, and operands could no longer be asked for ahead of their use).
 //
 //   attn_wide_kernel     portions of several tokens.  A workgroup of eight wavefronts owns a tile of 64 * QT tokens of one
 //                        head.  Blocks of 64 keys go through LDS (asked for a block ahead); wavefront w works on the tokens
@@ -72,7 +72,7 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
   const int* table = a.block_table + (size_t)seq * a.table_stride;
   const int kvh = h / (a.nh / a.nkv), vh = a.value_head(h);
   const int start = a.context_lens[seq] - q_len, window = a.window;
-  const int nks = (a.kd + 31) / 32, nts = (a.vd + 15) / 16, cpk = a.kd / 8;
+  const int cpk = a.kd / 8;
   const int shift = a.page_shift, mask = (1 << shift) - 1;
 
   // what the workgroup stages, and what this wavefront's tokens see
@@ -100,11 +100,10 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
   }
   HeadState<VDM> st[QT];
 
-  // columns of K between kd and the next multiple of 32 and rows of V^T between vd and the next multiple of 16 take part in
-  // the products: they hold zeros throughout
-  const int pad = 32 * nks - a.kd;
+  // columns of K from kd and rows of V^T from vd on hold zeros throughout
+  const int pad = KDM - a.kd;
   for (int i = tid; i < NBUF * kWideKeys * pad; i += kWideThreads) lk[(i / pad) * L::KROW + a.kd + i % pad] = (bf16)0.f;
-  const int vpad = 16 * nts - a.vd;
+  const int vpad = VDM - a.vd;
   for (int i = tid; i < NBUF * vpad * kWideKeys; i += kWideThreads) {
     const int b = i / (vpad * kWideKeys), e = i % (vpad * kWideKeys);
     lv[(b * VDM + a.vd + e / kWideKeys) * L::VROW + e % kWideKeys] = (bf16)0.f;
@@ -137,15 +136,14 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
     vpage = table[p];
   };
   auto load = [&]() {
+    // (no load stands under a branch: pieces and rows that do not exist are read from ones that do and not stored)
 #pragma unroll
     for (int i = 0; i < NK; ++i)
-      if (kon[i])
-        kr[i] = *reinterpret_cast<const bf16x8*>(
-            a.kc + ((((size_t)kpage[i] * a.nkv + kvh) << shift) + ((at + kkey[i]) & mask)) * a.kd + kcol[i]);
+      kr[i] = *reinterpret_cast<const bf16x8*>(a.kc + ((((size_t)kpage[i] * a.nkv + kvh) << shift) + ((at + kkey[i]) & mask)) * a.kd + kcol[i]);
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int d = 64 * i + vd_row;
-      if (d < a.vd) vr[i] = *reinterpret_cast<const bf16x8*>(a.vc + ((((size_t)vpage * a.nv + vh) * a.vd + d) << shift) + ((at + v8) & mask));
+      const int d = 64 * i + vd_row < a.vd ? 64 * i + vd_row : a.vd - 1;
+      vr[i] = *reinterpret_cast<const bf16x8*>(a.vc + ((((size_t)vpage * a.nv + vh) * a.vd + d) << shift) + ((at + v8) & mask));
     }
   };
   auto store = [&](int buf) {
@@ -172,14 +170,12 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
       for (int j = 0; j < QT; ++j) acc[t][j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
-      if (ks < nks) {
-        const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(kb + 32 * ks);
-        const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(kb + 16 * L::KROW + 32 * ks);
+      const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(kb + 32 * ks);
+      const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(kb + 16 * L::KROW + 32 * ks);
 #pragma unroll
-        for (int j = 0; j < QT; ++j) {
-          acc[0][j] = mfma16(k0, qf[j][ks], acc[0][j]);
-          acc[1][j] = mfma16(k1, qf[j][ks], acc[1][j]);
-        }
+      for (int j = 0; j < QT; ++j) {
+        acc[0][j] = mfma16(k0, qf[j][ks], acc[0][j]);
+        acc[1][j] = mfma16(k1, qf[j][ks], acc[1][j]);
       }
     }
     const bool masked = key0 < all_lo || key0 + 32 > all_hi;
@@ -214,12 +210,11 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
     for (int j = 0; j < QT; ++j) st[j].l = mfma16(ones, pb[j], st[j].l);
     const bf16* vb = lv + (buf * VDM + r) * L::VROW + 32 * half + 8 * g;
 #pragma unroll
-    for (int t = 0; t < OT; ++t)
-      if (t < nts) {
-        const bf16x8 va = *reinterpret_cast<const bf16x8*>(vb + 16 * t * L::VROW);
+    for (int t = 0; t < OT; ++t) {
+      const bf16x8 va = *reinterpret_cast<const bf16x8*>(vb + 16 * t * L::VROW);
 #pragma unroll
-        for (int j = 0; j < QT; ++j) st[j].o[t] = mfma16(va, pb[j], st[j].o[t]);
-      }
+      for (int j = 0; j < QT; ++j) st[j].o[t] = mfma16(va, pb[j], st[j].o[t]);
+    }
   };
 
   int key0 = (wg_lo / kWideKeys) * kWideKeys;
@@ -297,15 +292,21 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
 }
 
 // ---- single tokens, all heads over one key head ------------------------------------------------------------------------
-constexpr int kSharedWaves = 4;
+constexpr int kSharedWaves = 8;
+constexpr int kSharedBlock = 128;   // keys a block: a wavefront a tile of 16 of them
 
-// Grid (tiles of 16 heads, splits, sequences).
+// Grid (tiles of 16 heads, splits, sequences).  A block's scores are eight tiles of 16 keys x 16 heads, one a wavefront; they
+// share one reference maximum per head through LDS, and their probabilities lie in LDS as the operands of the second
+// product.  That product's units, (value head, 32 keys), are dealt out to the wavefronts; the V^T of a wavefront's first two
+// units is asked for together with the keys, so that a short context is one trip to memory.
 template <int KDM, int VDM>
 __global__ __launch_bounds__(kSharedWaves* kWave) void attn_shared_kernel(WideArgs a, float* __restrict__ part_o,
                                                                          float* __restrict__ part_ml, int split_keys, int max_splits) {
   constexpr int KS = KDM / 32, OT = VDM / 16;
   extern __shared__ float lds_o[];                    // [waves][16 heads][vd + 1]
-  __shared__ float lds_ml[kSharedWaves][16][2];
+  __shared__ float lds_max[kSharedWaves][16];
+  __shared__ float lds_l[4][16];
+  __shared__ __align__(16) bf16 lds_p[kSharedBlock / 32][16][32 + 8];
   const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave;
   const int g = lane / 16, r = lane % 16;
   const int seq = a.seq_ids ? a.seq_ids[blockIdx.z] : (int)blockIdx.z;
@@ -320,127 +321,129 @@ __global__ __launch_bounds__(kSharedWaves* kWave) void attn_shared_kernel(WideAr
   const int klo = s0 > lo ? s0 : lo, khi = s0 + split_keys < ctx ? s0 + split_keys : ctx;   // never empty
   const int* table = a.block_table + (size_t)seq * a.table_stride;
   const int shift = a.page_shift, mask = (1 << shift) - 1;
-  const int nks = (a.kd + 31) / 32, nts = (a.vd + 15) / 16;
   const int head0 = blockIdx.x * 16;
   const int heads = a.nh - head0 < 16 ? a.nh - head0 : 16;
   const int my_head = head0 + (r < heads ? r : heads - 1);
   const int my_vh = my_head / (a.nh / a.nv);
-  const int vh0 = head0 / (a.nh / a.nv), vh1 = (head0 + heads - 1) / (a.nh / a.nv);
+  const int vh0 = head0 / (a.nh / a.nv);
+  const int units = 4 * ((head0 + heads - 1) / (a.nh / a.nv) - vh0 + 1);
 
+  // queries as they are up to kd and zeros from there on: what the keys' loads bring beyond kd does not matter
   bf16x8 qf[KS];
   const bf16* qrow = a.q + ((size_t)row * a.nh + my_head) * a.kd;
 #pragma unroll
-  for (int ks = 0; ks < KS; ++ks) qf[ks] = (32 * ks + 8 * g < a.kd) ? *reinterpret_cast<const bf16x8*>(qrow + 32 * ks + 8 * g) : zero8();
-  HeadState<VDM> st;
-  const float c = a.sm.c, over = kLazyLog2 / c;
-  for (int key0 = s0 + 32 * wave; key0 < khi; key0 += 32 * kSharedWaves) {
-    if (key0 + 32 <= klo) continue;
-    const bf16* krow[2];
-    const bf16* vrow[2];     // the value head 0 of the page of each run of four keys
+  for (int ks = 0; ks < KS; ++ks) {
+    const int at = 32 * ks + 8 * g;
+    const bf16x8 x = *reinterpret_cast<const bf16x8*>(qrow + (at < a.kd ? at : 0));
+    qf[ks] = at < a.kd ? x : zero8();
+  }
+  f32x4 o[OT], l{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int t = 0; t < 2; ++t) {
-      int key = key0 + 8 * (r / 4) + 4 * t + (r % 4);
-      key = key < klo ? klo : (key >= khi ? khi - 1 : key);
-      krow[t] = a.kc + (((size_t)table[key >> shift] << shift) + (key & mask)) * a.kd + 8 * g;
-      int ck = key0 + 8 * g + 4 * t;
-      if (ck + 3 < klo) ck = klo & ~3;
-      if (ck >= khi) ck = (khi - 1) & ~3;
-      vrow[t] = a.vc + ((((size_t)table[ck >> shift] * a.nv) * a.vd) << shift) + (ck & mask);
+  for (int t = 0; t < OT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float ref = -INFINITY;                              // the column's largest score so far, the same in every wavefront
+  const float c = a.sm.c;
+  for (int b0 = s0; b0 < khi; b0 += kSharedBlock) {
+    if (b0 + kSharedBlock <= klo) continue;
+    const int step0 = b0 + 32 * (wave / 2), tt = wave % 2;
+    // row r of the tile is key 8 (r / 4) + 4 tt + r % 4 of its 32
+    int key = step0 + 8 * (r / 4) + 4 * tt + (r % 4);
+    key = key < klo ? klo : (key >= khi ? khi - 1 : key);
+    const bf16* krow = a.kc + (((size_t)table[key >> shift] << shift) + (key & mask)) * a.kd;
+    bf16x8 kf[KS];
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int at = 32 * ks + 8 * g;
+      kf[ks] = *reinterpret_cast<const bf16x8*>(krow + (at < a.kd ? at : 0));
     }
-    bf16x8 kf[2][KS];
+    // the eight keys 8g .. of unit u's 32, of its value head: one 16-byte piece (pages hold eight keys or more)
+    auto load_values = [&](int u, bf16x8* va) {
+      int ck = b0 + 32 * (u % 4) + 8 * g;
+      if (ck + 7 < klo) ck = klo & ~7;
+      if (ck >= khi) ck = (khi - 1) & ~7;
+      const bf16* v = a.vc + ((((size_t)table[ck >> shift] * a.nv + vh0 + u / 4) * a.vd) << shift) + (ck & mask);
 #pragma unroll
-    for (int t = 0; t < 2; ++t)
-#pragma unroll
-      for (int ks = 0; ks < KS; ++ks)
-        if (ks < nks) kf[t][ks] = (32 * ks + 8 * g < a.kd) ? *reinterpret_cast<const bf16x8*>(krow[t] + 32 * ks) : zero8();
-    const bool joined = shift >= 3 && __all(vrow[1] == vrow[0] + 4);
-    bf16x8 va[OT];
-    auto load_values = [&](int vh) {
-#pragma unroll
-      for (int t = 0; t < OT; ++t)
-        if (t < nts) {
-          const int d = 16 * t + r < a.vd ? 16 * t + r : a.vd - 1;    // rows past the value's width are not written out
-          const size_t off = ((size_t)vh * a.vd + d) << shift;
-          if (joined) {
-            va[t] = *reinterpret_cast<const bf16x8*>(vrow[0] + off);
-          } else {
-            union {
-              bf16x8 v8;
-              short4_t h[2];
-            } u;
-            u.h[0] = *reinterpret_cast<const short4_t*>(vrow[0] + off);
-            u.h[1] = *reinterpret_cast<const short4_t*>(vrow[1] + off);
-            va[t] = u.v8;
-          }
-        }
-    };
-    load_values(vh0);
-    f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
-#pragma unroll
-    for (int ks = 0; ks < KS; ++ks)
-      if (ks < nks) {
-        acc[0] = mfma16(kf[0][ks], qf[ks], acc[0]);
-        acc[1] = mfma16(kf[1][ks], qf[ks], acc[1]);
+      for (int t = 0; t < OT; ++t) {
+        const int d = 16 * t + r < a.vd ? 16 * t + r : a.vd - 1;      // rows past the value's width are not written out
+        va[t] = *reinterpret_cast<const bf16x8*>(v + ((size_t)d << shift));
       }
-    float s[8];
+    };
+    const int u0 = wave < units ? wave : units - 1, u1 = wave + kSharedWaves < units ? wave + kSharedWaves : units - 1;
+    bf16x8 va0[OT], va1[OT];
+    load_values(u0, va0);
+    load_values(u1, va1);
+    f32x4 acc{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const int key = key0 + 8 * g + i;
-      s[i] = (key >= klo && key < khi) ? acc[i / 4][i % 4] : -INFINITY;
+    for (int ks = 0; ks < KS; ++ks) acc = mfma16(kf[ks], qf[ks], acc);
+    float s[4], mx = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int k = step0 + 8 * g + 4 * tt + i;
+      s[i] = (k >= klo && k < khi) ? acc[i] : -INFINITY;
+      mx = fmaxf(mx, s[i]);
     }
-    float mx = s[0];
+    mx = xor_max16_32(mx);
+    if (g == 0) lds_max[wave][r] = mx;
+    __syncthreads();
+    float m_new = ref;
 #pragma unroll
-    for (int i = 1; i < 8; ++i) mx = fmaxf(mx, s[i]);
-    if (__any(mx > st.lim)) {
-      asm volatile("" ::: "memory");
-      move_reference<VDM>(st, mx, c, over);
+    for (int w = 0; w < kSharedWaves; ++w) m_new = fmaxf(m_new, lds_max[w][r]);   // finite: a block that is worked on has a visible key
+    const float alpha = ref == -INFINITY ? 1.0f : __builtin_amdgcn_exp2f((ref - m_new) * c);   // the first block rescales nothing
+    ref = m_new;
+    bf16x4 p4;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) p4[i] = (bf16)__builtin_amdgcn_exp2f((s[i] - m_new) * c);
+    *reinterpret_cast<bf16x4*>(&lds_p[wave / 2][r][8 * g + 4 * tt]) = p4;
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < OT; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o[t][i] *= alpha;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) l[i] *= alpha;
+    if (wave < 4) l = mfma16(ones8(), *reinterpret_cast<const bf16x8*>(&lds_p[wave][r][8 * g]), l);
+    auto add_unit = [&](int u, const bf16x8* va) {
+      const bf16x8 pb = *reinterpret_cast<const bf16x8*>(&lds_p[u % 4][r][8 * g]);
+      bf16x8 pm;   // the probabilities of the heads that read the unit's value head
+#pragma unroll
+      for (int i = 0; i < 8; ++i) pm[i] = my_vh == vh0 + u / 4 ? pb[i] : (bf16)0.f;
+#pragma unroll
+      for (int t = 0; t < OT; ++t) o[t] = mfma16(va[t], pm, o[t]);
+    };
+    if (wave < units) add_unit(u0, va0);
+    if (wave + kSharedWaves < units) add_unit(u1, va1);
+    for (int u = wave + 2 * kSharedWaves; u < units; u += kSharedWaves) {
+      load_values(u, va0);
+      add_unit(u, va0);
     }
-    const bf16x8 pb = probabilities(s, c, st.shift);
-    st.l = mfma16(ones8(), pb, st.l);
-    for (int vh = vh0; vh <= vh1; ++vh) {
-      bf16x8 pm;   // the probabilities of the heads that read this value head
-#pragma unroll
-      for (int i = 0; i < 8; ++i) pm[i] = my_vh == vh ? pb[i] : (bf16)0.f;
-#pragma unroll
-      for (int t = 0; t < OT; ++t)
-        if (t < nts) st.o[t] = mfma16(va[t], pm, st.o[t]);
-      if (vh < vh1) load_values(vh + 1);
-    }
+    __syncthreads();                                  // the probabilities have been read
   }
   const int ostride = a.vd + 1;
-  if (g == 0) {
-    lds_ml[wave][r][0] = st.reference();
-    lds_ml[wave][r][1] = st.l[0];
-  }
+  if (wave < 4 && g == 0) lds_l[wave][r] = l[0];
 #pragma unroll
   for (int t = 0; t < OT; ++t)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int d = 16 * t + 4 * g + i;
-      if (d < a.vd) lds_o[((size_t)wave * 16 + r) * ostride + d] = st.o[t][i];
+      if (d < a.vd) lds_o[((size_t)wave * 16 + r) * ostride + d] = o[t][i];
     }
+  if (wave == 0 && g == 0) lds_max[0][r] = ref;
   __syncthreads();
   for (int e = tid; e < heads * a.vd; e += kSharedWaves * kWave) {
     const int j = e / a.vd, d = e % a.vd;
-    float mm = lds_ml[0][j][0];
+    float ov = 0.f;
 #pragma unroll
-    for (int v = 1; v < kSharedWaves; ++v) mm = fmaxf(mm, lds_ml[v][j][0]);
-    float o = 0.f, l = 0.f;
-#pragma unroll
-    for (int v = 0; v < kSharedWaves; ++v) {   // in the order of the wavefronts
-      const float f = lds_ml[v][j][0] == -INFINITY ? 0.f : exp2f(lds_ml[v][j][0] - mm);
-      o += lds_o[((size_t)v * 16 + j) * ostride + d] * f;
-      l += lds_ml[v][j][1] * f;
-    }
+    for (int v = 0; v < kSharedWaves; ++v) ov += lds_o[((size_t)v * 16 + j) * ostride + d];   // in the order of the wavefronts
+    const float lv = (lds_l[0][j] + lds_l[1][j]) + (lds_l[2][j] + lds_l[3][j]);
+    const float mm = lds_max[0][j] * c;               // the exponent's reference
     const int h = head0 + j;
     if (nsplit == 1) {
-      a.out[(size_t)row * a.out_stride + (size_t)h * a.vd + d] = (bf16)(o / (l + a.sm.sink_term(h, mm)));
+      a.out[(size_t)row * a.out_stride + (size_t)h * a.vd + d] = (bf16)(ov / (lv + a.sm.sink_term(h, mm)));
     } else {
       const size_t slot = ((size_t)blockIdx.z * a.nh + h) * max_splits + blockIdx.y;
-      part_o[slot * a.vd + d] = o;
+      part_o[slot * a.vd + d] = ov;
       if (d == 0) {
         part_ml[slot * 2] = mm;
-        part_ml[slot * 2 + 1] = l;
+        part_ml[slot * 2 + 1] = lv;
       }
     }
   }
@@ -569,7 +572,7 @@ extern "C" int pa_attn_shared(void* stream, const void* q, const void* kc, const
                               int split_keys, int max_splits) {
   if (nseq == 0) return 0;
   if (int rc = wide_check("attn_shared", nseq, nh, 1, nv, kd, vd, page_size, table_stride, window, scale, out_stride, q, kc, vc, out)) return rc;
-  PA_REQUIRE(split_keys > 0 && split_keys % 32 == 0 && max_splits > 0 && max_splits <= 65535 && nseq <= 65535 && work,
+  PA_REQUIRE(split_keys > 0 && split_keys % kSharedBlock == 0 && max_splits > 0 && max_splits <= 65535 && nseq <= 65535 && work,
              "attn_shared: splits of %d keys, %d at most", split_keys, max_splits);
   WideArgs a{(const bf16*)q, (const bf16*)kc, (const bf16*)vc, block_table, table_stride, seq_ids, cu_q, context_lens, (bf16*)out,
              (size_t)out_stride, nh, 1, nv, kd, vd, __builtin_ctz(page_size), window, score_map(scale, 0.f, sink)};

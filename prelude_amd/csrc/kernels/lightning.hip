@@ -275,8 +275,16 @@ __global__ __launch_bounds__(kLaThreads, 2) void lightning_attn_kernel(
   }
 }
 
-// alpha = sigmoid(z)^(1 / tau), z = w . low + bias: log sigmoid(z) = min(z, 0) - log(1 + e^-|z|), which loses nothing at either end.
+// alpha = sigmoid(z)^(1 / tau), z = w . low + bias: log sigmoid(z) = min(z, 0) - log(1 + e^-|z|), which loses nothing at either
+// end.  Behind bfloat16 projections the hardware's exponential and logarithm serve (log(1 + e) is then off by the rounding
+// of 1 + e, which is that of alpha itself).
+template <typename T>
 __device__ __forceinline__ float gla_alpha(float z, float inv_tau) {
+  if (sizeof(T) == 2) {
+    constexpr float kLog2 = 1.4426950408889634f;
+    const float e = __builtin_amdgcn_exp2f(-fabsf(z) * kLog2);
+    return __builtin_amdgcn_exp2f((fminf(z, 0.f) * kLog2 - __builtin_amdgcn_logf(1.0f + e)) * inv_tau);
+  }
   return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);
 }
 // One channel's row of A2 against a token's low-rank vector in LDS, in ascending order.
@@ -295,17 +303,44 @@ __device__ __forceinline__ float gla_dot(const T* __restrict__ w, const float* l
   return acc;
 }
 
-// alpha [tokens, channels].  Grid (tokens, runs of 256 channels); LDS: the token's low-rank vector.
+// alpha [tokens, channels].  Grid (runs of kGlaTokens tokens, runs of 256 channels); LDS: the tokens' low-rank vectors.  A
+// thread reads its channel's row of A2 once for all of them (the sums in gla_dot's order).
+constexpr int kGlaTokens = 8;
+
 template <typename T>
 __global__ __launch_bounds__(256) void gla_decay_kernel(const T* __restrict__ p, long ld, int low_off, const T* __restrict__ a2,
-                                                        const float* __restrict__ bias, float* __restrict__ alpha, int channels,
-                                                        int rank, float inv_tau) {
+                                                        const float* __restrict__ bias, float* __restrict__ alpha, int tokens,
+                                                        int channels, int rank, float inv_tau) {
   extern __shared__ float low[];
-  const size_t t = blockIdx.x;
-  for (int i = threadIdx.x; i < rank; i += 256) low[i] = to_f32(p[t * ld + low_off + i]);
+  const int t0 = blockIdx.x * kGlaTokens;
+  for (int i = threadIdx.x; i < kGlaTokens * rank; i += 256) {
+    const int t = t0 + i / rank < tokens ? t0 + i / rank : tokens - 1;
+    low[i] = to_f32(p[(size_t)t * ld + low_off + i % rank]);
+  }
   __syncthreads();
   const int c = blockIdx.y * 256 + threadIdx.x;
-  if (c < channels) alpha[t * channels + c] = gla_alpha(gla_dot(a2 + (size_t)c * rank, low, rank) + bias[c], inv_tau);
+  if (c >= channels) return;
+  const T* w = a2 + (size_t)c * rank;
+  float acc[kGlaTokens] = {};
+  if (sizeof(T) == 2 && rank % 8 == 0) {
+    for (int i = 0; i < rank; i += 8) {
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(w + i);
+#pragma unroll
+      for (int k = 0; k < kGlaTokens; ++k)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[k] = fmaf((float)v[e], low[k * rank + i + e], acc[k]);
+    }
+  } else {
+    for (int i = 0; i < rank; ++i) {
+      const float v = to_f32(w[i]);
+#pragma unroll
+      for (int k = 0; k < kGlaTokens; ++k) acc[k] = fmaf(v, low[k * rank + i], acc[k]);
+    }
+  }
+  const float b = bias[c];
+#pragma unroll
+  for (int k = 0; k < kGlaTokens; ++k)
+    if (t0 + k < tokens) alpha[(size_t)(t0 + k) * channels + c] = gla_alpha<T>(acc[k] + b, inv_tau);
 }
 
 // Sequences of exactly one token (a decode step): the same sums as the kernel above gives for them, bit for bit, in a
@@ -350,7 +385,7 @@ __global__ __launch_bounds__(kLaThreads) void lightning_step_kernel(
     __syncthreads();
     if ((int)threadIdx.x < 4 * R) {
       const int c = h * dim + ((int)threadIdx.x < dim ? (int)threadIdx.x : dim - 1);
-      as[threadIdx.x] = gla_alpha(gla_dot(a2 + (size_t)c * rank, low, rank) + decay[c], inv_tau);
+      as[threadIdx.x] = gla_alpha<T>(gla_dot(a2 + (size_t)c * rank, low, rank) + decay[c], inv_tau);
     }
   }
   __syncthreads();
@@ -535,7 +570,7 @@ extern "C" int pa_lightning_attn_chunked(void* stream, int dtype, const void* qk
 
 // ---- gated linear attention ------------------------------------------------------------------------------------------
 static int gla_low_check(const char* what, long ld, int low_off, int rank) {
-  PA_REQUIRE(rank > 0 && rank <= 8192 && low_off >= 0 && low_off + (long)rank <= ld, "%s: a low-rank vector of %d at column %d of a row of %ld",
+  PA_REQUIRE(rank > 0 && rank <= 2048 && low_off >= 0 && low_off + (long)rank <= ld, "%s: a low-rank vector of %d at column %d of a row of %ld",
              what, rank, low_off, ld);
   return 0;
 }
@@ -546,14 +581,15 @@ extern "C" int pa_gla_decay(void* stream, int dtype, const void* p, long ld, int
   PA_REQUIRE(tokens > 0 && channels > 0 && tau > 0.f && (channels + 255) / 256 <= 65535, "gla_decay: bad sizes tokens=%d channels=%d tau=%g",
              tokens, channels, (double)tau);
   if (int rc = gla_low_check("gla_decay", ld, low_off, rank)) return rc;
-  dim3 grid(tokens, (channels + 255) / 256);
+  dim3 grid((tokens + kGlaTokens - 1) / kGlaTokens, (channels + 255) / 256);
+  const size_t lds = (size_t)kGlaTokens * rank * sizeof(float);
   hipStream_t st = (hipStream_t)stream;
   if (dtype == kF32)
-    hipLaunchKernelGGL(gla_decay_kernel<float>, grid, dim3(256), rank * sizeof(float), st, (const float*)p, ld, low_off,
-                       (const float*)a2, bias, alpha, channels, rank, 1.f / tau);
+    hipLaunchKernelGGL(gla_decay_kernel<float>, grid, dim3(256), lds, st, (const float*)p, ld, low_off,
+                       (const float*)a2, bias, alpha, tokens, channels, rank, 1.f / tau);
   else if (dtype == kBF16)
-    hipLaunchKernelGGL(gla_decay_kernel<bf16>, grid, dim3(256), rank * sizeof(float), st, (const bf16*)p, ld, low_off,
-                       (const bf16*)a2, bias, alpha, channels, rank, 1.f / tau);
+    hipLaunchKernelGGL(gla_decay_kernel<bf16>, grid, dim3(256), lds, st, (const bf16*)p, ld, low_off,
+                       (const bf16*)a2, bias, alpha, tokens, channels, rank, 1.f / tau);
   else
     return pa::fail("gla_decay: unknown element type code %d", dtype);
   return check_launch("gla_decay");

@@ -100,6 +100,23 @@ __global__ __launch_bounds__(kTalkThreads) void talking_prepare_kernel(
   }
   __syncthreads();
   T* dst = q_out + t * (size_t)nh * kd + (size_t)c * hd;
+  if (hd % 8 == 0) {                                        // sixteen or thirty-two bytes a thread
+    typedef T vec8 __attribute__((ext_vector_type(8)));
+    for (int i = threadIdx.x; i < nh * hd / 8; i += kTalkThreads) {
+      const int h = i / (hd / 8), d = 8 * (i % (hd / 8));
+      float acc[8] = {};
+      for (int g = 0; g < group; ++g) {
+        const float m = ts[g * nh + h];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[e] = fmaf(m, qs[g * hd + d + e], acc[e]);
+      }
+      vec8 v;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = from_f32<T>(acc[e]);
+      *reinterpret_cast<vec8*>(dst + (size_t)h * kd + d) = v;
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < nh * hd; i += kTalkThreads) {
     const int h = i / hd, d = i % hd;
     float acc = 0.f;
