@@ -2108,7 +2108,10 @@ def attention_wide_supported(kd: int, vd: int, page_size: int) -> bool:
 
 
 SHARED_SPLIT_KEYS = (128, 256, 512, 1024, 2048, 4096)   # keys a split of a single token's context, all heads over one key head
-SHARED_SPLIT_WORKGROUPS = 1024                          # the shortest split whose launch stays within this many workgroups
+# The shortest split whose launch stays within one round of the chip (a workgroup a compute unit), keys of 256 and four
+# value heads of 128 under a window of 1,024, the merge included: 8 sequences 12.1 us in splits of 128, 15.1 of 256; 32
+# sequences 28.2, 21.9 and 26.1 us in splits of 128, 256 and 512; 64 sequences 38.5, 34.6, 26.9 and 38.9 to 1,024
+SHARED_SPLIT_WORKGROUPS = 256
 
 
 def shared_split_plan(n_seqs: int, heads: int, max_context: int, window: int, page_size: int):
