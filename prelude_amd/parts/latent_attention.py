@@ -65,13 +65,14 @@ class LatentAttention(Mixer):
     LAUNCHES = 8   # down projections, prep, query up, absorb, rotation, attention, value up, output
     GRAPH_SAFE_PORTIONS = True   # launches follow the step's shape alone (the expanded form below runs in direct steps only)
     # A step that brings this many tokens or more (and is run directly, in bfloat16, with head sizes the matrix-core
-    # attention takes) attends in the expanded form: the keys and values of every
-    # head are made from the latents its sequences can see, by one product, into temporary pages, and the queries
-    # attend to them as they stand.  The form above moves both maps to the query side and pays rank + rot
-    # multiplications a (query, key, head) where this one pays head_dim and value_dim; what it costs instead is the
-    # product over the window's latents, which a short portion does not win back (measured at a latent of 512, heads of
-    # 128 and a window of 1,024: level at some 350 tokens).
-    EXPAND_FROM_TOKENS = 384
+    # attention takes) attends in the expanded form: the keys and values of every head are made from the latents its
+    # sequences can see, by one product, into temporary pages (a key's rotated part copied beside it), and the queries
+    # attend to them as they stand.  The form above moves both maps to the query side and pays rank + rot multiplications a
+    # (query, key, head) for the score and rank for the sum where this one pays head_dim + rot and value_dim; what it costs
+    # instead is the product over the visible latents, which a short portion does not win back (measured at a latent of 512
+    # and 16 heads of 128 + 64, whole prompts of twelve runs, six of them of this kind: 192 tokens 2.10 ms in both forms, 256
+    # 2.22 in both, 384 2.22 against 2.59, 2,048 4.87 against 8.08).
+    EXPAND_FROM_TOKENS = 256
 
     def __init__(self, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, value_dim: int, kv_rank: int,
                  q_rank: int, norm_eps: float, scale: Optional[float] = None, position: Optional[str] = None,

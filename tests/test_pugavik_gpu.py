@@ -180,7 +180,7 @@ def test_prepare_in_front_of_mixed_scores(gpu, dtype, nh, nkv, hd, vd, rot, bias
 
 # ---- attention on the matrix cores for any widths ---------------------------------------------------------------------------
 WIDE = [  # heads, key heads, value heads, key width, value width, window, page
-    (4, 1, 2, 96, 80, 72, 16), (4, 1, 2, 32, 24, 24, 8), (16, 1, 4, 256, 128, 200, 16), (20, 1, 5, 40, 12, 0, 16), (3, 1, 3, 136, 64, 1, 8),
+    (4, 1, 2, 112, 88, 60, 16), (4, 1, 2, 32, 24, 24, 8), (16, 1, 4, 256, 128, 200, 16), (20, 1, 5, 40, 12, 0, 16), (3, 1, 3, 136, 64, 1, 8),
     (4, 4, 4, 192, 128, 0, 16), (6, 3, 3, 48, 36, 65, 32), (4, 4, 2, 64, 128, 130, 16), (2, 1, 1, 512, 256, 0, 16), (2, 1, 2, 264, 100, 33, 64),
     (5, 1, 1, 8, 4, 0, 8), (8, 1, 8, 128, 200, 128, 16), (34, 1, 2, 64, 64, 0, 16)]
 
