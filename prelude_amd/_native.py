@@ -107,8 +107,8 @@ _KERNEL_API = {
     "pa_sample_wide": (I, [P, P, P, P, P, P, P, P, I, I, I]),
     "pa_group_norm_step": (I, [P, I, P, P, P, P, P, P, I, I, I, F]),
     "pa_poly_norm": (I, [P, I, P, P, P, P, I, I, F]),
-    "pa_head_norm_gate": (I, [P, I, P, P, c_long, P, P, c_long, I, I, I, F, I, F]),
-    "pa_attn_masked": (I, [P, I, P, P, P, P, I, P, P, P, c_long, I, I, I, I, I, I, I, I, F, F, P, P, P, c_long, F, P, P, I, I, I]),
+    "pa_head_norm_gate": (I, [P, I, P, P, c_long, P, P, c_long, I, I, I, F, I, F, I, P, P, F]),
+    "pa_attn_masked": (I, [P, I, P, P, P, P, I, P, P, P, c_long, I, I, I, I, I, I, I, I, F, F, P, P, P, c_long, F, P, P, I, I, I, I, I]),
     "pa_attn_masked_mfma_supports": (I, [I, I, I]),
     "pa_qkv_prepare": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, P, I, I, I, I, I, I, F]),
     "pa_delta_prepare": (I, [P, I, P, c_long, I, I, P, I, P, P, P, P, P, c_long, I, P, P, P, P, P, I, I, I, I, I, I]),
@@ -116,14 +116,14 @@ _KERNEL_API = {
     "pa_rotate_halves_f32": (I, [P, I, P, c_long, I, I, I, P, P, P, I, I, I, I, I, F]),
     "pa_latent_gather": (I, [P, I, P, P, I, P, P, P, I, I, I, I]),
     "pa_pair_embed": (I, [P, I, P, P, P, P, P, P, P, P, P, I, I, I, I, c_long, c_long, F]),
-    "pa_time_conv_add": (I, [P, I, P, P, P, P, P, P, P, I, I, I, I, I]),
+    "pa_time_conv": (I, [P, I, P, c_long, P, P, P, P, P, P, P, P, c_long, I, I, I, I, I, I, I]),
     "pa_stream_add_row": (I, [P, P, P, I, I]),
     "pa_latent_expand": (I, [P, I, P, P, P, I, P, P, P, P, P, I, I, I, I, I, I, I]),
     "pa_latent_queries": (I, [P, I, P, c_long, P, P, P, I, I, I, I, I]),
     "pa_attn_wide_supports": (I, [I, I, I]),
-    "pa_attn_wide": (I, [P, P, P, P, P, I, P, P, P, P, c_long, I, I, I, I, I, I, I, I, I, F, P]),
+    "pa_attn_wide": (I, [P, P, P, P, P, I, P, P, P, P, c_long, I, I, I, I, I, I, I, I, I, F, P, I, P, c_long]),
     "pa_attn_shared_workspace": (c_long, [I, I, I, I]),
-    "pa_attn_shared": (I, [P, P, P, P, P, I, P, P, P, P, c_long, P, I, I, I, I, I, I, I, F, P, I, I]),
+    "pa_attn_shared": (I, [P, P, P, P, P, I, P, P, P, P, c_long, P, I, I, I, I, I, I, I, I, F, P, I, I, I, P, c_long]),
     "pa_layer_norm_step": (I, [P, I, P, P, I, c_long, P, P, P, P, P, I, I, F]),
     "pa_stream_sum": (I, [P, I, P, P, P, P, P, I, I]),
     "pa_embed_scaled": (I, [P, I, P, P, P, I, I, I, F]),
@@ -135,14 +135,27 @@ _KERNEL_API = {
     "pa_gla_chunked_workspace": (c_long, [I, I, I, I, I, I]),
     "pa_gla_attn_chunked": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, P, P, I, I, I, I, I, I, F, I]),
     "pa_stream_add_branches": (I, [P, I, P, P, P, c_long]),
-    "pa_qkv_rope_prepare": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I]),
+    "pa_qkv_rope_prepare": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, F]),
     "pa_diff_combine": (I, [P, I, P, P, I, I, I, F, F, F]),
     "pa_sigmoid_gate": (I, [P, I, P, c_long, P, c_long, P, I, I]),
     "pa_cap_logits": (I, [P, P, c_long, F]),
+    "pa_branches_norm_step": (I, [P, I, P, P, I, P, F, P, P, I, P, F, c_long, F, P, P, P, P, I, I, F]),
+    "pa_gated_group_norm": (I, [P, I, P, P, c_long, P, P, c_long, I, I, I, F, F]),
+    "pa_ssd_gates": (I, [P, I, P, c_long, I, P, P, P, P, I, I]),
+    "pa_mlstm_max_copies": (I, [I]),
+    "pa_mlstm_gates": (I, [P, I, P, c_long, I, I, P, P, F, P, P, P, P, P, P, I, I, I, I]),
+    "pa_decay_scan": (I, [P, I, P, c_long, I, I, I, P, P, P, P, P, F, P, P, P, P, I, I, I, I, I, I, I]),
+    "pa_decay_scan_step": (I, [P, I, P, c_long, I, I, I, P, c_long, I, I, P, P, P, F, P, P, P, P, P, F, P, P, P, P, I, I, I, I, I]),
+    "pa_decay_scan_chunked_supports": (I, [P, c_long, I, I, I, I, I]),
+    "pa_decay_scan_chunked_workspace": (c_long, [I, I, I, I, I, I]),
+    "pa_decay_scan_chunked": (I, [P, P, c_long, I, I, I, P, P, P, P, P, F, P, P, P, P, P, P, I, I, I, I, I, I, I]),
+    "pa_lru_gates": (I, [P, I, P, P, P, P, P, P, P, P, P, P, P, c_long, P, I, P, P, P, c_long, F, I, I, I]),
+    "pa_lru_scan_workspace": (c_long, [I, I, I]),
+    "pa_lru_scan": (I, [P, I, P, P, P, P, P, P, P, c_long, P, I, P, P, P, c_long, F, P, I, I, I, I]),
 }
 
 _HOST_API = {
-    "pa_cache_create": (P, [I, I, IP, IP, IP, I]),
+    "pa_cache_create": (P, [I, I, IP, IP, IP, IP, I]),
     "pa_cache_destroy": (None, [P]),
     "pa_cache_open": (I, [P, c_longlong, I]),
     "pa_cache_reserve": (I, [P, c_longlong, I]),

@@ -43,24 +43,29 @@ class PageTables:
     """Pools, per-request tables and state slots (host side only; no GPU needed)."""
 
     def __init__(self, page_size: int, groups: Sequence[Tuple[int, ...]], state_slots: int = 0):
-        """``groups``: (number of pages, window or 0[, first positions a window keeps]) per group."""
+        """``groups``: (number of pages, window or 0[, first positions a window keeps[, chunk]]) per group.  A chunk goes with a
+        window of the same size: positions see back to the start of their own chunk of that many places."""
         if page_size < 1:
             raise CacheError(f"page size {page_size} must be positive")
-        groups = [(int(g[0]), int(g[1]), int(g[2]) if len(g) > 2 else 0) for g in groups]
-        for n, w, k in groups:
+        groups = [(int(g[0]), int(g[1]), int(g[2]) if len(g) > 2 else 0, int(g[3]) if len(g) > 3 else 0) for g in groups]
+        for n, w, k, c in groups:
             if n < 1 or w < 0 or k < 0:
                 raise CacheError(f"a cache group needs at least one page, a window >= 0 and kept first positions >= 0, "
                                  f"got ({n}, {w}, {k})")
+            if c and (c != w or k):
+                raise CacheError(f"a chunk of {c} positions goes with a window of as many and no kept first positions, got ({n}, {w}, {k})")
             if n * page_size >= 2 ** 31:
                 raise CacheError(f"{n} pages of {page_size} tokens exceed 32-bit slot numbers")
         self._lib = host()
         self.page_size = int(page_size)
-        self.groups = [(n, w) for n, w, _ in groups]
-        self.keep_first = [k for _, _, k in groups]
+        self.groups = [(g[0], g[1]) for g in groups]
+        self.keep_first = [g[2] for g in groups]
+        self.chunks = [g[3] for g in groups]
         n = (ctypes.c_int * len(groups))(*[g[0] for g in groups])
         w = (ctypes.c_int * len(groups))(*[g[1] for g in groups])
         k = (ctypes.c_int * len(groups))(*[g[2] for g in groups])
-        self._h = self._lib.pa_cache_create(self.page_size, len(self.groups), n, w, k, int(state_slots))
+        c = (ctypes.c_int * len(groups))(*[g[3] for g in groups])
+        self._h = self._lib.pa_cache_create(self.page_size, len(self.groups), n, w, k, c, int(state_slots))
         if not self._h:
             raise CacheError("cache manager could not be created")
 

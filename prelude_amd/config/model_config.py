@@ -917,3 +917,142 @@ class PugavikConfig:
         return cls(vocab=_positive(raw, "vocab", int, a, ""), width=_positive(raw, "width", int, a, ""),
                    norm_eps=_positive(_obj(raw, "norm", a), "eps", float, a, "norm."), embed_scale=scale, loop_start=start,
                    loop_stop=stop, loop_times=times, layers=tuple(layers), has_loop=loop is not None)
+
+
+# ---------------------------------------------------------------------------
+@dataclasses.dataclass(frozen=True)
+class PogoraxAttentionConfig:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    chunk: int = 0          # the query at i sees the key at j <= i when floor(i / chunk) = floor(j / chunk); 0: every j <= i
+    rot_dims: int = 0       # the first dimensions of a head that turn, in pairs
+    rot_base: float = 1.0
+
+
+@dataclasses.dataclass(frozen=True)
+class PogoraxMLSTMConfig:
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+
+@dataclasses.dataclass(frozen=True)
+class PogoraxGriffinConfig:
+    width: int
+    blocks: int
+    conv: int
+
+
+@dataclasses.dataclass(frozen=True)
+class PogoraxParallelConfig:
+    left: PogoraxAttentionConfig
+    right: object           # PogoraxMLSTMConfig | PogoraxGriffinConfig
+
+
+@dataclasses.dataclass(frozen=True)
+class PogoraxMamba2Config:
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int
+
+
+@dataclasses.dataclass(frozen=True)
+class PogoraxLayerConfig:
+    type: str
+    mixer: object           # PogoraxParallelConfig | PogoraxMamba2Config
+    ff: int                 # inner size of the dense feed-forward; 0: the layer has none
+
+
+@dataclasses.dataclass(frozen=True)
+class PogoraxConfig:
+    """Pogorax: a decoder of pre-norm layers listed one by one in ``layers``.  Mixers: ``mamba2``; ``parallel`` (attention inside
+    chunks of the sequence with a gate on its output, beside mLSTM's matrix memory) and ``parallel_2`` (causal attention on rotated
+    unit queries and keys, beside Griffin's recurrent block), both half the sum of their members' outputs, each brought to unit RMS.
+    The feed-forward is dense and gated (GELU in its tanh form), or absent.  Every size and constant is read from here; there is no
+    longest position and no end-of-sequence id."""
+    vocab: int
+    width: int
+    norm_eps: float
+    embed_scale: float
+    layers: Tuple[PogoraxLayerConfig, ...]
+
+    ARCH = "Pogorax"
+    MIXERS = ("parallel", "mamba2", "parallel_2")
+
+    @classmethod
+    def _attention(cls, m: Mapping[str, Any], mw: str, chunked: bool) -> PogoraxAttentionConfig:
+        a = cls.ARCH
+        heads, kv_heads, dim, vdim = (_positive(m, k, int, a, mw) for k in ("heads", "kv_heads", "dim", "vdim"))
+        if heads % kv_heads:
+            raise ConfigError(f"failed to parse {a} config: `{mw}heads` ({heads}) is no multiple of `kv_heads` ({kv_heads})")
+        scale = _positive(m, "scale", float, a, mw)
+        if chunked:
+            return PogoraxAttentionConfig(heads, kv_heads, dim, vdim, scale,
+                                          chunk=_positive(_obj(m, "mask", a, mw), "size", int, a, mw + "mask."))
+        rot = _obj(m, "rot", a, mw)
+        try:
+            dims = _get(rot, "dims", int, a)
+        except ConfigError as e:
+            raise ConfigError(str(e).replace("`dims`", f"`{mw}rot.dims`")) from None
+        if dims % 2 or dims > dim:
+            raise ConfigError(f"failed to parse {a} config: `{mw}rot.dims` ({dims}) must be even and at most `dim` ({dim})")
+        return PogoraxAttentionConfig(heads, kv_heads, dim, vdim, scale, rot_dims=dims,
+                                      rot_base=_positive(rot, "base", float, a, mw + "rot.") if dims else 1.0)
+
+    @classmethod
+    def _mixer(cls, kind: str, m: Mapping[str, Any], mw: str):
+        a = cls.ARCH
+        if kind == "mamba2":
+            c = PogoraxMamba2Config(**{k: _positive(m, k, int, a, mw) for k in ("heads", "vdim", "state", "groups", "conv", "norm_groups")})
+            if c.heads % c.groups:
+                raise ConfigError(f"failed to parse {a} config: `{mw}heads` ({c.heads}) is no multiple of `groups` ({c.groups})")
+            if c.heads * c.vdim % c.norm_groups:
+                raise ConfigError(f"failed to parse {a} config: `{mw}norm_groups` ({c.norm_groups}) does not divide the inner size "
+                                  f"({c.heads * c.vdim})")
+            return c
+        left, right = _obj(m, "left", a, mw), _obj(m, "right", a, mw)
+        rw = mw + "right."
+        if kind == "parallel":
+            r = PogoraxMLSTMConfig(*(_positive(right, k, int, a, rw) for k in ("heads", "dim", "vdim")), _positive(right, "gate_cap", float, a, rw))
+        else:
+            r = PogoraxGriffinConfig(*(_positive(right, k, int, a, rw) for k in ("width", "blocks", "conv")))
+            if r.width % r.blocks:
+                raise ConfigError(f"failed to parse {a} config: `{rw}blocks` ({r.blocks}) does not divide `width` ({r.width})")
+        return PogoraxParallelConfig(cls._attention(left, mw + "left.", chunked=kind == "parallel"), r)
+
+    @classmethod
+    def from_dict(cls, raw: Mapping[str, Any]) -> "PogoraxConfig":
+        a = cls.ARCH
+        layers_raw = raw.get("layers")
+        if not isinstance(layers_raw, list) or not layers_raw:
+            raise ConfigError(f"failed to parse {a} config: `layers` must be a non-empty list")
+        layers = []
+        for i, lr in enumerate(layers_raw):
+            w = f"layers[{i}]."
+            if not isinstance(lr, dict):
+                raise ConfigError(f"failed to parse {a} config: `layers[{i}]` must be an object")
+            kind = _get(lr, "type", str, a)
+            if kind not in cls.MIXERS:
+                raise ConfigError(f"failed to parse {a} config: `{w}type` {kind!r} is not one of {list(cls.MIXERS)}")
+            f = _obj(lr, "mlp", a, w, optional=True)
+            ff = 0
+            if f is not None:
+                fk = _get(f, "kind", str, a, default="dense")
+                if fk != "dense":
+                    raise ConfigError(f"failed to parse {a} config: `{w}mlp.kind` {fk!r} is not one of ['dense']")
+                ff = _positive(f, "ff", int, a, w + "mlp.")
+            layers.append(PogoraxLayerConfig(kind, cls._mixer(kind, _obj(lr, "mixer", a, w), w + "mixer."), ff))
+        emb = _obj(raw, "embedding", a)
+        try:
+            scale = _get(emb, "scale", float, a)
+        except ConfigError as e:
+            raise ConfigError(str(e).replace("`scale`", "`embedding.scale`")) from None
+        return cls(vocab=_positive(raw, "vocab", int, a, ""), width=_positive(raw, "width", int, a, ""),
+                   norm_eps=_positive(_obj(raw, "norm", a), "eps", float, a, "norm."), embed_scale=scale, layers=tuple(layers))

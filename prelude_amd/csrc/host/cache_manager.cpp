@@ -170,6 +170,7 @@ bool CacheManager::open(int64_t id, bool need_state) {
 int CacheManager::first_key_needed(int g, int start) const {
   const int w = groups_[g].window;
   if (w <= 0) return 0;
+  if (groups_[g].chunk > 0) return start / groups_[g].chunk * groups_[g].chunk;
   return std::max(0, start - w + 1);
 }
 

@@ -26,6 +26,8 @@ struct GroupSpec {
   int window = 0;  // keys a layer of this group looks back over, the query's own included; 0 = all
   int keep_first = 0;  // with a window: the first positions stay visible to every later token, so the pages that hold them
                        // are never given back while the request lives
+  int chunk = 0;  // with a window of as many keys: positions see back to the start of their own chunk of that many places
+                  // (counted from the request's start) and no further, so a chunk's pages go when the next one begins
 };
 
 // A fixed set of pages.  A page goes to whoever asks, first-in first-out, but a request's pages are kept in runs

@@ -328,14 +328,15 @@ int pa_poly_norm(void* stream, int dtype, const void* x, const float* bias, cons
 // out[r, h, :] = o[r, h, :] / sqrt(mean(o[r, h, :]^2) + eps) * w (null: none; vdim elements shared by the heads)
 //                * act(gate[r, h, :]) * scale;  act 0 sigmoid, 1 silu.
 int pa_head_norm_gate(void* stream, int dtype, const float* o, const void* gate, long gate_stride, const float* w, void* out,
-                      long out_stride, int nrows, int heads, int vdim, float eps, int act, float scale);
+                      long out_stride, int nrows, int heads, int vdim, float eps, int act, float scale,
+                      int weight_per_head, const float* den, const float* floor_in, float den_eps);
 
 // ---- attention with a window that keeps first tokens, a bias by distance, a gate a head (attention_masked.hip) ----
 int pa_attn_masked(void* stream, int dtype, const void* q, const void* k_cache, const void* v_cache, const int* block_table,
                    int table_stride, const int* seq_of_token, const int* positions, void* out, long out_stride, int tokens,
                    int nh, int nkv, int hd, int vd, int page_size, int window, int keep_first, float scale, float softcap,
                    const float* slopes, const float* sink, const void* gate, long gate_stride, float out_scale, const int* cu_q,
-                   const int* context_lens, int nseq, int max_q_len, int nv);
+                   const int* context_lens, int nseq, int max_q_len, int nv, int chunk, int gate_wide);
 int pa_attn_masked_mfma_supports(int hd, int vd, int page_size);
 int pa_qkv_prepare(void* stream, int dtype, const void* p, long stride, int q_off, int k_off, int v_off, const float* qw,
                    const float* kw, const int* slots, void* q_out, void* k_cache, void* v_cache, int tokens, int nh, int nkv,
@@ -356,23 +357,26 @@ int pa_rotate_halves_f32(void* stream, int dtype, const void* p, long stride, in
 int pa_pair_embed(void* stream, int dtype, const int* ids, const int* positions, const int* seq_of_token, const int* cu_q,
                   const int* state_slots, int* prev_state, const void* table, const void* pair, float* out, int tokens,
                   int hidden, int vocab, int buckets, long mul_prev, long mul_cur, float scale);
-int pa_time_conv_add(void* stream, int dtype, const void* h, const float* w, float* state, const int* seq_of_token,
-                     const int* cu_q, const int* state_slots, void* out, int tokens, int nseq, int channels, int taps,
-                     int all_single);
+// act 0 none, 1 SiLU; in_bias is added to every input (also as it is carried), bias to the sum; add_input: plus the input.
+int pa_time_conv(void* stream, int dtype, const void* h, long stride, const float* w, const float* in_bias, const float* bias,
+                 float* state, const int* seq_of_token, const int* cu_q, const int* state_slots, void* out, long out_stride,
+                 int tokens, int nseq, int channels, int taps, int act, int add_input, int all_single);
 // ---- attention on the matrix cores for keys and values of any widths (attention_wide.hip), bfloat16 ----
 // q [tokens, nh, kd], K [page, nkv, offset, kd], V [page, nv, vd, offset]; nv <= nkv: key head k goes with value head k mod nv,
 // else the query heads are dealt out to the value heads in runs.  kd a multiple of 8 up to 512, vd of 4 up to 256, pages of a
-// power of two from 8 on.  pa_attn_wide: the listed sequences' portions; pa_attn_shared: single tokens, all heads over one
+// power of two from 8 on.  chunk > 0: a query sees its own chunk of that many places alone; gate (or null): the output times
+// sigmoid(gate [tokens, nh * vd]).  pa_attn_wide: the listed sequences' portions; pa_attn_shared: single tokens, the heads over one
 // key head, in splits of split_keys keys (work: pa_attn_shared_workspace words).
 int pa_attn_wide_supports(int kd, int vd, int page_size);
 int pa_attn_wide(void* stream, const void* q, const void* kc, const void* vc, const int* block_table, int table_stride,
                  const int* seq_ids, const int* cu_q, const int* context_lens, void* out, long out_stride, int nseq, int max_q_len,
-                 int nh, int nkv, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink);
+                 int nh, int nkv, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink, int chunk,
+                 const void* gate, long gate_stride);
 long pa_attn_shared_workspace(int nseq, int nh, int vd, int max_splits);
 int pa_attn_shared(void* stream, const void* q, const void* kc, const void* vc, const int* block_table, int table_stride,
                    const int* seq_ids, const int* cu_q, const int* context_lens, void* out, long out_stride, float* work, int nseq,
-                   int nh, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink, int split_keys,
-                   int max_splits);
+                   int nh, int nkv, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink,
+                   int split_keys, int max_splits, int chunk, const void* gate, long gate_stride);
 // ---- layer norm around a 32-bit stream (layer_norm.hip) ----
 // residual += y (a tensor of `dtype`, or `slices` 32-bit partial sums slice_stride elements apart, or neither), then out =
 // layer norm of the row, times w plus b.  With rows: of those rows alone, the residual read only.
@@ -402,13 +406,51 @@ int pa_stream_add_branches(void* stream, int dtype, float* x, const void* a, con
 int pa_qkv_rope_prepare(void* stream, int dtype, const void* p, long stride, int q_off, int k_off, int v_off,
                         const float* inv_freq, const int* positions, const int* slots, const float* q_scale, void* q_out,
                         void* k_cache, void* v_cache, int tokens, int nq, int nk, int nv, int hd, int vd, int rot, int pairs,
-                        int page_size);
+                        int page_size, int unit, float eps);
 int pa_diff_combine(void* stream, int dtype, const void* a, void* out, int tokens, int heads, int vd, float lambda, float eps,
                     float scale);
 int pa_sigmoid_gate(void* stream, int dtype, const void* o, long o_stride, const void* gate, long gate_stride, void* out,
                     int rows, int width);
 int pa_cap_logits(void* stream, float* x, long total, float cap);
 
+// ---- branches brought to unit RMS in front of a stream, a gate in front of a norm in groups (layer_norm.hip, rowwise_groups.hip) ----
+// residual += c0 norm(y0) w0 (+ c1 norm(y1) w1), a y a tensor of `dtype` or `slices` 32-bit partial sums; out = the RMS norm of
+// the new rows times w (with `rows`: of those alone, the residual is read only).
+int pa_branches_norm_step(void* stream, int dtype, const void* y0, const float* parts0, int slices0, const float* w0, float c0,
+                          const void* y1, const float* parts1, int slices1, const float* w1, float c1, long slice_stride,
+                          float branch_eps, float* residual, const float* w, void* out, const int* rows, int nrows, int hidden,
+                          float eps);
+int pa_gated_group_norm(void* stream, int dtype, const float* y, const void* z, long z_stride, const float* w, void* out,
+                        long out_stride, int nrows, int width, int groups, float eps, float scale);
+// ---- recurrences with one decay a token and head (decay_scan.hip) ----
+int pa_ssd_gates(void* stream, int dtype, const void* p, long ld, int off, const float* bias, const float* a_log, float* la, float* b,
+                 int tokens, int heads);
+int pa_mlstm_max_copies(int vdim);
+int pa_mlstm_gates(void* stream, int dtype, const void* p, long ld, int i_off, int f_off, const float* i_bias, const float* f_bias,
+                   float cap, float* m, const int* state_slots, const int* cu_q, float* la, float* b, float* floor_out, int nseq,
+                   int heads, int vdim, int min_len);
+int pa_decay_scan(void* stream, int dtype, const void* p, long ld, int q_off, int k_off, int v_off, const float* la, const float* b,
+                  float* s, float* n, const float* skip, float q_scale, const int* state_slots, const int* cu_q, float* out, float* den,
+                  int nseq, int tokens, int heads, int group, int dim, int vdim, int min_len);
+int pa_decay_scan_step(void* stream, int dtype, const void* p, long ld, int q_off, int k_off, int v_off, const void* z, long z_ld,
+                       int z_off, int f_off, const float* bias, const float* f_bias, const float* a_log, float cap, float* m, float* floor_out, float* s,
+                       float* n, const float* skip, float q_scale, const int* state_slots, const int* cu_q, float* out, float* den,
+                       int nseq, int heads, int group, int dim, int vdim);
+int pa_decay_scan_chunked_supports(const void* p, long ld, int q_off, int k_off, int v_off, int dim, int vdim);
+long pa_decay_scan_chunked_workspace(int nlisted, int tokens, int heads, int dim, int vdim, int with_n);
+int pa_decay_scan_chunked(void* stream, const void* p, long ld, int q_off, int k_off, int v_off, const float* la, const float* b, float* s,
+                          float* n, const float* skip, float q_scale, const int* state_slots, const int* cu_q, const int* seq_ids,
+                          float* out, float* den, float* work, int nlisted, int tokens, int max_len, int heads, int group, int dim,
+                          int vdim);
+// ---- a gated linear recurrence a channel (lru.hip) ----
+int pa_lru_gates(void* stream, int dtype, const void* u, const void* wr, const void* wi, const float* br, const float* bi,
+                 const float* rate, float* state, const int* seq_of_token, const int* state_slots, const int* cu_q, const void* y,
+                 long y_ld, const float* y_bias, int act, float* a, float* x, void* out, long out_ld, float out_scale, int tokens,
+                 int width, int blocks);
+long pa_lru_scan_workspace(int nlisted, int tokens, int width);
+int pa_lru_scan(void* stream, int dtype, const void* u, const float* rate, float* state, const int* state_slots, const int* cu_q,
+                const int* seq_ids, const void* y, long y_ld, const float* y_bias, int act, float* a, float* x, void* out, long out_ld,
+                float out_scale, float* work, int nlisted, int tokens, int max_len, int width);
 #ifdef __cplusplus
 }
 #endif

@@ -3,11 +3,12 @@
 //
 //   * a window that keeps the first tokens: the query at i sees the key at j <= i when i - j < window (0: no window)
 //     or j < keep_first;
+//   * chunks: it sees the keys of its own chunk of `chunk` places alone;
 //   * a bias by distance: slope_h * (i - j) is taken off the (scaled, capped) score;
 //   * values of a width of their own (vdim);
 //   * a sink per head in the softmax's denominator;
-//   * a gate per (token, head): the head's output times sigmoid(gate), and a constant `out_scale`, before it is
-//     rounded; the output may lie inside a wider row (`out_stride`).
+//   * a gate per (token, head), or per (token, head, value column) (`gate_wide`): the output times sigmoid(gate), and a
+//     constant `out_scale`, before it is rounded; the output may lie inside a wider row (`out_stride`).
 //
 // And the kernel in front of it: a token's queries, keys and values taken from the merged projection, queries and
 // keys optionally brought to unit RMS over the whole projection (all heads at once) and multiplied by a weight of
@@ -42,7 +43,8 @@ __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
     const int* __restrict__ block_table, int table_stride, const int* __restrict__ seq_of_token,
     const int* __restrict__ positions, T* __restrict__ out, size_t out_stride, int nh, int nkv, int hd, int vd,
     int page_size, int window, int keep_first, float scale, float softcap, const float* __restrict__ slopes,
-    const float* __restrict__ sink, const T* __restrict__ gate, size_t gate_stride, float out_scale, int nv) {
+    const float* __restrict__ sink, const T* __restrict__ gate, size_t gate_stride, float out_scale, int nv, int chunk,
+    int gate_wide) {
   extern __shared__ float qs_all[];            // a query a wavefront
   __shared__ float ps[kMaskedWaves][kWave];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
@@ -53,7 +55,7 @@ __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
   const int pos = positions[t];
   const int seq = seq_of_token[t];
   const int hi = pos;
-  int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  int lo = first_visible(pos, window, chunk);
   int kept = keep_first < lo ? keep_first : lo;   // keys [0, kept) are seen beside [lo, hi]
   if (kept < 0) kept = 0;
   if (kept >= lo) { lo = 0; kept = 0; }           // the two ranges meet: one range from the start
@@ -75,9 +77,9 @@ __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
 
   float m = -INFINITY, l = 0.f;
   float o[kMaskedMaxDim / kWave] = {};
-  for (int chunk = 0; chunk <= last_chunk; ++chunk) {
-    if (chunk == kept_chunks && chunk < first_window_chunk) chunk = first_window_chunk;
-    const int c0 = chunk * kWave;
+  for (int block = 0; block <= last_chunk; ++block) {
+    if (block == kept_chunks && block < first_window_chunk) block = first_window_chunk;
+    const int c0 = block * kWave;
     const int c = c0 + lane;
     const bool valid = active && c <= hi && (c >= lo || c < kept);
     float s = -INFINITY;
@@ -124,12 +126,17 @@ __global__ __launch_bounds__(kMaskedWaves* kWave) void attn_masked_kernel(
       const float alpha = expf(m - m_fin);
       inv = alpha / (l * alpha + expf(sink[h] - m_fin));
     }
-    if (gate) inv *= 1.0f / (1.0f + expf(-to_f32(gate[(size_t)t * gate_stride + h])));
+    const T* grow = gate ? gate + (size_t)t * gate_stride : nullptr;
+    if (gate && !gate_wide) inv *= 1.0f / (1.0f + expf(-to_f32(grow[h])));
     inv *= out_scale;
 #pragma unroll
     for (int e = 0; e < kMaskedMaxDim / kWave; ++e) {
       const int d = lane + e * kWave;
-      if (d < vd) orow[d] = from_f32<T>(o[e] * inv);
+      if (d < vd) {
+        float v = o[e] * inv;
+        if (gate && gate_wide) v *= 1.0f / (1.0f + expf(-to_f32(grow[(size_t)h * vd + d])));
+        orow[d] = from_f32<T>(v);
+      }
     }
   }
 }
@@ -250,6 +257,8 @@ struct MaskedArgs {
   size_t gate_stride;
   float out_scale;
   int nv;                   // value heads in a page: key head k goes with value head k mod nv
+  int chunk;
+  int gate_wide;            // the gate has a column per value column of every head instead of one per head
 };
 
 // Grid (tiles of 64 tokens, nkv * head groups, sequences); WAVES wavefronts: four, or eight for steps in which every
@@ -284,10 +293,10 @@ __global__ __launch_bounds__(WAVES* kWave, WAVES == 8 ? 1 : 2) void attn_masked_
   const int my_pos = start + t0 + r;
   const int last_valid = t0 + 15 < q_len ? t0 + 15 : q_len - 1;
   const int last_pos = start + last_valid, first_pos = start + t0;
-  int lo = (window > 0 && first_pos - window + 1 > 0) ? first_pos - window + 1 : 0;
+  int lo = first_visible(first_pos, window, a.chunk);
   const int hi = last_pos + 1;
-  const int my_lo = (window > 0 && my_pos - window + 1 > 0) ? my_pos - window + 1 : 0;
-  const int all_lo = (window > 0 && last_pos - window + 1 > 0) ? last_pos - window + 1 : 0;
+  const int my_lo = first_visible(my_pos, window, a.chunk);
+  const int all_lo = first_visible(last_pos, window, a.chunk);
   const int all_hi = first_pos + 1;
   int kept = keep < lo ? keep : 0;           // keys [0, kept) are walked apart from [lo, hi)
   if (keep >= lo) lo = 0;                    // the two ranges meet: one range from the start
@@ -326,13 +335,20 @@ __global__ __launch_bounds__(WAVES* kWave, WAVES == 8 ? 1 : 2) void attn_masked_
     for (int j = 0; j < GT; ++j) {
       const int h = head0 + j;
       float inv = a.out_scale / (st[j].l[0] + a.sm.sink_term(h, st[j].reference()));
-      if (a.gate) inv *= 1.0f / (1.0f + __expf(-(float)a.gate[t * a.gate_stride + h]));
+      if (a.gate && !a.gate_wide) inv *= 1.0f / (1.0f + __expf(-(float)a.gate[t * a.gate_stride + h]));
       bf16* orow = a.out + t * a.out_stride + (size_t)h * VD;
 #pragma unroll
       for (int tt = 0; tt < OT; ++tt) {
         bf16x4 v;
+        float w[4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = (bf16)(st[j].o[tt][i] * inv);
+        for (int i = 0; i < 4; ++i) w[i] = st[j].o[tt][i] * inv;
+        if (a.gate && a.gate_wide) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) w[i] /= 1.0f + __expf(-(float)a.gate[t * a.gate_stride + (size_t)h * VD + 16 * tt + 4 * g + i]);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = (bf16)w[i];
         *reinterpret_cast<bf16x4*>(orow + 16 * tt + 4 * g) = v;
       }
     }
@@ -372,7 +388,7 @@ __global__ __launch_bounds__(WAVES* kWave, WAVES == 8 ? 1 : 2) void attn_masked_
     }
     const int h = head0 + j;
     float inv = a.out_scale / (l + a.sm.sink_term(h, mm));
-    if (a.gate) inv *= 1.0f / (1.0f + __expf(-(float)a.gate[(size_t)row0 * a.gate_stride + h]));
+    if (a.gate) inv /= 1.0f + __expf(-(float)a.gate[(size_t)row0 * a.gate_stride + (a.gate_wide ? (size_t)h * VD + d : (size_t)h)]);
     a.out[(size_t)row0 * a.out_stride + (size_t)h * VD + d] = (bf16)(o * inv);
   }
 }
@@ -442,7 +458,7 @@ extern "C" int pa_attn_masked(void* stream, int dtype, const void* q, const void
                               void* out, long out_stride, int tokens, int nh, int nkv, int hd, int vd, int page_size,
                               int window, int keep_first, float scale, float softcap, const float* slopes,
                               const float* sink, const void* gate, long gate_stride, float out_scale, const int* cu_q,
-                              const int* context_lens, int nseq, int max_q_len, int nv) {
+                              const int* context_lens, int nseq, int max_q_len, int nv, int chunk, int gate_wide) {
   if (tokens == 0) return 0;
   if (nv <= 0) nv = nkv;
   PA_REQUIRE(nkv % nv == 0 || (nv % nkv == 0 && nh % nv == 0), "attn_masked: %d key heads and %d value heads for %d query heads",
@@ -452,9 +468,10 @@ extern "C" int pa_attn_masked(void* stream, int dtype, const void* q, const void
   PA_REQUIRE(nh % nkv == 0, "attn_masked: %d query heads are not a multiple of %d KV heads", nh, nkv);
   PA_REQUIRE(hd > 0 && hd <= kMaskedMaxKey && vd > 0 && vd <= kMaskedMaxDim,
              "attn_masked: key width %d is outside 1..%d or value width %d outside 1..%d", hd, kMaskedMaxKey, vd, kMaskedMaxDim);
+  PA_REQUIRE(chunk >= 0 && (chunk == 0 || keep_first == 0), "attn_masked: chunks of %d places beside kept first tokens", chunk);
   PA_REQUIRE(window >= 0 && keep_first >= 0, "attn_masked: window %d or kept first tokens %d negative", window, keep_first);
   PA_REQUIRE(softcap >= 0.f, "attn_masked: a score cap of %g is negative (0 means none)", (double)softcap);
-  PA_REQUIRE(out_stride >= (long)nh * vd && (!gate || gate_stride >= nh), "attn_masked: output stride %ld or gate stride %ld "
+  PA_REQUIRE(out_stride >= (long)nh * vd && (!gate || gate_stride >= (gate_wide ? (long)nh * vd : nh)), "attn_masked: output stride %ld or gate stride %ld "
              "too small for %d heads of %d", out_stride, gate_stride, nh, vd);
   hipStream_t st = (hipStream_t)stream;
   if (dtype == kBF16 && nv <= nkv && pa_attn_masked_mfma_supports(hd, vd, page_size) && cu_q && context_lens && nseq > 0 && max_q_len > 0) {
@@ -464,7 +481,7 @@ extern "C" int pa_attn_masked(void* stream, int dtype, const void* q, const void
     MaskedArgs a{(const bf16*)q, (const bf16*)k_cache, (const bf16*)v_cache, block_table, table_stride, cu_q, context_lens,
                  (bf16*)out, (size_t)out_stride, nh, nkv, __builtin_ctz(page_size), window, window > 0 ? keep_first : 0,
                  score_map(scale, softcap, sink), softcap > 0.f ? 1.0f : 1.0f / scale, slopes, (const bf16*)gate,
-                 (size_t)gate_stride, out_scale, nv};
+                 (size_t)gate_stride, out_scale, nv, chunk, gate_wide};
     dim3 mgrid((max_q_len + 63) / 64, nkv * (group / gt), nseq);
     const bool singles = max_q_len == 1;
 #define PA_MASKED(D, V, GT)                                                                                   \
@@ -501,12 +518,12 @@ extern "C" int pa_attn_masked(void* stream, int dtype, const void* q, const void
     hipLaunchKernelGGL(attn_masked_kernel<float>, grid, dim3(kMaskedWaves * kWave), lds, st, (const float*)q,
                        (const float*)k_cache, (const float*)v_cache, block_table, table_stride, seq_of_token, positions,
                        (float*)out, (size_t)out_stride, nh, nkv, hd, vd, page_size, window, keep_first, scale, softcap, slopes,
-                       sink, (const float*)gate, (size_t)gate_stride, out_scale, nv);
+                       sink, (const float*)gate, (size_t)gate_stride, out_scale, nv, chunk, gate_wide);
   } else if (dtype == kBF16) {
     hipLaunchKernelGGL(attn_masked_kernel<bf16>, grid, dim3(kMaskedWaves * kWave), lds, st, (const bf16*)q,
                        (const bf16*)k_cache, (const bf16*)v_cache, block_table, table_stride, seq_of_token, positions,
                        (bf16*)out, (size_t)out_stride, nh, nkv, hd, vd, page_size, window, keep_first, scale, softcap, slopes,
-                       sink, (const bf16*)gate, (size_t)gate_stride, out_scale, nv);
+                       sink, (const bf16*)gate, (size_t)gate_stride, out_scale, nv, chunk, gate_wide);
   } else {
     return pa::fail("attn_masked: unknown element type code %d", dtype);
   }

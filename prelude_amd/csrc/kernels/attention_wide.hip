@@ -1,8 +1,9 @@
 // Paged causal attention on the matrix cores for keys and values of widths of their own that are not known when this is
 // compiled: keys of `kd` elements (a multiple of 8 up to 512), values of `vd` (a multiple of 4 up to 256), `nkv` key heads and
 // `nv` value heads (fewer value heads than key heads: key head k goes with value head k mod nv; more: the query heads are
-// dealt out to them in runs as to the key heads), an optional window and an optional sink per head.  bfloat16 storage,
-// 32-bit scores, sums and softmax.  The inner arithmetic and its operand layout are those of attention_mfma_core.h; the
+// dealt out to them in runs as to the key heads), an optional window, optional chunks (a query sees the keys of its own chunk
+// of `chunk` places alone), an optional sink per head and an optional gate (the output times sigmoid(gate), a number per value
+// column of every head).  bfloat16 storage, 32-bit scores, sums and softmax.  The inner arithmetic and its operand layout are those of attention_mfma_core.h; the
 // kernels are compiled for bounds of the widths; what lies between a width and its bound takes part in the products as
 // zeros (a branch around it would end a basic block, and operands could no longer be asked for ahead of their use).
 //
@@ -11,9 +12,9 @@
 //                        of group w % 4 (QT times 16 of them, which share every operand read from LDS) and on one half of
 //                        every block's keys, w / 4; the halves' sums are merged through LDS at the end.  Which keys are
 //                        added up in which order follows from their positions alone.
-//   attn_shared_kernel   single tokens where all query heads read the same key head (nkv = 1): sixteen heads are the sixteen
-//                        columns of a score tile, so every key is read once for all of them; the probabilities are masked
-//                        per value head where their sums are formed.  The keys are cut into splits anchored at multiples
+//   attn_shared_kernel   single tokens: up to sixteen query heads that read the same key head are the columns of a score
+//                        tile, so every key is read once for all of them; the probabilities are masked per value head where
+//                        their sums are formed.  The keys are cut into splits anchored at multiples
 //                        of split_keys; attn_shared_merge_kernel adds the splits up.
 #include "common.h"
 #include "api.h"
@@ -38,6 +39,12 @@ struct WideArgs {
   size_t out_stride;
   int nh, nkv, nv, kd, vd, page_shift, window;
   ScoreMap sm;
+  int chunk;
+  const bf16* gate;     // [tokens, gate_stride], a column per value column of every head; or null
+  size_t gate_stride;
+  __device__ __forceinline__ float gated(float v, size_t row, int h, int d) const {
+    return gate ? v / (1.0f + __expf(-(float)gate[row * gate_stride + (size_t)h * vd + d])) : v;
+  }
   __device__ __forceinline__ int value_head(int h) const { return nv <= nkv ? (h / (nh / nkv)) % nv : h / (nh / nv); }
 };
 
@@ -78,15 +85,15 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
   // what the workgroup stages, and what this wavefront's tokens see
   const int wg_first = start + tile * kTile;
   const int wg_last = start + (tile * kTile + kTile - 1 < q_len ? tile * kTile + kTile - 1 : q_len - 1);
-  const int wg_lo = (window > 0 && wg_first - window + 1 > 0) ? wg_first - window + 1 : 0;
+  const int wg_lo = first_visible(wg_first, window, a.chunk);
   const int wg_hi = wg_last + 1;
   const int t0 = tile * kTile + tg * 16 * QT;
   const bool wave_on = t0 < q_len;
   const int last_valid = t0 + 16 * QT - 1 < q_len ? t0 + 16 * QT - 1 : q_len - 1;
   const int first_pos = start + t0, last_pos = start + last_valid;
-  const int lo = (window > 0 && first_pos - window + 1 > 0) ? first_pos - window + 1 : 0;
+  const int lo = first_visible(first_pos, window, a.chunk);
   const int hi = last_pos + 1;
-  const int all_lo = (window > 0 && last_pos - window + 1 > 0) ? last_pos - window + 1 : 0;
+  const int all_lo = first_visible(last_pos, window, a.chunk);
   const int all_hi = first_pos + 1;
 
   bf16x8 qf[QT][KS];
@@ -189,7 +196,7 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
         for (int i = 0; i < 4; ++i) s[4 * t + i] = acc[t][j][i];
       if (masked) {
         const int my_pos = first_pos + 16 * j + r;
-        const int my_lo = window > 0 ? my_pos - window + 1 : 0;
+        const int my_lo = first_visible(my_pos, window, a.chunk);
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
           const int key = key0 + 8 * g + i;
@@ -285,17 +292,18 @@ __global__ __launch_bounds__(kWideThreads) void attn_wide_kernel(WideArgs a) {
       if (16 * tt + 4 * g < a.vd) {
         bf16x4 v;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = (bf16)((st[j].o[tt][i] * fa + m[(2 + 4 * tt + i) * kWave] * fb) * inv);
+        for (int i = 0; i < 4; ++i)
+          v[i] = (bf16)a.gated((st[j].o[tt][i] * fa + m[(2 + 4 * tt + i) * kWave] * fb) * inv, row0 + t, h, 16 * tt + 4 * g + i);
         *reinterpret_cast<bf16x4*>(orow + 16 * tt + 4 * g) = v;
       }
   }
 }
 
-// ---- single tokens, all heads over one key head ------------------------------------------------------------------------
+// ---- single tokens: the heads over one key head together ------------------------------------------------------------------------
 constexpr int kSharedWaves = 8;
 constexpr int kSharedBlock = 128;   // keys a block: a wavefront a tile of 16 of them
 
-// Grid (tiles of 16 heads, splits, sequences).  A block's scores are eight tiles of 16 keys x 16 heads, one a wavefront; they
+// Grid (key heads x tiles of 16 of a key head's query heads, splits, sequences).  A block's scores are eight tiles of 16 keys x 16 heads, one a wavefront; they
 // share one reference maximum per head through LDS, and their probabilities lie in LDS as the operands of the second
 // product.  That product's units, (value head, 32 keys), are dealt out to the wavefronts; the V^T of a wavefront's first two
 // units is asked for together with the keys, so that a short context is one trip to memory.
@@ -313,7 +321,7 @@ __global__ __launch_bounds__(kSharedWaves* kWave) void attn_shared_kernel(WideAr
   const int row = a.cu_q[seq];
   const int ctx = a.context_lens[seq];
   const int pos = ctx - 1;
-  const int lo = (a.window > 0 && pos - a.window + 1 > 0) ? pos - a.window + 1 : 0;
+  const int lo = first_visible(pos, a.window, a.chunk);
   const int first_split = lo / split_keys;
   const int nsplit = (ctx + split_keys - 1) / split_keys - first_split;
   if ((int)blockIdx.y >= nsplit) return;
@@ -321,12 +329,14 @@ __global__ __launch_bounds__(kSharedWaves* kWave) void attn_shared_kernel(WideAr
   const int klo = s0 > lo ? s0 : lo, khi = s0 + split_keys < ctx ? s0 + split_keys : ctx;   // never empty
   const int* table = a.block_table + (size_t)seq * a.table_stride;
   const int shift = a.page_shift, mask = (1 << shift) - 1;
-  const int head0 = blockIdx.x * 16;
-  const int heads = a.nh - head0 < 16 ? a.nh - head0 : 16;
+  const int group = a.nh / a.nkv, tiles = (group + 15) / 16;
+  const int kvh = blockIdx.x / tiles, tile = blockIdx.x % tiles;
+  const int head0 = kvh * group + tile * 16;
+  const int heads = group - tile * 16 < 16 ? group - tile * 16 : 16;
   const int my_head = head0 + (r < heads ? r : heads - 1);
-  const int my_vh = my_head / (a.nh / a.nv);
-  const int vh0 = head0 / (a.nh / a.nv);
-  const int units = 4 * ((head0 + heads - 1) / (a.nh / a.nv) - vh0 + 1);
+  const int my_vh = a.value_head(my_head);
+  const int vh0 = a.value_head(head0);
+  const int units = 4 * (a.value_head(head0 + heads - 1) - vh0 + 1);
 
   // queries as they are up to kd and zeros from there on: what the keys' loads bring beyond kd does not matter
   bf16x8 qf[KS];
@@ -348,7 +358,7 @@ __global__ __launch_bounds__(kSharedWaves* kWave) void attn_shared_kernel(WideAr
     // row r of the tile is key 8 (r / 4) + 4 tt + r % 4 of its 32
     int key = step0 + 8 * (r / 4) + 4 * tt + (r % 4);
     key = key < klo ? klo : (key >= khi ? khi - 1 : key);
-    const bf16* krow = a.kc + (((size_t)table[key >> shift] << shift) + (key & mask)) * a.kd;
+    const bf16* krow = a.kc + ((((size_t)table[key >> shift] * a.nkv + kvh) << shift) + (key & mask)) * a.kd;
     bf16x8 kf[KS];
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
@@ -437,7 +447,7 @@ __global__ __launch_bounds__(kSharedWaves* kWave) void attn_shared_kernel(WideAr
     const float mm = lds_max[0][j] * c;               // the exponent's reference
     const int h = head0 + j;
     if (nsplit == 1) {
-      a.out[(size_t)row * a.out_stride + (size_t)h * a.vd + d] = (bf16)(ov / (lv + a.sm.sink_term(h, mm)));
+      a.out[(size_t)row * a.out_stride + (size_t)h * a.vd + d] = (bf16)a.gated(ov / (lv + a.sm.sink_term(h, mm)), row, h, d);
     } else {
       const size_t slot = ((size_t)blockIdx.z * a.nh + h) * max_splits + blockIdx.y;
       part_o[slot * a.vd + d] = ov;
@@ -456,7 +466,7 @@ __global__ __launch_bounds__(256) void attn_shared_merge_kernel(WideArgs a, cons
   const int seq = a.seq_ids ? a.seq_ids[blockIdx.y] : (int)blockIdx.y;
   const int ctx = a.context_lens[seq];
   const int pos = ctx - 1;
-  const int lo = (a.window > 0 && pos - a.window + 1 > 0) ? pos - a.window + 1 : 0;
+  const int lo = first_visible(pos, a.window, a.chunk);
   const int nsplit = (ctx + split_keys - 1) / split_keys - lo / split_keys;
   if (nsplit == 1) return;                            // written by the first kernel
   const size_t base = ((size_t)blockIdx.y * a.nh + h) * max_splits;
@@ -483,7 +493,8 @@ __global__ __launch_bounds__(256) void attn_shared_merge_kernel(WideArgs a, cons
         l += pl[i] * f;
       }
   }
-  if (d < a.vd) a.out[(size_t)a.cu_q[seq] * a.out_stride + (size_t)h * a.vd + d] = (bf16)(o / (l + a.sm.sink_term(h, mm)));
+  const size_t row = a.cu_q[seq];
+  if (d < a.vd) a.out[row * a.out_stride + (size_t)h * a.vd + d] = (bf16)a.gated(o / (l + a.sm.sink_term(h, mm)), row, h, d);
 }
 
 template <int KDM, int VDM, int QT, int NBUF>
@@ -506,7 +517,7 @@ static int launch_shared(hipStream_t st, const WideArgs& a, float* work, int nse
   if (allowed != hipSuccess) return pa::fail("attn_shared: %zu bytes of LDS refused: %s", lds, hipGetErrorString(allowed));
   float* part_ml = work;
   float* part_o = work + (size_t)nseq * a.nh * max_splits * 2;
-  hipLaunchKernelGGL((attn_shared_kernel<KDM, VDM>), dim3((a.nh + 15) / 16, max_splits, nseq), dim3(kSharedWaves * kWave), lds, st, a,
+  hipLaunchKernelGGL((attn_shared_kernel<KDM, VDM>), dim3(a.nkv * ((a.nh / a.nkv + 15) / 16), max_splits, nseq), dim3(kSharedWaves * kWave), lds, st, a,
                      part_o, part_ml, split_keys, max_splits);
   if (int rc = check_launch("attn_shared")) return rc;
   if (max_splits == 1) return 0;
@@ -538,12 +549,14 @@ static int wide_check(const char* what, int nseq, int nh, int nkv, int nv, int k
 extern "C" int pa_attn_wide(void* stream, const void* q, const void* kc, const void* vc, const int* block_table, int table_stride,
                             const int* seq_ids, const int* cu_q, const int* context_lens, void* out, long out_stride, int nseq,
                             int max_q_len, int nh, int nkv, int nv, int kd, int vd, int page_size, int window, float scale,
-                            const float* sink) {
+                            const float* sink, int chunk, const void* gate, long gate_stride) {
   if (nseq == 0 || max_q_len == 0) return 0;
   if (int rc = wide_check("attn_wide", nseq, nh, nkv, nv, kd, vd, page_size, table_stride, window, scale, out_stride, q, kc, vc, out)) return rc;
+  PA_REQUIRE(chunk >= 0 && (!gate || gate_stride >= (long)nh * vd), "attn_wide: chunks of %d places or a gate of %ld columns", chunk, gate_stride);
   PA_REQUIRE(max_q_len > 0 && nseq <= 65535 && (max_q_len + 63) / 64 <= 65535, "attn_wide: portions of %d tokens", max_q_len);
   WideArgs a{(const bf16*)q, (const bf16*)kc, (const bf16*)vc, block_table, table_stride, seq_ids, cu_q, context_lens, (bf16*)out,
-             (size_t)out_stride, nh, nkv, nv, kd, vd, __builtin_ctz(page_size), window, score_map(scale, 0.f, sink)};
+             (size_t)out_stride, nh, nkv, nv, kd, vd, __builtin_ctz(page_size), window, score_map(scale, 0.f, sink), chunk,
+             (const bf16*)gate, (size_t)gate_stride};
   hipStream_t st = (hipStream_t)stream;
   if (vd <= 64) {
     if (kd <= 64) return launch_wide<64, 64, 2, 2>(st, a, nseq, max_q_len);
@@ -568,14 +581,16 @@ extern "C" long pa_attn_shared_workspace(int nseq, int nh, int vd, int max_split
 
 extern "C" int pa_attn_shared(void* stream, const void* q, const void* kc, const void* vc, const int* block_table, int table_stride,
                               const int* seq_ids, const int* cu_q, const int* context_lens, void* out, long out_stride, float* work,
-                              int nseq, int nh, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink,
-                              int split_keys, int max_splits) {
+                              int nseq, int nh, int nkv, int nv, int kd, int vd, int page_size, int window, float scale, const float* sink,
+                              int split_keys, int max_splits, int chunk, const void* gate, long gate_stride) {
   if (nseq == 0) return 0;
-  if (int rc = wide_check("attn_shared", nseq, nh, 1, nv, kd, vd, page_size, table_stride, window, scale, out_stride, q, kc, vc, out)) return rc;
+  if (int rc = wide_check("attn_shared", nseq, nh, nkv, nv, kd, vd, page_size, table_stride, window, scale, out_stride, q, kc, vc, out)) return rc;
+  PA_REQUIRE(chunk >= 0 && (!gate || gate_stride >= (long)nh * vd), "attn_shared: chunks of %d places or a gate of %ld columns", chunk, gate_stride);
   PA_REQUIRE(split_keys > 0 && split_keys % kSharedBlock == 0 && max_splits > 0 && max_splits <= 65535 && nseq <= 65535 && work,
              "attn_shared: splits of %d keys, %d at most", split_keys, max_splits);
   WideArgs a{(const bf16*)q, (const bf16*)kc, (const bf16*)vc, block_table, table_stride, seq_ids, cu_q, context_lens, (bf16*)out,
-             (size_t)out_stride, nh, 1, nv, kd, vd, __builtin_ctz(page_size), window, score_map(scale, 0.f, sink)};
+             (size_t)out_stride, nh, nkv, nv, kd, vd, __builtin_ctz(page_size), window, score_map(scale, 0.f, sink), chunk,
+             (const bf16*)gate, (size_t)gate_stride};
   hipStream_t st = (hipStream_t)stream;
   if (vd <= 128) {
     if (kd <= 128) return launch_shared<128, 128>(st, a, work, nseq, split_keys, max_splits);

@@ -55,6 +55,17 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// The first key the query at `pos` sees: the whole past, a sliding window of `window` places (its own included), or the start
+// of its own chunk of `chunk` places, counted from the sequence's start (0: none of that kind).
+__device__ __forceinline__ int first_visible(int pos, int window, int chunk) {
+  int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  if (chunk > 0) {
+    const int c = pos / chunk * chunk;
+    lo = c > lo ? c : lo;
+  }
+  return lo;
+}
+
 // Sum over a block of up to 1024 threads; every thread gets the result.
 // `scratch` is LDS for at least 16 floats.  The order of the additions is
 // fixed by the thread layout alone, so a row's result never depends on what

@@ -3,6 +3,8 @@
 //   pa_layer_norm_step   residual += y (a branch's output, as a tensor or as the 32-bit partial sums of a product cut along
 //                        its inner size; absent: nothing is added), then out = (x - mean) / sqrt(mean((x - mean)^2) + eps)
 //                        * w + b of the new row.  With `rows` only those rows are normed and the residual is read only.
+//   pa_branches_norm_step   residual += sum_b c_b norm_b(y_b) over one or two branches' outputs (each over its own root mean
+//                        square, times its weight), then out = the RMS norm of the new row times w; `rows` as above
 //   pa_stream_sum        out = x + y + extra + row, any of the last three absent; out may be x
 //   pa_embed_scaled      out[t] = table[id] * scale, 32-bit
 //   pa_activate          out = act(x) * scale on columns of wider rows: act GELU in its tanh form or SiLU
@@ -150,6 +152,124 @@ __global__ __launch_bounds__(kLnThreads) void layer_norm_step_kernel(Pending<T> 
   }
   const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)hidden + eps);
   for (int i = threadIdx.x; i < hidden; i += kLnThreads) out[r * hidden + i] = from_f32<T>((value(i) - mean) * inv * w[i] + b[i]);
+}
+
+// One or two branches beside each other in front of a 32-bit stream.
+template <typename T>
+struct NormedBranches {
+  Pending<T> y[2];           // the second may be empty
+  const float* w[2];
+  float c[2];
+  float eps;
+};
+
+template <typename T>
+__device__ __forceinline__ void pending_load8(const Pending<T>& p, size_t at, float* v) {
+  if (p.y) {
+    ln_load8(p.y + at, v);
+    return;
+  }
+  ln_load8(p.parts + at, v);
+  for (int k = 1; k < p.slices; ++k) {
+    float u[8];
+    ln_load8(p.parts + k * p.slice_stride + at, u);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] += u[i];
+  }
+}
+
+// A workgroup a row of up to 8 * 256 * VPT elements, everything in registers in pieces of eight.
+template <typename T, int VPT>
+__global__ __launch_bounds__(kLnThreads) void branches_norm_step_vec_kernel(NormedBranches<T> nb, float* __restrict__ residual,
+                                                                            const float* __restrict__ w, T* __restrict__ out,
+                                                                            const int* __restrict__ rows, int hidden, float eps) {
+  __shared__ float scratch[16], scratch2[16];
+  const size_t r = blockIdx.x;
+  const size_t src = rows ? (size_t)rows[r] : r;
+  float* res = residual + src * hidden;
+  const int pieces = hidden / 8;
+  const bool two = nb.y[1].any();
+  float x[VPT][8], a[VPT][8], b[VPT][8];
+  float sa = 0.f, sb = 0.f;
+#pragma unroll
+  for (int v = 0; v < VPT; ++v) {
+    const int piece = v * kLnThreads + threadIdx.x;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[v][i] = a[v][i] = b[v][i] = 0.f;
+    if (piece < pieces) {
+      ln_load8(res + 8 * piece, x[v]);
+      pending_load8(nb.y[0], src * hidden + 8 * piece, a[v]);
+      if (two) pending_load8(nb.y[1], src * hidden + 8 * piece, b[v]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        sa += a[v][i] * a[v][i];
+        sb += b[v][i] * b[v][i];
+      }
+    }
+  }
+  const float fa = nb.c[0] / sqrtf(block_sum(sa, scratch) / (float)hidden + nb.eps);
+  const float fb = two ? nb.c[1] / sqrtf(block_sum(sb, scratch2) / (float)hidden + nb.eps) : 0.f;
+  float ss = 0.f;
+#pragma unroll
+  for (int v = 0; v < VPT; ++v) {
+    const int piece = v * kLnThreads + threadIdx.x;
+    if (piece < pieces) {
+      float wa[8], wb[8];
+      ln_load8(nb.w[0] + 8 * piece, wa);
+      if (two) ln_load8(nb.w[1] + 8 * piece, wb);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        float y = a[v][i] * fa * wa[i];
+        if (two) y += b[v][i] * fb * wb[i];
+        x[v][i] += y;
+        ss += x[v][i] * x[v][i];
+      }
+      if (!rows) ln_store8(res + 8 * piece, x[v]);
+    }
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)hidden + eps);
+#pragma unroll
+  for (int v = 0; v < VPT; ++v) {
+    const int piece = v * kLnThreads + threadIdx.x;
+    if (piece < pieces) {
+      float o[8], wv[8];
+      ln_load8(w + 8 * piece, wv);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) o[i] = x[v][i] * inv * wv[i];
+      ln_store8(out + r * hidden + 8 * piece, o);
+    }
+  }
+}
+
+// Rows of any width up to 16384, the new row in LDS.
+template <typename T>
+__global__ __launch_bounds__(kLnThreads) void branches_norm_step_kernel(NormedBranches<T> nb, float* __restrict__ residual,
+                                                                        const float* __restrict__ w, T* __restrict__ out,
+                                                                        const int* __restrict__ rows, int hidden, float eps) {
+  extern __shared__ float new_row[];
+  __shared__ float scratch[16];
+  const size_t r = blockIdx.x;
+  const size_t src = rows ? (size_t)rows[r] : r;
+  float* res = residual + src * hidden;
+  for (int i = threadIdx.x; i < hidden; i += kLnThreads) new_row[i] = res[i];
+  for (int b = 0; b < 2; ++b) {
+    if (!nb.y[b].any()) continue;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < hidden; i += kLnThreads) {
+      const float v = nb.y[b].at(src * hidden + i);
+      ss += v * v;
+    }
+    const float f = nb.c[b] / sqrtf(block_sum(ss, scratch) / (float)hidden + nb.eps);
+    for (int i = threadIdx.x; i < hidden; i += kLnThreads) new_row[i] += nb.y[b].at(src * hidden + i) * f * nb.w[b][i];
+  }
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < hidden; i += kLnThreads) {   // (a thread comes back to its own elements alone)
+    const float v = new_row[i];
+    if (!rows) res[i] = v;
+    ss += v * v;
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)hidden + eps);
+  for (int i = threadIdx.x; i < hidden; i += kLnThreads) out[r * hidden + i] = from_f32<T>(new_row[i] * inv * w[i]);
 }
 
 // V elements a thread (V = 4 where the row width allows).
@@ -326,4 +446,39 @@ extern "C" int pa_activate(void* stream, int dtype, const void* x, long x_stride
   }
 #undef PA_ACT
   return check_launch("activate");
+}
+
+template <typename T>
+static void launch_branches_norm(hipStream_t st, const NormedBranches<T>& nb, float* residual, const float* w, T* out, const int* rows,
+                                 int nrows, int hidden, float eps) {
+  bool vec = hidden % 8 == 0 && hidden <= 8 * kLnThreads * 4 && aligned16(residual) && aligned16(w) && aligned16(out);
+  for (int b = 0; b < 2; ++b)
+    vec = vec && aligned16(nb.y[b].y) && aligned16(nb.y[b].parts) && nb.y[b].slice_stride % 4 == 0 && aligned16(nb.w[b]);
+  const dim3 grid(nrows), block(kLnThreads);
+#define PA_BNORM(V) hipLaunchKernelGGL((branches_norm_step_vec_kernel<T, V>), grid, block, 0, st, nb, residual, w, out, rows, hidden, eps)
+  if (!vec)
+    hipLaunchKernelGGL(branches_norm_step_kernel<T>, grid, block, hidden * sizeof(float), st, nb, residual, w, out, rows, hidden, eps);
+  else if (hidden <= 8 * kLnThreads) PA_BNORM(1);
+  else if (hidden <= 8 * kLnThreads * 2) PA_BNORM(2);
+  else PA_BNORM(4);
+#undef PA_BNORM
+}
+
+extern "C" int pa_branches_norm_step(void* stream, int dtype, const void* y0, const float* parts0, int slices0, const float* w0, float c0,
+                                     const void* y1, const float* parts1, int slices1, const float* w1, float c1, long slice_stride,
+                                     float branch_eps, float* residual, const float* w, void* out, const int* rows, int nrows, int hidden,
+                                     float eps) {
+  if (nrows == 0) return 0;
+  PA_REQUIRE(nrows > 0 && hidden > 0 && hidden <= 16384 && residual && w && out, "branches_norm_step: bad sizes rows=%d hidden=%d", nrows, hidden);
+  PA_REQUIRE((y0 != nullptr) != (slices0 > 0) && (slices0 == 0 || parts0) && w0 && !(y1 && slices1 > 0) && (slices1 == 0 || parts1) &&
+             (!(y1 || slices1 > 0) || w1), "branches_norm_step: a branch is a tensor or partial sums, with a weight");
+  hipStream_t st = (hipStream_t)stream;
+#define PA_BRANCHES(T)                                                                                                            \
+  launch_branches_norm<T>(st, NormedBranches<T>{{{(const T*)y0, parts0, slices0, (size_t)slice_stride}, {(const T*)y1, parts1, slices1, (size_t)slice_stride}}, \
+                                                {w0, w1}, {c0, c1}, branch_eps}, residual, w, (T*)out, rows, nrows, hidden, eps)
+  if (dtype == kF32) PA_BRANCHES(float);
+  else if (dtype == kBF16) PA_BRANCHES(bf16);
+  else return pa::fail("branches_norm_step: unknown element type code %d", dtype);
+#undef PA_BRANCHES
+  return check_launch("branches_norm_step");
 }

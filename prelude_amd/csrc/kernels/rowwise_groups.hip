@@ -268,13 +268,16 @@ __global__ __launch_bounds__(256) void poly_norm_vec_kernel(const bf16* __restri
   }
 }
 
-// A wavefront a (row, head): out[r, h, :] = o[r, h, :] / sqrt(mean(o[r, h, :]^2) + eps) * w * act(gate[r, h, :]) * scale.
-// w (or null: no weight) has `vdim` elements shared by the heads; gate act: 0 sigmoid(g), 1 g * sigmoid(g).
+// A wavefront a (row, head): out[r, h, :] = u / sqrt(mean(u^2) + eps) * w * act(gate[r, h, :]) * scale with u = o[r, h, :], or,
+// with `den`, u = o[r, h, :] / (max(|den[r, h]|, floor[r, h]) + den_eps).
+// w (or null: no weight) has `vdim` elements, shared by the heads (w_stride 0) or `vdim` a head; gate act: 0 sigmoid(g), 1 g * sigmoid(g).
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                                             size_t gate_stride, const float* __restrict__ w,
                                                             T* __restrict__ out, size_t out_stride, int nrows, int heads,
-                                                            int vdim, float eps, int act, float scale) {
+                                                            int vdim, float eps, int act, float scale, size_t w_stride,
+                                                            const float* __restrict__ den, const float* __restrict__ floor_in,
+                                                            float den_eps) {
   const int lane = threadIdx.x % kWave;
   const size_t item = (size_t)blockIdx.x * (blockDim.x / kWave) + threadIdx.x / kWave;
   if (item >= (size_t)nrows * heads) return;
@@ -284,7 +287,9 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   float ss = 0.f;
   for (int i = lane; i < vdim; i += kWave) ss += src[i] * src[i];
   ss = wave_sum(ss);
-  const float inv = 1.0f / sqrtf(ss / (float)vdim + eps);
+  const float f = den ? 1.0f / (fmaxf(fabsf(den[item]), floor_in[item]) + den_eps) : 1.0f;
+  const float inv = f / sqrtf(f * f * (ss / (float)vdim) + eps);
+  if (w) w += h * w_stride;
   const T* g = gate + r * gate_stride + (size_t)h * vdim;
   T* dst = out + r * out_stride + (size_t)h * vdim;
   for (int i = lane; i < vdim; i += kWave) {
@@ -292,6 +297,63 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
     const float sg = 1.0f / (1.0f + expf(-gv));
     dst[i] = from_f32<T>(src[i] * inv * (w ? w[i] : 1.0f) * (act == 1 ? gv * sg : sg) * scale);
   }
+}
+
+// A workgroup a (row, group): out = u / sqrt(mean(u^2) + eps) * w over the group's elements, u = y * silu(z).
+template <typename T, int VPT>
+__global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(const float* __restrict__ y, const T* __restrict__ z, size_t z_stride,
+                                                                   const float* __restrict__ w, T* __restrict__ out, size_t out_stride,
+                                                                   int width, int groups, float eps, float scale) {
+  __shared__ float scratch[16];
+  const size_t r = blockIdx.x;
+  const int len = width / groups, c0 = blockIdx.y * len, pieces = len / 8;
+  float u[VPT][8], wv[VPT][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int v = 0; v < VPT; ++v) {
+    const int piece = v * blockDim.x + threadIdx.x;
+    if (piece < pieces) {
+      float zv[8];
+      load8(y + r * width + c0 + 8 * piece, u[v]);
+      load8(z + r * z_stride + c0 + 8 * piece, zv);
+      load8(w + c0 + 8 * piece, wv[v]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        u[v][i] *= zv[i] / (1.0f + expf(-zv[i]));
+        ss += u[v][i] * u[v][i];
+      }
+    }
+  }
+  const float inv = scale / sqrtf(block_sum(ss, scratch) / (float)len + eps);
+#pragma unroll
+  for (int v = 0; v < VPT; ++v) {
+    const int piece = v * blockDim.x + threadIdx.x;
+    if (piece < pieces) {
+      float o[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) o[i] = u[v][i] * inv * wv[v][i];
+      store8(out + r * out_stride + c0 + 8 * piece, o);
+    }
+  }
+}
+template <typename T>
+__global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ z, size_t z_stride,
+                                                               const float* __restrict__ w, T* __restrict__ out, size_t out_stride,
+                                                               int width, int groups, float eps, float scale) {
+  __shared__ float scratch[16];
+  const size_t r = blockIdx.x;
+  const int len = width / groups, c0 = blockIdx.y * len;
+  auto value = [&](int i) {
+    const float zv = to_f32(z[r * z_stride + c0 + i]);
+    return y[r * width + c0 + i] * (zv / (1.0f + expf(-zv)));
+  };
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < len; i += blockDim.x) {
+    const float v = value(i);
+    ss += v * v;
+  }
+  const float inv = scale / sqrtf(block_sum(ss, scratch) / (float)len + eps);
+  for (int i = threadIdx.x; i < len; i += blockDim.x) out[r * out_stride + c0 + i] = from_f32<T>(value(i) * inv * w[c0 + i]);
 }
 
 }  // namespace pa
@@ -366,8 +428,11 @@ extern "C" int pa_poly_norm(void* stream, int dtype, const void* x, const float*
 }
 
 extern "C" int pa_head_norm_gate(void* stream, int dtype, const float* o, const void* gate, long gate_stride, const float* w,
-                                 void* out, long out_stride, int nrows, int heads, int vdim, float eps, int act, float scale) {
+                                 void* out, long out_stride, int nrows, int heads, int vdim, float eps, int act, float scale,
+                                 int weight_per_head, const float* den, const float* floor_in, float den_eps) {
   if (nrows == 0) return 0;
+  PA_REQUIRE((den == nullptr) == (floor_in == nullptr), "head_norm_gate: a denominator and its floor go together");
+  const size_t w_stride = weight_per_head ? (size_t)vdim : 0;
   PA_REQUIRE(nrows > 0 && heads > 0 && vdim > 0 && gate_stride >= (long)heads * vdim && out_stride >= (long)heads * vdim,
              "head_norm_gate: bad sizes rows=%d heads=%d vdim=%d gate stride=%ld out stride=%ld", nrows, heads, vdim,
              gate_stride, out_stride);
@@ -377,11 +442,42 @@ extern "C" int pa_head_norm_gate(void* stream, int dtype, const float* o, const 
   const int blocks = (int)((items + 3) / 4);
   if (dtype == kF32)
     hipLaunchKernelGGL(head_norm_gate_kernel<float>, dim3(blocks), dim3(256), 0, st, o, (const float*)gate, (size_t)gate_stride,
-                       w, (float*)out, (size_t)out_stride, nrows, heads, vdim, eps, act, scale);
+                       w, (float*)out, (size_t)out_stride, nrows, heads, vdim, eps, act, scale, w_stride, den, floor_in, den_eps);
   else if (dtype == kBF16)
     hipLaunchKernelGGL(head_norm_gate_kernel<bf16>, dim3(blocks), dim3(256), 0, st, o, (const bf16*)gate, (size_t)gate_stride, w,
-                       (bf16*)out, (size_t)out_stride, nrows, heads, vdim, eps, act, scale);
+                       (bf16*)out, (size_t)out_stride, nrows, heads, vdim, eps, act, scale, w_stride, den, floor_in, den_eps);
   else
     return pa::fail("head_norm_gate: unknown element type code %d", dtype);
   return check_launch("head_norm_gate");
+}
+
+// out [nrows, width] = norm_g(y * silu(z)) * w * scale: y 32-bit, z of the engine's type; norm_g: the row in `groups` equal parts.
+extern "C" int pa_gated_group_norm(void* stream, int dtype, const float* y, const void* z, long z_stride, const float* w, void* out,
+                                   long out_stride, int nrows, int width, int groups, float eps, float scale) {
+  if (nrows == 0) return 0;
+  PA_REQUIRE(nrows > 0 && width > 0 && groups > 0 && groups <= 65535 && width % groups == 0 && z_stride >= width && out_stride >= width,
+             "gated_group_norm: bad sizes rows=%d width=%d groups=%d", nrows, width, groups);
+  hipStream_t st = (hipStream_t)stream;
+  const int len = width / groups, pieces = len / 8;
+  auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const bool vec = len % 8 == 0 && pieces <= 256 * 4 && z_stride % 8 == 0 && out_stride % 8 == 0 && aligned(y) && aligned(z) && aligned(w) && aligned(out);
+  const int threads = pieces >= 256 ? 256 : 64 * ((pieces + 63) / 64);
+  const dim3 grid(nrows, groups);
+#define PA_GGN(T, V) hipLaunchKernelGGL((gated_group_norm_vec_kernel<T, V>), grid, dim3(threads), 0, st, y, (const T*)z, (size_t)z_stride, w, \
+                                        (T*)out, (size_t)out_stride, width, groups, eps, scale)
+#define PA_GGN_T(T)                                                                                                              \
+  do {                                                                                                                           \
+    if (!vec)                                                                                                                    \
+      hipLaunchKernelGGL(gated_group_norm_kernel<T>, grid, dim3(256), 0, st, y, (const T*)z, (size_t)z_stride, w, (T*)out,        \
+                         (size_t)out_stride, width, groups, eps, scale);                                                         \
+    else if (pieces <= 256) PA_GGN(T, 1);                                                                                        \
+    else if (pieces <= 512) PA_GGN(T, 2);                                                                                        \
+    else PA_GGN(T, 4);                                                                                                           \
+  } while (0)
+  if (dtype == kF32) PA_GGN_T(float);
+  else if (dtype == kBF16) PA_GGN_T(bf16);
+  else return pa::fail("gated_group_norm: unknown element type code %d", dtype);
+#undef PA_GGN_T
+#undef PA_GGN
+  return check_launch("gated_group_norm");
 }

@@ -12,7 +12,7 @@
 
 namespace pa {
 
-// s = x (+ residual) (or the residual's rows alone, x and parts null), all in 32-bit; residual <- s unrounded (unless `rows`); out = round(s * rsqrt(mean(s^2) + eps) * w).
+// s = x (+ residual) (or the residual alone, x and parts null), all in 32-bit; residual <- s unrounded (unless `rows`); out = round(s * rsqrt(mean(s^2) + eps) * w).
 // x may come as `slices` 32-bit partial sums, [slices, rows, hidden], added in order in place of the load of x.
 // One workgroup a row; NV elements a thread held in registers between the two passes when the row fits.
 template <typename T, int NV>
@@ -53,7 +53,7 @@ __global__ __launch_bounds__(256) void rmsnorm_wide_kernel(const T* __restrict__
     for (int j = 0; j < NV; ++j) {
       const int i = threadIdx.x + j * 256;
       if (i < hidden) {
-        if (rr && !rows) rr[i] = v[j];
+        if (rr && !rows && (xr || pr)) rr[i] = v[j];
         orow[i] = from_f32<T>(v[j] * inv * w[i]);
       }
     }
@@ -66,7 +66,7 @@ __global__ __launch_bounds__(256) void rmsnorm_wide_kernel(const T* __restrict__
     const float inv = rsqrtf(ss / (float)hidden + eps);
     for (int i = threadIdx.x; i < hidden; i += 256) {
       const float s = value(i);
-      if (rr && !rows) rr[i] = s;
+      if (rr && !rows && (xr || pr)) rr[i] = s;
       orow[i] = from_f32<T>(s * inv * w[i]);
     }
   }
@@ -255,8 +255,8 @@ extern "C" int pa_rmsnorm_wide(void* stream, int dtype, const void* x, const flo
                                float eps) {
   if (nrows == 0) return 0;
   PA_REQUIRE(nrows > 0 && hidden > 0, "rmsnorm_wide: bad sizes rows=%d hidden=%d", nrows, hidden);
-  PA_REQUIRE(!(x && parts) && (x || parts || (residual && rows)),
-             "rmsnorm_wide: give x or partial sums (one of them), or the residual and the rows to norm alone");
+  PA_REQUIRE(!(x && parts) && (x || parts || residual),
+             "rmsnorm_wide: give x or partial sums (one of them), or the residual to norm alone");
   PA_REQUIRE(!parts || slices >= 1, "rmsnorm_wide: %d slices", slices);
   hipStream_t st = (hipStream_t)stream;
   if (dtype == kF32)

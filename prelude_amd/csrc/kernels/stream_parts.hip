@@ -3,13 +3,13 @@
 //   pa_pair_embed          out[t] = table[id] * scale + pair[(prev * mul_prev + id * mul_cur) mod buckets], 32-bit; the
 //                          previous token of a portion's first token comes from a per-request slot, which then takes
 //                          the portion's last token; a sequence's first token reads row `buckets`
-//   pa_time_conv_add       out = h + conv(h): a causal convolution over time on each channel (weights [taps, channels]),
-//                          the last taps - 1 inputs carried per request
+//   pa_time_conv           out = act(conv(h + in_bias) + bias) (+ h): a causal convolution over time on each channel
+//                          (weights [taps, channels]), the last taps - 1 inputs carried per request
 //   pa_stream_add_row      x[t] += row, in place
 //   pa_stream_add_branches x += a + b, in place (b may be absent)
 //   pa_qkv_rope_prepare    queries, keys and values out of a merged projection: the first `rot` dimensions of every
-//                          query and key head turned by position (in halves or in pairs), queries times a number per
-//                          head, keys and values into the paged cache; keys and values have widths and head counts
+//                          query and key head turned by position (in halves or in pairs), heads optionally over their own
+//                          root mean square, queries times a number per head, keys and values into the paged cache; keys and values have widths and head counts
 //                          of their own
 //   pa_diff_combine        out[t, h] = u / sqrt(mean(u^2) + eps) * scale with u = a[t, h] - lambda a[t, heads + h]
 //   pa_sigmoid_gate        out = o * sigmoid(gate)
@@ -53,17 +53,19 @@ __global__ __launch_bounds__(256) void pair_embed_kernel(const int* __restrict__
   }
 }
 
-// state [slots, taps - 1, C] 32-bit: the inputs at the taps - 1 positions before the portion's start, oldest first (zeros
-// before the sequence's start).  A thread owns V consecutive channels of a token (V = 8: 16-byte pieces of bfloat16).  A
-// sequence that brings one token is the only reader of its slot, so its thread moves the carried inputs on itself;
-// portions leave that to time_conv_carry_kernel, which runs behind this one.
+// state [slots, taps - 1, C] 32-bit: the inputs (in_bias added) at the taps - 1 positions before the portion's start, oldest
+// first (zeros before the sequence's start).  A thread owns V consecutive channels of a token (V = 8: 16-byte pieces of
+// bfloat16).  A sequence that brings one token is the only reader of its slot, so its thread moves the carried inputs on
+// itself; portions leave that to time_conv_carry_kernel, which runs behind this one.
 constexpr int kConvMaxTaps = 17;
 
 template <typename T, int V>
-__global__ __launch_bounds__(256) void time_conv_add_kernel(const T* __restrict__ h, const float* __restrict__ w,
-                                                            float* __restrict__ state, const int* __restrict__ seq_of_token,
-                                                            const int* __restrict__ cu_q, const int* __restrict__ state_slots,
-                                                            T* __restrict__ out, int C, int taps) {
+__global__ __launch_bounds__(256) void time_conv_kernel(const T* __restrict__ h, size_t stride, const float* __restrict__ w,
+                                                        const float* __restrict__ in_bias, const float* __restrict__ bias,
+                                                        float* __restrict__ state, const int* __restrict__ seq_of_token,
+                                                        const int* __restrict__ cu_q, const int* __restrict__ state_slots,
+                                                        T* __restrict__ out, size_t out_stride, int C, int taps, int act,
+                                                        int add_input) {
   typedef T vec_t __attribute__((ext_vector_type(V)));
   const int t = blockIdx.x;
   const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
@@ -74,10 +76,15 @@ __global__ __launch_bounds__(256) void time_conv_add_kernel(const T* __restrict_
   const bool single = cu_q[seq + 1] - begin == 1;
   const int keep = taps - 1;
   float* st = keep > 0 ? state + (size_t)state_slots[seq] * keep * C : nullptr;
-  const vec_t xv = *reinterpret_cast<const vec_t*>(h + (size_t)t * C + c);
-  float x[V], acc[V];
+  float x[V], acc[V], ib[V];
+  auto input = [&](int at, float* v) {
+    const vec_t pv = *reinterpret_cast<const vec_t*>(h + (size_t)at * stride + c);
 #pragma unroll
-  for (int e = 0; e < V; ++e) x[e] = to_f32(xv[e]), acc[e] = 0.f;
+    for (int e = 0; e < V; ++e) v[e] = to_f32(pv[e]) + ib[e];
+  };
+#pragma unroll
+  for (int e = 0; e < V; ++e) ib[e] = in_bias ? in_bias[c + e] : 0.f, acc[e] = bias ? bias[c + e] : 0.f;
+  input(t, x);
   for (int j = 0; j < taps; ++j) {
     const int back = keep - j;   // the input `back` positions before this token
     float v[V];
@@ -85,9 +92,7 @@ __global__ __launch_bounds__(256) void time_conv_add_kernel(const T* __restrict_
 #pragma unroll
       for (int e = 0; e < V; ++e) v[e] = x[e];
     } else if (rel - back >= 0) {
-      const vec_t pv = *reinterpret_cast<const vec_t*>(h + (size_t)(t - back) * C + c);
-#pragma unroll
-      for (int e = 0; e < V; ++e) v[e] = to_f32(pv[e]);
+      input(t - back, v);
     } else {
       const float* sp = st + (size_t)(rel - back + keep) * C + c;
 #pragma unroll
@@ -108,15 +113,20 @@ __global__ __launch_bounds__(256) void time_conv_add_kernel(const T* __restrict_
   }
   vec_t ov;
 #pragma unroll
-  for (int e = 0; e < V; ++e) ov[e] = from_f32<T>(x[e] + acc[e]);
-  *reinterpret_cast<vec_t*>(out + (size_t)t * C + c) = ov;
+  for (int e = 0; e < V; ++e) {
+    float y = acc[e];
+    if (act == 1) y = y / (1.0f + expf(-y));
+    if (add_input) y += x[e];
+    ov[e] = from_f32<T>(y);
+  }
+  *reinterpret_cast<vec_t*>(out + (size_t)t * out_stride + c) = ov;
 }
 
 // A thread a (sequence, channel) of the sequences that bring more than one token: it reads all it needs before it writes.
 template <typename T>
-__global__ __launch_bounds__(256) void time_conv_carry_kernel(const T* __restrict__ h, float* __restrict__ state,
-                                                              const int* __restrict__ cu_q, const int* __restrict__ state_slots,
-                                                              int C, int taps) {
+__global__ __launch_bounds__(256) void time_conv_carry_kernel(const T* __restrict__ h, size_t stride, const float* __restrict__ in_bias,
+                                                              float* __restrict__ state, const int* __restrict__ cu_q,
+                                                              const int* __restrict__ state_slots, int C, int taps) {
   const int seq = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
@@ -124,10 +134,11 @@ __global__ __launch_bounds__(256) void time_conv_carry_kernel(const T* __restric
   if (n <= 1) return;
   const int keep = taps - 1;
   float* st = state + (size_t)state_slots[seq] * keep * C;
+  const float ib = in_bias ? in_bias[c] : 0.f;
   float fresh[kConvMaxTaps - 1];
   for (int i = 0; i < keep; ++i) {
     const int rel = n - keep + i;   // the step's token this place now holds, or an older input when negative
-    fresh[i] = rel >= 0 ? to_f32(h[(size_t)(begin + rel) * C + c]) : st[(size_t)(i + n) * C + c];
+    fresh[i] = rel >= 0 ? to_f32(h[(size_t)(begin + rel) * stride + c]) + ib : st[(size_t)(i + n) * C + c];
   }
   for (int i = 0; i < keep; ++i) st[(size_t)i * C + c] = fresh[i];
 }
@@ -166,7 +177,7 @@ __global__ __launch_bounds__(kPrepWaves* kWave) void qkv_rope_prepare_kernel(
     const T* __restrict__ p, size_t stride, int q_off, int k_off, int v_off, const float* __restrict__ inv_freq,
     const int* __restrict__ positions, const int* __restrict__ slots, const float* __restrict__ q_scale, T* __restrict__ q_out,
     T* __restrict__ k_cache, T* __restrict__ v_cache, int tokens, int nq, int nk, int nv, int hd, int vd, int rot, int pairs,
-    int page_size) {
+    int page_size, int unit_rms, float eps) {
   __shared__ float xs[kPrepWaves][kPrepMaxDim];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int heads = nq + nk + nv;
@@ -188,12 +199,19 @@ __global__ __launch_bounds__(kPrepWaves* kWave) void qkv_rope_prepare_kernel(
   const bool is_q = h < nq;
   const bool turns = active && h < nq + nk;
   const T* src = is_q ? row + q_off + (size_t)h * hd : row + k_off + (size_t)(h - nq) * hd;
+  float ss = 0.f;
   if (turns)
-    for (int i = lane; i < hd; i += kWave) xs[wave][i] = to_f32(src[i]);
+    for (int i = lane; i < hd; i += kWave) {
+      const float v = to_f32(src[i]);
+      xs[wave][i] = v;
+      ss += v * v;
+    }
   __syncthreads();
   if (!turns || (!is_q && slot < 0)) return;
   T* dst = is_q ? q_out + ((size_t)t * nq + h) * hd : k_cache + (((size_t)page * nk + (h - nq)) * page_size + off) * hd;
-  const float mul = (is_q && q_scale) ? q_scale[h] : 1.0f;
+  float mul = (is_q && q_scale) ? q_scale[h] : 1.0f;
+  // the turned head over its own root mean square: turning leaves the sum of squares as it is
+  if (unit_rms) mul *= 1.0f / sqrtf(wave_sum(ss) / (float)hd + eps);
   const int half = rot / 2;
   const int pos = rot > 0 ? positions[t] : 0;
   for (int i = lane; i < hd; i += kWave) {
@@ -282,36 +300,40 @@ extern "C" int pa_pair_embed(void* stream, int dtype, const int* ids, const int*
   return check_launch("pair_embed");
 }
 
-extern "C" int pa_time_conv_add(void* stream, int dtype, const void* h, const float* w, float* state, const int* seq_of_token,
-                                const int* cu_q, const int* state_slots, void* out, int tokens, int nseq, int channels, int taps,
-                                int all_single) {
+extern "C" int pa_time_conv(void* stream, int dtype, const void* h, long stride, const float* w, const float* in_bias,
+                            const float* bias, float* state, const int* seq_of_token, const int* cu_q, const int* state_slots,
+                            void* out, long out_stride, int tokens, int nseq, int channels, int taps, int act, int add_input,
+                            int all_single) {
   if (tokens == 0) return 0;
-  PA_REQUIRE(tokens > 0 && nseq > 0 && channels > 0 && taps >= 1 && taps <= kConvMaxTaps, "time_conv_add: bad sizes tokens=%d "
+  PA_REQUIRE(tokens > 0 && nseq > 0 && channels > 0 && taps >= 1 && taps <= kConvMaxTaps, "time_conv: bad sizes tokens=%d "
              "sequences=%d channels=%d taps=%d", tokens, nseq, channels, taps);
-  PA_REQUIRE(taps == 1 || state, "time_conv_add: %d taps need the carried inputs", taps);
-  PA_REQUIRE((channels + 255) / 256 <= 65535, "time_conv_add: %d channels exceed the grid", channels);
+  PA_REQUIRE(taps == 1 || state, "time_conv: %d taps need the carried inputs", taps);
+  PA_REQUIRE(stride >= channels && out_stride >= channels, "time_conv: strides %ld and %ld for %d channels", stride, out_stride, channels);
+  PA_REQUIRE(act == 0 || act == 1, "time_conv: unknown activation code %d", act);
+  PA_REQUIRE((channels + 255) / 256 <= 65535, "time_conv: %d channels exceed the grid", channels);
   hipStream_t st = (hipStream_t)stream;
-  const bool wide = channels % 8 == 0 && (reinterpret_cast<uintptr_t>(h) & 15) == 0 && (reinterpret_cast<uintptr_t>(out) & 15) == 0;
+  const bool wide = channels % 8 == 0 && stride % 8 == 0 && out_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(h) & 15) == 0 &&
+                    (reinterpret_cast<uintptr_t>(out) & 15) == 0;
   const int per = wide ? 8 : 1;
   dim3 grid(tokens, (channels / per + 255) / 256), cgrid(nseq, (channels + 255) / 256);
   const int threads = channels / per >= 256 ? 256 : 64 * ((channels / per + 63) / 64);
+#define PA_CONV_V(T, V)                                                                                                         \
+  hipLaunchKernelGGL((time_conv_kernel<T, V>), grid, dim3(threads), 0, st, (const T*)h, (size_t)stride, w, in_bias, bias, state, \
+                     seq_of_token, cu_q, state_slots, (T*)out, (size_t)out_stride, channels, taps, act, add_input)
 #define PA_CONV(T)                                                                                                              \
   do {                                                                                                                          \
-    if (wide)                                                                                                                   \
-      hipLaunchKernelGGL((time_conv_add_kernel<T, 8>), grid, dim3(threads), 0, st, (const T*)h, w, state, seq_of_token, cu_q,    \
-                         state_slots, (T*)out, channels, taps);                                                                 \
-    else                                                                                                                        \
-      hipLaunchKernelGGL((time_conv_add_kernel<T, 1>), grid, dim3(threads), 0, st, (const T*)h, w, state, seq_of_token, cu_q,    \
-                         state_slots, (T*)out, channels, taps);                                                                 \
+    if (wide) PA_CONV_V(T, 8);                                                                                                  \
+    else PA_CONV_V(T, 1);                                                                                                       \
     if (taps > 1 && !all_single)                                                                                                \
-      hipLaunchKernelGGL(time_conv_carry_kernel<T>, cgrid, dim3(256), 0, st, (const T*)h, state, cu_q, state_slots, channels,   \
-                         taps);                                                                                                 \
+      hipLaunchKernelGGL(time_conv_carry_kernel<T>, cgrid, dim3(256), 0, st, (const T*)h, (size_t)stride, in_bias, state, cu_q,  \
+                         state_slots, channels, taps);                                                                          \
   } while (0)
   if (dtype == kF32) PA_CONV(float);
   else if (dtype == kBF16) PA_CONV(bf16);
-  else return pa::fail("time_conv_add: unknown element type code %d", dtype);
+  else return pa::fail("time_conv: unknown element type code %d", dtype);
 #undef PA_CONV
-  return check_launch("time_conv_add");
+#undef PA_CONV_V
+  return check_launch("time_conv");
 }
 
 extern "C" int pa_stream_add_row(void* stream, float* x, const float* row, int tokens, int hidden) {
@@ -346,7 +368,7 @@ extern "C" int pa_stream_add_branches(void* stream, int dtype, float* x, const v
 extern "C" int pa_qkv_rope_prepare(void* stream, int dtype, const void* p, long stride, int q_off, int k_off, int v_off,
                                    const float* inv_freq, const int* positions, const int* slots, const float* q_scale,
                                    void* q_out, void* k_cache, void* v_cache, int tokens, int nq, int nk, int nv, int hd, int vd,
-                                   int rot, int pairs, int page_size) {
+                                   int rot, int pairs, int page_size, int unit_rms, float eps) {
   if (tokens == 0) return 0;
   PA_REQUIRE(tokens > 0 && nq >= 0 && hd > 0 && hd <= kPrepMaxDim && p && (q_out || nq == 0) && (nq > 0 || slots),
              "qkv_rope_prepare: bad sizes tokens=%d nq=%d hd=%d", tokens, nq, hd);
@@ -367,11 +389,11 @@ extern "C" int pa_qkv_rope_prepare(void* stream, int dtype, const void* p, long 
   if (dtype == kF32)
     hipLaunchKernelGGL(qkv_rope_prepare_kernel<float>, grid, dim3(kPrepWaves * kWave), 0, st, (const float*)p, (size_t)stride, q_off,
                        k_off, v_off, inv_freq, positions, slots, q_scale, (float*)q_out, (float*)k_cache, (float*)v_cache, tokens,
-                       nq, nk, nv, hd, vd, rot, pairs ? 1 : 0, page_size);
+                       nq, nk, nv, hd, vd, rot, pairs ? 1 : 0, page_size, unit_rms, eps);
   else if (dtype == kBF16)
     hipLaunchKernelGGL(qkv_rope_prepare_kernel<bf16>, grid, dim3(kPrepWaves * kWave), 0, st, (const bf16*)p, (size_t)stride, q_off,
                        k_off, v_off, inv_freq, positions, slots, q_scale, (bf16*)q_out, (bf16*)k_cache, (bf16*)v_cache, tokens, nq,
-                       nk, nv, hd, vd, rot, pairs ? 1 : 0, page_size);
+                       nk, nv, hd, vd, rot, pairs ? 1 : 0, page_size, unit_rms, eps);
   else
     return pa::fail("qkv_rope_prepare: unknown element type code %d", dtype);
   return check_launch("qkv_rope_prepare");

@@ -225,8 +225,7 @@ class CausalLM:
             normed = self.final_norm.forward_rows(None, residual, step.want_rows,
                                                   out_dtype=hidden.dtype if hidden is not None else self.dtype)
             return self.head.forward(normed)
-        if not self.final_norm.TAKES_SLICE_SUMS:
-            from ..ops import kernels as K
-            hidden = K.as_tensor(hidden)
+        from ..parts.block import as_norm_takes
+        hidden = as_norm_takes(self.final_norm, hidden)
         normed = self.final_norm.forward_rows(hidden, residual, step.want_rows)
         return self.head.forward(normed)

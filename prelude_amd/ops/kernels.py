@@ -354,6 +354,12 @@ class LinearWeight:
         return self.rows[:n]
 
 
+def pad_rows(w: torch.Tensor, multiple: int = 8) -> torch.Tensor:
+    """The weight with rows of zeros behind it up to a multiple: the product's rows are then whole 16-byte pieces."""
+    extra = -w.shape[0] % multiple
+    return w if extra == 0 else torch.cat([w, w.new_zeros((extra, *w.shape[1:]))], dim=0)
+
+
 def prepare_weight(w: torch.Tensor) -> LinearWeight:
     """What a part keeps of a weight it multiplies by: called once when weights are loaded."""
     tiles = None
@@ -687,9 +693,58 @@ def _skinny_slices(m: int, n: int, k: int) -> int:
     return 1
 
 
+class NormedBranches:
+    """One or two branches' outputs [T, H] (tensors or ``SliceSums``) that stand for sum_b scale_b norm(y_b) weight_b, norm(y)
+    being y over its own sqrt(mean(y^2) + eps): what a mixer made of members hands on.  A norm that says ``TAKES_BRANCHES``
+    brings them to unit RMS and adds them to the stream itself."""
+
+    def __init__(self, branches, weights, scales, eps: float):
+        if not 1 <= len(branches) <= 2 or not len(branches) == len(weights) == len(scales):
+            raise NativeError(f"NormedBranches: {len(branches)} branches, {len(weights)} weights and {len(scales)} scales")
+        self.branches, self.weights, self.scales, self.eps = list(branches), list(weights), list(scales), float(eps)
+        self.shape, self.dtype = tuple(branches[0].shape), branches[0].dtype
+
+    def materialize(self) -> torch.Tensor:
+        """The sum in 32-bit, for a reader that does not take branches."""
+        residual = torch.zeros(self.shape, dtype=torch.float32, device=self.weights[0].device)
+        branches_norm_step(self, residual, torch.ones_like(self.weights[0]), 1.0)
+        return residual
+
+
+def branches_norm_step(nb: "NormedBranches", residual: torch.Tensor, weight: torch.Tensor, eps: float,
+                       rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """residual += the branches' sum, in 32-bit and in place, then the RMS norm of the new ``residual`` [T, H] times ``weight`` in
+    the branches' type.  With ``rows`` (int32 [R]): of those rows of the sum alone, and the residual is read only."""
+    m, h = residual.shape
+    tensors, stride = [], 0
+    for y, w in zip(nb.branches, nb.weights):
+        if tuple(y.shape) != (m, h) or tuple(w.shape) != (h,) or y.dtype != nb.dtype:
+            raise NativeError(f"branches_norm_step: branch {tuple(y.shape)} {y.dtype} / weight {tuple(w.shape)} beside a stream {(m, h)}")
+        t, parts = (None, y.parts) if isinstance(y, SliceSums) else (y, None)
+        _dev(t, parts, w)
+        _f32(w, "branch norm weight")
+        stride = m * h
+        tensors.append((t, parts, 0 if parts is None else parts.shape[0], w))
+    if len(tensors) == 1:
+        tensors.append((None, None, 0, None))
+    _dev(residual, weight, rows)
+    _f32(residual, "residual")
+    _f32(weight, "norm weight")
+    n = m
+    if rows is not None:
+        _i32(rows, "rows")
+        n = rows.shape[0]
+    out = torch.empty((n, h), dtype=nb.dtype, device=residual.device)
+    scales = list(nb.scales) + [0.0]
+    args = [a for (t, p, s, w), c in zip(tensors, scales) for a in (_ptr(t), _ptr(p), s, _ptr(w), float(c))]
+    check(kernels().pa_branches_norm_step(_stream(), _CODES[nb.dtype], *args, stride, nb.eps, _ptr(residual), _ptr(weight), _ptr(out),
+                                          _ptr(rows), n, h, float(eps)))
+    return out
+
+
 def as_tensor(x):
-    """A product that may have come back as ``SliceSums``, as a tensor."""
-    return x.materialize() if isinstance(x, SliceSums) else x
+    """A product that may have come back as ``SliceSums`` (or as ``NormedBranches``), as a tensor."""
+    return x.materialize() if isinstance(x, (SliceSums, NormedBranches)) else x
 
 
 def set_skinny_max_rows(n: int) -> None:
@@ -1105,13 +1160,15 @@ def rmsnorm_wide(x, weight: torch.Tensor, eps: float, residual: Optional[torch.T
     _f32(weight, "norm weight")
     _f32(residual, "residual")
     if x is None:
-        # nothing waits to be added: the norm of the stream's wanted rows alone, in ``out_dtype``
-        if residual is None or rows is None or out_dtype is None:
-            raise NativeError("rmsnorm_wide: without x it norms rows of the residual and needs residual, rows and out_dtype")
-        _i32(rows, "rows")
-        out = torch.empty((rows.shape[0], residual.shape[1]), dtype=out_dtype, device=weight.device)
+        # nothing waits to be added: the norm of the stream alone (of its wanted rows), in ``out_dtype``
+        if residual is None or out_dtype is None:
+            raise NativeError("rmsnorm_wide: without x it norms the residual and needs residual and out_dtype")
+        if rows is not None:
+            _i32(rows, "rows")
+        n = residual.shape[0] if rows is None else rows.shape[0]
+        out = torch.empty((n, residual.shape[1]), dtype=out_dtype, device=weight.device)
         check(kernels().pa_rmsnorm_wide(_stream(), _CODES[out_dtype], None, None, 0, 0, _ptr(residual), _ptr(weight), _ptr(out),
-                                        _ptr(rows), rows.shape[0], residual.shape[1], float(eps)))
+                                        _ptr(rows), n, residual.shape[1], float(eps)))
         return out
     m, h = x.shape
     if weight.shape != (h,) or (residual is not None and tuple(residual.shape) != (m, h)):
@@ -1676,20 +1733,23 @@ HEAD_GATES = {"sigmoid": 0, "silu": 1}
 
 
 def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor], eps: float, gate_activation: str = "sigmoid",
-                   out: Optional[torch.Tensor] = None, scale: float = 1.0) -> torch.Tensor:
-    """o float32 [T, heads, vdim]: every head over its own sqrt(mean^2 + eps), times ``weight`` (float32 [vdim], shared by
-    the heads; None: none), times act(gate) (``gate`` [T, heads * vdim] of the engine's type, rows may lie inside a
+                   out: Optional[torch.Tensor] = None, scale: float = 1.0, den: Optional[torch.Tensor] = None,
+                   floor: Optional[torch.Tensor] = None, den_eps: float = 0.0) -> torch.Tensor:
+    """o float32 [T, heads, vdim], with ``den`` and ``floor`` (float32 [T, heads]) first over max(|den|, floor) + ``den_eps``:
+    every head over its own sqrt(mean^2 + eps), times ``weight`` (float32 [vdim], shared by the heads, or [heads * vdim];
+    None: none), times act(gate) (``gate`` [T, heads * vdim] of the engine's type, rows may lie inside a
     wider tensor), times ``scale``.  Written to ``out`` (rows may lie inside a wider tensor) or a fresh [T, heads * vdim]."""
-    _dev(o, weight)
-    _f32(o, "head_norm_gate input")
-    _f32(weight, "norm weight")
+    _dev(o, weight, den, floor)
+    for v, name in ((o, "head_norm_gate input"), (weight, "norm weight"), (den, "denominator"), (floor, "denominator's floor")):
+        _f32(v, name)
     if o.dim() != 3 or not o.is_contiguous():
         raise NativeError(f"head_norm_gate: o {tuple(o.shape)} is not a contiguous [T, heads, vdim]")
     t, heads, vdim = o.shape
     if gate_activation not in HEAD_GATES:
         raise NativeError(f"head_norm_gate: gate activation {gate_activation!r} is not one of {sorted(HEAD_GATES)}")
     if not gate.is_cuda or gate.dim() != 2 or gate.stride(1) != 1 or tuple(gate.shape) != (t, heads * vdim) or \
-            (weight is not None and tuple(weight.shape) != (vdim,)):
+            (weight is not None and tuple(weight.shape) not in ((vdim,), (heads * vdim,))) or \
+            any(v is not None and tuple(v.shape) != (t, heads) for v in (den, floor)):
         raise NativeError(f"head_norm_gate: gate {tuple(gate.shape)} / weight for o {tuple(o.shape)}")
     if out is None:
         out = torch.empty((t, heads * vdim), dtype=gate.dtype, device=o.device)
@@ -1698,7 +1758,8 @@ def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.T
     if t:
         check(kernels().pa_head_norm_gate(_stream(), _code(gate), _ptr(o), gate.data_ptr(), gate.stride(0), _ptr(weight),
                                           out.data_ptr(), out.stride(0), t, heads, vdim, float(eps), HEAD_GATES[gate_activation],
-                                          float(scale)))
+                                          float(scale), 1 if weight is not None and weight.shape[0] != vdim else 0, _ptr(den), _ptr(floor),
+                                          float(den_eps)))
     return out
 
 
@@ -1746,12 +1807,13 @@ def attention_masked_mfma_supported(hd: int, vd: int, page_size: int) -> bool:
 def attention_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, group, step, window: int, keep_first: int,
                      scale: float, softcap: float = 0.0, slopes: Optional[torch.Tensor] = None,
                      sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
-                     out: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
+                     out: Optional[torch.Tensor] = None, out_scale: float = 1.0, chunk: int = 0) -> torch.Tensor:
     """Paged causal attention of one step over one cache group, any mix of portions and single tokens.  The query at
-    i sees the key at j <= i when i - j < ``window`` (0: no window) or j < ``keep_first``.  score = q.k * scale, bent
+    i sees the key at j <= i when i - j < ``window`` (0: no window) or j < ``keep_first``, and with ``chunk`` only when both
+    lie in one chunk of that many places.  score = q.k * scale, bent
     to cap * tanh(score / cap) for ``softcap`` > 0, less ``slopes``[h] * (i - j); ``sink`` [heads] joins the softmax's
-    denominator; ``gate`` [T, heads] (rows may lie inside a wider tensor): a head's output times sigmoid(gate), and
-    ``out_scale``, before rounding.  q [T, nh, hd]; K cache [pages, nkv, page, hd]; V cache [pages, nkv, vd, page].
+    denominator; ``gate`` [T, heads] or [T, heads * vd] (rows may lie inside a wider tensor): a head's output, or every one of
+    its columns, times sigmoid(gate), and ``out_scale``, before rounding.  q [T, nh, hd]; K cache [pages, nkv, page, hd]; V cache [pages, nkv, vd, page].
     Returns (or fills ``out``, whose rows may lie inside a wider tensor) [T, nh * vd].
 
     bfloat16 with keys and values of one width the matrix cores take (32, 64, 96, 128) and pages of a power of two runs
@@ -1771,7 +1833,8 @@ def attention_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             _f32(v, name)
             if tuple(v.shape) != (nh,):
                 raise NativeError(f"attention_masked: {name} {tuple(v.shape)} for {nh} heads")
-    if gate is not None and (not gate.is_cuda or gate.dtype != q.dtype or gate.dim() != 2 or tuple(gate.shape) != (t, nh) or gate.stride(1) != 1):
+    if gate is not None and (not gate.is_cuda or gate.dtype != q.dtype or gate.dim() != 2 or gate.shape[0] != t or
+                             gate.shape[1] not in (nh, nh * vd) or gate.stride(1) != 1):
         raise NativeError(f"attention_masked: gate {tuple(gate.shape)} {gate.dtype} for {t} tokens of {nh} heads")
     if out is None:
         out = torch.empty((t, nh * vd), dtype=q.dtype, device=q.device)
@@ -1784,7 +1847,8 @@ def attention_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                                        float(softcap), _ptr(slopes), _ptr(sink), gate.data_ptr() if gate is not None else None,
                                        gate.stride(0) if gate is not None else 0, float(out_scale), _ptr(getattr(step, "cu_q", None)),
                                        _ptr(getattr(step, "context_lens", None)), int(getattr(step, "num_seqs", 0)),
-                                       int(getattr(step, "max_q_len", 0) or getattr(step, "max_prefill_q", 0) or 1), nv))
+                                       int(getattr(step, "max_q_len", 0) or getattr(step, "max_prefill_q", 0) or 1), nv, int(chunk),
+                                       1 if gate is not None and gate.shape[1] != nh else 0))
     return out
 
 
@@ -1879,24 +1943,31 @@ def pair_embed(ids: torch.Tensor, step, prev_state: torch.Tensor, table: torch.T
     return out
 
 
-def time_conv_add(h: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tensor], step) -> torch.Tensor:
-    """h + conv(h) with conv(h)_t = sum_j w[j] h_(t - taps + 1 + j) over time within each sequence, zeros before its
-    start.  h [T, C]; ``weight`` float32 [taps, C] (a tap's weights side by side: the stored [C, taps] transposed);
-    ``state`` float32 [slots, taps - 1, C]: a request's last taps - 1 inputs, read for the places before the portion and
-    moved on afterwards."""
-    _dev(h, weight, state, step.seq_of_token, step.cu_q, step.state_slots)
-    _f32(weight, "convolution weight")
-    _f32(state, "carried inputs")
+def time_conv(h: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tensor], step, in_bias: Optional[torch.Tensor] = None,
+              bias: Optional[torch.Tensor] = None, activation: Optional[str] = None, add_input: bool = False) -> torch.Tensor:
+    """act(conv(h + in_bias) + bias), plus h + in_bias where ``add_input``: conv(x)_t = sum_j w[j] x_(t - taps + 1 + j) over time
+    within each sequence, zeros before its start.  h [T, C] (rows may lie inside a wider tensor); ``weight`` float32 [taps, C]
+    (a tap's weights side by side: the stored [C, taps] transposed); ``activation`` None or ``"silu"``; ``state`` float32
+    [slots, taps - 1, C]: a request's last taps - 1 inputs, read for the places before the portion and moved on afterwards.
+    All of it in 32-bit, rounded once: [T, C] of h's type."""
+    _dev(weight, state, in_bias, bias, step.seq_of_token, step.cu_q, step.state_slots)
+    for t, name in ((weight, "convolution weight"), (state, "carried inputs"), (in_bias, "input bias"), (bias, "convolution bias")):
+        _f32(t, name)
     t, c = h.shape
     taps = weight.shape[0]
-    if weight.dim() != 2 or weight.shape[1] != c or not h.is_contiguous() or \
-            (taps > 1 and (state is None or tuple(state.shape[1:]) != (taps - 1, c))):
-        raise NativeError(f"time_conv_add: h {tuple(h.shape)} / weight {tuple(weight.shape)} / state "
+    if weight.dim() != 2 or weight.shape[1] != c or not h.is_cuda or h.stride(1) != 1 or \
+            (taps > 1 and (state is None or tuple(state.shape[1:]) != (taps - 1, c))) or \
+            any(v is not None and tuple(v.shape) != (c,) for v in (in_bias, bias)):
+        raise NativeError(f"time_conv: h {tuple(h.shape)} / weight {tuple(weight.shape)} / state "
                           f"{None if state is None else tuple(state.shape)}")
-    out = torch.empty_like(h)
+    if activation not in (None, "silu"):
+        raise NativeError(f"time_conv: activation {activation!r} is not one of None, 'silu'")
+    out = torch.empty((t, c), dtype=h.dtype, device=h.device)
     # a step of single tokens alone: every thread moves its sequence's carried inputs on itself, no second launch
-    check(kernels().pa_time_conv_add(_stream(), _code(h), _ptr(h), _ptr(weight), _ptr(state), _ptr(step.seq_of_token), _ptr(step.cu_q),
-                                     _ptr(step.state_slots), _ptr(out), t, int(step.num_seqs), c, taps,
+    if t:
+        check(kernels().pa_time_conv(_stream(), _code(h), h.data_ptr(), h.stride(0), _ptr(weight), _ptr(in_bias), _ptr(bias), _ptr(state),
+                                     _ptr(step.seq_of_token), _ptr(step.cu_q), _ptr(step.state_slots), _ptr(out), c, t,
+                                     int(step.num_seqs), c, taps, 1 if activation == "silu" else 0, 1 if add_input else 0,
                                      1 if int(getattr(step, "max_q_len", 0)) == 1 else 0))
     return out
 
@@ -1925,16 +1996,18 @@ def stream_add_branches_(x: torch.Tensor, a: torch.Tensor, b: Optional[torch.Ten
 
 def qkv_rope_prepare(p: torch.Tensor, q_off: int, k_off: int, v_off: int, inv_freq: Optional[torch.Tensor], positions: torch.Tensor,
                      slots: Optional[torch.Tensor], k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], nq: int,
-                     nk: int, nv: int, hd: int, vd: int, rot: int, pairs: bool, q_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     nk: int, nv: int, hd: int, vd: int, rot: int, pairs: bool, q_scale: Optional[torch.Tensor] = None,
+                     unit_eps: Optional[float] = None) -> torch.Tensor:
     """From the merged projection ``p`` [T, width]: the queries [T, nq, hd]; ``nk`` key heads of ``hd`` into K
     [pages, nk, page, hd] and ``nv`` value heads of ``vd`` into V [pages, nv, vd, page] at ``slots`` (None: queries
     only).  The first ``rot`` dimensions of every query and key head are turned by position * inv_freq[i], dimension i
-    with i + rot / 2, or with ``pairs`` 2i with 2i + 1; ``q_scale`` [nq]: a number per query head."""
-    _dev(p, inv_freq, positions, slots, k_cache, v_cache, q_scale)
+    with i + rot / 2, or with ``pairs`` 2i with 2i + 1; ``unit_eps``: then every query and key head over its own
+    sqrt(mean^2 + unit_eps); ``q_scale`` [nq]: a number per query head."""
+    _dev(inv_freq, positions, slots, k_cache, v_cache, q_scale)
     _f32(inv_freq, "rotary frequencies")
     _f32(q_scale, "query scales")
     _i32(positions, "positions")
-    if p.dim() != 2 or p.stride(1) != 1:
+    if not p.is_cuda or p.dim() != 2 or p.stride(1) != 1:
         raise NativeError(f"qkv_rope_prepare: projection {tuple(p.shape)} with strides {p.stride()}")
     t = p.shape[0]
     if rot and (inv_freq is None or tuple(inv_freq.shape) != (rot // 2,)):
@@ -1955,7 +2028,8 @@ def qkv_rope_prepare(p: torch.Tensor, q_off: int, k_off: int, v_off: int, inv_fr
         check(kernels().pa_qkv_rope_prepare(_stream(), _code(p), p.data_ptr(), p.stride(0), int(q_off), int(k_off), int(v_off),
                                             _ptr(inv_freq), _ptr(positions), _ptr(slots), _ptr(q_scale), _ptr(q),
                                             _ptr(k_cache) if caching else None, _ptr(v_cache) if caching else None, t, nq, nk, nv,
-                                            hd, vd, int(rot), 1 if pairs else 0, page))
+                                            hd, vd, int(rot), 1 if pairs else 0, page, 0 if unit_eps is None else 1,
+                                            float(unit_eps or 0.0)))
     return q
 
 
@@ -2107,19 +2181,19 @@ def attention_wide_supported(kd: int, vd: int, page_size: int) -> bool:
     return bool(kernels().pa_attn_wide_supports(int(kd), int(vd), int(page_size)))
 
 
-SHARED_SPLIT_KEYS = (128, 256, 512, 1024, 2048, 4096)   # keys a split of a single token's context, all heads over one key head
+SHARED_SPLIT_KEYS = (128, 256, 512, 1024, 2048, 4096)   # keys a split of a single token's context
 # The shortest split whose launch stays within one round of the chip (a workgroup a compute unit), keys of 256 and four
 # value heads of 128 under a window of 1,024, the merge included: 8 sequences 12.1 us in splits of 128, 15.1 of 256; 32
 # sequences 28.2, 21.9 and 26.1 us in splits of 128, 256 and 512; 64 sequences 38.5, 34.6, 26.9 and 38.9 to 1,024
 SHARED_SPLIT_WORKGROUPS = 256
 
 
-def shared_split_plan(n_seqs: int, heads: int, max_context: int, window: int, page_size: int):
-    """(keys a split, most splits a sequence) for a step of ``n_seqs`` single tokens whose contexts are at most
-    ``max_context`` tokens.  It follows the context rounded up (``decode_context_bound``), so that a step run directly and
+def shared_split_plan(n_seqs: int, heads: int, max_context: int, window: int, page_size: int, key_heads: int = 1):
+    """(keys a split, most splits a sequence) for a step of ``n_seqs`` single tokens of ``heads`` heads over ``key_heads`` whose
+    contexts are at most ``max_context`` tokens, of which ``window`` are seen (0: all).  It follows the context rounded up (``decode_context_bound``), so that a step run directly and
     one replayed from a graph are cut alike."""
     bound = decode_context_bound(max_context, page_size)
-    tiles = -(-int(heads) // 16)
+    tiles = key_heads * -(-int(heads) // (16 * key_heads))
 
     def splits(keys):
         span = min(bound, window) if window else bound
@@ -2129,11 +2203,13 @@ def shared_split_plan(n_seqs: int, heads: int, max_context: int, window: int, pa
 
 
 def attention_wide(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, group, step, window: int, scale: float,
-                   sink: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                   sink: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None, chunk: int = 0,
+                   gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Paged causal attention of one step on the matrix cores for key and value widths of any size (``attention_wide_supported``),
     bfloat16: q [T, nh, kd], K [pages, nkv, page, kd], V [pages, nv, vd, page] (value heads as in ``attention_masked``), a window
-    (0: none), a sink per head.  Portions are tiles of tokens; where all heads read one key head, single tokens have a kernel
-    that reads every key once for all heads.  Returns (or fills ``out``, whose rows may lie inside a wider tensor) [T, nh * vd]."""
+    (0: none), chunks (``chunk`` > 0: a query sees its own chunk of that many places alone), a sink per head, a gate (``gate``
+    [T, nh * vd], rows may lie inside a wider tensor: the output times sigmoid(gate) before it is rounded).  Portions are tiles
+    of tokens; single tokens have a kernel that reads every key once for all heads over it.  Returns (or fills ``out``, whose rows may lie inside a wider tensor) [T, nh * vd]."""
     _dev(q, k_cache, v_cache, sink, group.block_table)
     t, nh, kd = q.shape
     pages, nkv, page, _ = k_cache.shape
@@ -2147,23 +2223,23 @@ def attention_wide(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
         out = torch.empty((t, nh * vd), dtype=q.dtype, device=q.device)
     elif out.dtype != q.dtype or tuple(out.shape) != (t, nh * vd) or out.stride(1) != 1:
         raise NativeError(f"attention_wide: out {tuple(out.shape)} {out.dtype}")
+    if gate is not None and (not gate.is_cuda or gate.dtype != q.dtype or tuple(gate.shape) != (t, nh * vd) or gate.stride(1) != 1):
+        raise NativeError(f"attention_wide: gate {tuple(gate.shape)} {gate.dtype} for {t} tokens of {nh} heads of {vd}")
     args = (_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(group.block_table), group.block_table.shape[1])
+    more = (int(chunk), None, 0) if gate is None else (int(chunk), gate.data_ptr(), gate.stride(0))
     if step.n_decode:
         every = step.n_prefill == 0 and step.n_decode == step.num_seqs
         ids = None if every else _ptr(step.decode_seqs)
-        if nkv == 1:
-            keys, splits = shared_split_plan(step.n_decode, nh, step.max_decode_context, window, page)
-            work = torch.empty(int(kernels().pa_attn_shared_workspace(step.n_decode, nh, vd, splits)), dtype=torch.float32, device=q.device)
-            check(kernels().pa_attn_shared(_stream(), *args, ids, _ptr(step.cu_q), _ptr(step.context_lens), out.data_ptr(), out.stride(0),
-                                           _ptr(work), step.n_decode, nh, nv, kd, vd, page, int(window), float(scale), _ptr(sink), keys,
-                                           splits))
-        else:
-            check(kernels().pa_attn_wide(_stream(), *args, ids, _ptr(step.cu_q), _ptr(step.context_lens), out.data_ptr(), out.stride(0),
-                                         step.n_decode, 1, nh, nkv, nv, kd, vd, page, int(window), float(scale), _ptr(sink)))
+        seen = min(window, chunk) if window and chunk else (window or chunk)
+        keys, splits = shared_split_plan(step.n_decode, nh, step.max_decode_context, seen, page, nkv)
+        work = torch.empty(int(kernels().pa_attn_shared_workspace(step.n_decode, nh, vd, splits)), dtype=torch.float32, device=q.device)
+        check(kernels().pa_attn_shared(_stream(), *args, ids, _ptr(step.cu_q), _ptr(step.context_lens), out.data_ptr(), out.stride(0),
+                                       _ptr(work), step.n_decode, nh, nkv, nv, kd, vd, page, int(window), float(scale), _ptr(sink), keys,
+                                       splits, *more))
     if step.n_prefill:
         check(kernels().pa_attn_wide(_stream(), *args, _ptr(step.prefill_seqs), _ptr(step.cu_q), _ptr(step.context_lens), out.data_ptr(),
                                      out.stride(0), step.n_prefill, int(step.max_prefill_q), nh, nkv, nv, kd, vd, page, int(window),
-                                     float(scale), _ptr(sink)))
+                                     float(scale), _ptr(sink), *more))
     return out
 
 
@@ -2244,4 +2320,170 @@ def gated_linear_attention(p: torch.Tensor, q_off: int, k_off: int, v_off: int, 
             work = torch.empty((max(words, 1),), dtype=torch.float32, device=p.device)
             check(kernels().pa_gla_attn_chunked(_stream(), *cols, _ptr(alpha), *where, _ptr(step.prefill_seqs), _ptr(out), _ptr(work),
                                                 step.n_prefill, t, int(step.max_prefill_q), heads, dim, vdim, q_scale, int(chunk)))
+    return out
+
+
+# ---------------------------------------------------------------------------
+# Recurrences with one decay a token and head (Mamba-2, mLSTM); a gated linear recurrence a channel
+def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, out: Optional[torch.Tensor] = None,
+                     scale: float = 1.0) -> torch.Tensor:
+    """y * silu(z), in ``groups`` equal consecutive parts of a row each over its own sqrt(mean^2 + eps), times ``weight`` and
+    ``scale``: y float32 [T, N], z [T, N] of the engine's type (rows may lie inside a wider tensor), ``weight`` float32 [N]."""
+    _dev(y, weight)
+    _f32(y, "gated_group_norm input")
+    _f32(weight, "norm weight")
+    t, n = y.shape
+    if not z.is_cuda or tuple(z.shape) != (t, n) or z.stride(1) != 1 or tuple(weight.shape) != (n,):
+        raise NativeError(f"gated_group_norm: y {tuple(y.shape)} / z {tuple(z.shape)} / weight {tuple(weight.shape)}")
+    if out is None:
+        out = torch.empty((t, n), dtype=z.dtype, device=y.device)
+    elif out.dtype != z.dtype or tuple(out.shape) != (t, n) or out.stride(1) != 1:
+        raise NativeError(f"gated_group_norm: out {tuple(out.shape)} {out.dtype}")
+    if t:
+        check(kernels().pa_gated_group_norm(_stream(), _code(z), _ptr(y), z.data_ptr(), z.stride(0), _ptr(weight), out.data_ptr(), out.stride(0),
+                                            t, n, int(groups), float(eps), float(scale)))
+    return out
+
+
+DECAY_SCAN_CHUNKED = True   # portions of a bfloat16 engine on the matrix cores in chunks, where the widths allow it
+
+
+def _scan_state(state, n_state, heads: int, dim: int, vdim: int, what: str) -> None:
+    _dev(state, n_state)
+    _f32(state, "state")
+    _f32(n_state, "sum of keys")
+    if state.dim() != 4 or tuple(state.shape[1:]) != (heads, dim, vdim) or \
+            (n_state is not None and tuple(n_state.shape) != (state.shape[0], heads, dim)):
+        raise NativeError(f"{what}: state {tuple(state.shape)} for {heads} heads of {dim} and {vdim}")
+
+
+def _decay_scan_portions(p, cols, la, b, state, n_state, skip, q_scale, step, out, den, heads, group, dim, vdim) -> None:
+    t = p.shape[0]
+    where = (_ptr(la), _ptr(b), _ptr(state), _ptr(n_state), _ptr(skip), float(q_scale), _ptr(step.state_slots), _ptr(step.cu_q))
+    if DECAY_SCAN_CHUNKED and p.dtype == torch.bfloat16 and step.n_prefill > 0 and \
+            kernels().pa_decay_scan_chunked_supports(p.data_ptr(), p.stride(0), *cols, dim, vdim):
+        words = kernels().pa_decay_scan_chunked_workspace(step.n_prefill, t, heads, dim, vdim, 0 if n_state is None else 1)
+        work = torch.empty((max(words, 1),), dtype=torch.float32, device=p.device)
+        check(kernels().pa_decay_scan_chunked(_stream(), p.data_ptr(), p.stride(0), *cols, *where, _ptr(step.prefill_seqs), _ptr(out), _ptr(den),
+                                              _ptr(work), step.n_prefill, t, int(step.max_prefill_q), heads, group, dim, vdim))
+        return
+    check(kernels().pa_decay_scan(_stream(), _code(p), p.data_ptr(), p.stride(0), *cols, *where, _ptr(out), _ptr(den), step.num_seqs, t, heads,
+                                  group, dim, vdim, 2))
+
+
+def ssd_scan(p: torch.Tensor, q_off: int, k_off: int, v_off: int, dt: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor,
+             skip: torch.Tensor, state: torch.Tensor, step, heads: int, groups: int, dim: int, vdim: int) -> torch.Tensor:
+    """Per head, with s = softplus(dt + dt_bias): S <- exp(-exp(a_log) s) S + s k v^T, y = S^T q + skip v.
+
+    ``p`` [T, width]: a token's q and k [groups, dim] (head h reads group h / (heads / groups)) and v [heads, vdim] start at the
+    given columns; ``dt`` [T, heads] of p's type (rows may lie inside a wider tensor); state float32 [slots, heads, dim, vdim],
+    read and left by the step's sequences through ``step.state_slots``.  Returns float32 [T, heads, vdim].  Portions of a
+    bfloat16 engine run in chunks on the matrix cores (the same sums up to rounding, in another order)."""
+    _dev(dt_bias, a_log, skip)
+    for v, name in ((dt_bias, "step bias"), (a_log, "A_log"), (skip, "skip")):
+        _f32(v, name)
+        if tuple(v.shape) != (heads,):
+            raise NativeError(f"ssd_scan: {name} {tuple(v.shape)} for {heads} heads")
+    _scan_state(state, None, heads, dim, vdim, "ssd_scan")
+    t = p.shape[0]
+    if not p.is_cuda or p.dim() != 2 or p.stride(1) != 1 or heads % groups or not dt.is_cuda or tuple(dt.shape) != (t, heads) or \
+            dt.stride(1) != 1 or dt.dtype != p.dtype or max(q_off, k_off) + groups * dim > p.shape[1] or v_off + heads * vdim > p.shape[1]:
+        raise NativeError(f"ssd_scan: p {tuple(p.shape)} / dt {tuple(dt.shape)} for {heads} heads over {groups} groups of {dim} and {vdim}")
+    out = torch.empty((t, heads, vdim), dtype=torch.float32, device=p.device)
+    cols = (int(q_off), int(k_off), int(v_off))
+    if t and step.n_decode:
+        check(kernels().pa_decay_scan_step(_stream(), _code(p), p.data_ptr(), p.stride(0), *cols, dt.data_ptr(), max(dt.stride(0), heads), 0, 0,
+                                           _ptr(dt_bias), None, _ptr(a_log), 0.0, None, None, _ptr(state), None, _ptr(skip), 1.0,
+                                           _ptr(step.state_slots), _ptr(step.cu_q), _ptr(out), None, step.num_seqs, heads, heads // groups,
+                                           dim, vdim))
+    if t and step.n_prefill:
+        la, b = torch.empty((2, t, heads), dtype=torch.float32, device=p.device)
+        check(kernels().pa_ssd_gates(_stream(), _code(dt), dt.data_ptr(), max(dt.stride(0), heads), 0, _ptr(dt_bias), _ptr(a_log), _ptr(la),
+                                     _ptr(b), t, heads))
+        _decay_scan_portions(p, cols, la, b, state, None, skip, 1.0, step, out, None, heads, heads // groups, dim, vdim)
+    return out
+
+
+DECAY_SCAN_COLUMNS = 64   # value columns a workgroup of the single tokens' kernel
+
+
+def mlstm_max_copies(vdim: int) -> int:
+    """Copies of the running maximum a head's state holds: one per workgroup that reads it in a step of single tokens."""
+    return -(-int(vdim) // DECAY_SCAN_COLUMNS) + 1
+
+
+def mlstm_scan(p: torch.Tensor, q_off: int, k_off: int, v_off: int, i_off: int, f_off: int, i_bias: torch.Tensor, f_bias: torch.Tensor,
+               cap: float, state: torch.Tensor, n_state: torch.Tensor, m_state: torch.Tensor, step, heads: int, dim: int, vdim: int,
+               q_scale: float):
+    """The matrix memory of xLSTM.  Per head, with i = c tanh((z_i + i_bias) / c), f = log sigmoid(c tanh((z_f + f_bias) / c)), c = ``cap``,
+    and a running maximum m_t = max(f + m_(t-1), i):
+
+        S <- e^(f + m_(t-1) - m_t) S + e^(i - m_t) k v^T,   n likewise with k alone
+
+    ``p`` [T, width] (rows may lie inside a wider tensor) holds q, k [heads, dim], v [heads, vdim], z_i and z_f [heads] from the given
+    columns on; the state (S float32 [slots, heads, dim, vdim], n [slots, heads, dim], m [slots, heads, copies]: ``mlstm_max_copies``
+    equal numbers) is read and left by the step's sequences.  Returns float32 (S^T q q_scale [T, heads, vdim], n . q q_scale
+    [T, heads], e^(-m) [T, heads]).  Portions of a bfloat16 engine run in chunks on the matrix cores."""
+    _dev(i_bias, f_bias, m_state)
+    for v, name in ((i_bias, "gate bias"), (f_bias, "gate bias")):
+        _f32(v, name)
+        if tuple(v.shape) != (heads,):
+            raise NativeError(f"mlstm_scan: {name} {tuple(v.shape)} for {heads} heads")
+    _f32(m_state, "running maximum")
+    _scan_state(state, n_state, heads, dim, vdim, "mlstm_scan")
+    t = p.shape[0]
+    if not p.is_cuda or p.dim() != 2 or p.stride(1) != 1 or max(q_off, k_off) + heads * dim > p.shape[1] or v_off + heads * vdim > p.shape[1] or \
+            max(i_off, f_off) + heads > p.shape[1] or tuple(m_state.shape) != (state.shape[0], heads, mlstm_max_copies(vdim)):
+        raise NativeError(f"mlstm_scan: p {tuple(p.shape)} / m {tuple(m_state.shape)} for {heads} heads of {dim} and {vdim}")
+    if int(kernels().pa_mlstm_max_copies(vdim)) != mlstm_max_copies(vdim):
+        raise NativeError("mlstm_scan: the kernel library cuts a head's columns otherwise; rebuild it")
+    out = torch.empty((t, heads, vdim), dtype=torch.float32, device=p.device)
+    den, floor = torch.empty((2, t, heads), dtype=torch.float32, device=p.device)
+    cols = (int(q_off), int(k_off), int(v_off))
+    where = (_ptr(step.state_slots), _ptr(step.cu_q))
+    if t and step.n_decode:
+        check(kernels().pa_decay_scan_step(_stream(), _code(p), p.data_ptr(), p.stride(0), *cols, p.data_ptr(), p.stride(0), int(i_off), int(f_off),
+                                           _ptr(i_bias), _ptr(f_bias), None, float(cap), _ptr(m_state), _ptr(floor), _ptr(state), _ptr(n_state),
+                                           None, float(q_scale), *where, _ptr(out), _ptr(den), step.num_seqs, heads, 1, dim, vdim))
+    if t and step.n_prefill:
+        la, b = torch.empty((2, t, heads), dtype=torch.float32, device=p.device)
+        check(kernels().pa_mlstm_gates(_stream(), _code(p), p.data_ptr(), p.stride(0), int(i_off), int(f_off), _ptr(i_bias), _ptr(f_bias),
+                                       float(cap), _ptr(m_state), *where, _ptr(la), _ptr(b), _ptr(floor), step.num_seqs, heads, vdim, 2))
+        _decay_scan_portions(p, cols, la, b, state, n_state, None, q_scale, step, out, den, heads, 1, dim, vdim)
+    return out, den, floor
+
+
+def lru_scan(u: torch.Tensor, wr: torch.Tensor, wi: torch.Tensor, br: torch.Tensor, bi: torch.Tensor, rate: torch.Tensor, state: torch.Tensor,
+             y: torch.Tensor, y_bias: Optional[torch.Tensor], step, out: Optional[torch.Tensor] = None, out_scale: float = 1.0,
+             activation: str = "gelu_tanh") -> torch.Tensor:
+    """A gated linear recurrence on every channel: r = sigmoid(wr[n] u_n + br), i = sigmoid(wi[n] u_n + bi) per block n of channels,
+    log a = -r rate, S <- a S + sqrt(1 - a^2) i u, out = S act(y + y_bias) out_scale.
+
+    u [T, width]; ``wr``, ``wi`` [blocks, size, size] of u's type; biases and ``rate`` float32 [width]; state float32 [slots, width],
+    read and left by the step's sequences; ``y`` [T, width] (rows may lie inside a wider tensor).  Gates, decays and state are 32-bit."""
+    _dev(u, wr, wi, br, bi, rate, state, y_bias)
+    for v, name in ((br, "gate bias"), (bi, "gate bias"), (rate, "rate"), (state, "state"), (y_bias, "bias")):
+        _f32(v, name)
+    t, width = u.shape
+    blocks = wr.shape[0]
+    if wr.shape != wi.shape or wr.dim() != 3 or wr.shape[1] != wr.shape[2] or blocks * wr.shape[1] != width or wr.dtype != u.dtype or \
+            wi.dtype != u.dtype or any(tuple(v.shape) != (width,) for v in (br, bi, rate)) or tuple(state.shape[1:]) != (width,) or \
+            not y.is_cuda or tuple(y.shape) != (t, width) or y.stride(1) != 1 or y.dtype != u.dtype:
+        raise NativeError(f"lru_scan: u {tuple(u.shape)} / blocks {tuple(wr.shape)} / state {tuple(state.shape)} / y {tuple(y.shape)}")
+    act = gate_activation_code(activation)
+    if out is None:
+        out = torch.empty((t, width), dtype=u.dtype, device=u.device)
+    elif out.dtype != u.dtype or tuple(out.shape) != (t, width) or out.stride(1) != 1:
+        raise NativeError(f"lru_scan: out {tuple(out.shape)} {out.dtype}")
+    if not t:
+        return out
+    a, x = torch.empty((2, t, width), dtype=torch.float32, device=u.device)
+    tail = (y.data_ptr(), max(y.stride(0), width), _ptr(y_bias), act, _ptr(a), _ptr(x), out.data_ptr(), max(out.stride(0), width), float(out_scale))
+    check(kernels().pa_lru_gates(_stream(), _code(u), _ptr(u), _ptr(wr), _ptr(wi), _ptr(br), _ptr(bi), _ptr(rate), _ptr(state),
+                                 _ptr(step.seq_of_token), _ptr(step.state_slots), _ptr(step.cu_q), *tail, t, width, blocks))
+    if step.n_prefill:
+        words = kernels().pa_lru_scan_workspace(step.n_prefill, t, width)
+        work = torch.empty((max(words, 1),), dtype=torch.float32, device=u.device)
+        check(kernels().pa_lru_scan(_stream(), _code(u), _ptr(u), _ptr(rate), _ptr(state), _ptr(step.state_slots), _ptr(step.cu_q),
+                                    _ptr(step.prefill_seqs), *tail, _ptr(work), step.n_prefill, t, int(step.max_prefill_q), width))
     return out

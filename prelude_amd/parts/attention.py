@@ -165,15 +165,25 @@ class KeptFirstKVCacheSpec(KVCacheSpec):
     keep_first: int = 0
 
 
+@dataclasses.dataclass(frozen=True)
+class ChunkedKVCacheSpec(KVCacheSpec):
+    """Keys and values in pages where a position sees back to the start of its own chunk of ``chunk`` places: a chunk's pages are
+    given back when the next one begins (``window`` is the chunk's size)."""
+    chunk: int = 0
+
+
 @register_part("mixer", "windowed_attention")
 class WindowedAttention(Mixer):
-    """Grouped-query attention without rotation whose mask is a window that keeps the first tokens: the query at i
-    sees the key at j <= i when i - j < ``window`` (0: no window) or j < ``keep_first``.  Values have a width of their
-    own.  Optional, each a parameter: queries and keys brought to unit RMS over the whole projection (all heads at once)
+    """Grouped-query attention whose mask is a window that keeps the first tokens: the query at i
+    sees the key at j <= i when i - j < ``window`` (0: no window) or j < ``keep_first``; or chunks (``chunk`` > 0): it sees the
+    keys of its own chunk of that many places alone, counted from the sequence's start.  Values have a width of their
+    own.  Optional, each a parameter: the first ``rotary_dim`` dimensions of every query and key head turned in pairs by position
+    (``position``); every query and key head over its own sqrt(mean^2 + eps) behind that (``qk_norm="unit"``, no weight); queries and keys brought to unit RMS over the whole projection (all heads at once)
     times a weight of that size (``qk_norm="whole"``); scores bent to cap * tanh(score / cap) (``score_cap``); a bias by
     distance, slope_h (i - j) taken off the score with slope_h = 2^(-``slope_exponent`` (h + 1) / heads)
     (``slope_exponent`` > 0); a learned sink per head in the softmax's denominator (``sink="learned"``); a gate per
-    head, the head's output times sigmoid(W_g x)_h (``head_gate``).
+    head, the head's output times sigmoid(W_g x)_h (``head_gate``), or one per output column, all heads' outputs side by side
+    times sigmoid(W_g x) (``output_gate``).
 
     ``cache_window`` / ``cache_keep_first``: the mask the cache is kept for, where it is wider than this layer's own
     because other layers read the same keys (``window`` 0 = everything)."""
@@ -183,13 +193,26 @@ class WindowedAttention(Mixer):
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, scale: float,
                  window: int = 0, keep_first: int = 0, qk_norm: Optional[str] = None, norm_eps: float = 1e-6,
                  score_cap: float = 0.0, slope_exponent: float = 0.0, sink: Optional[str] = None, head_gate: bool = False,
-                 own_keys: bool = True, cache_window: Optional[int] = None, cache_keep_first: Optional[int] = None):
+                 own_keys: bool = True, cache_window: Optional[int] = None, cache_keep_first: Optional[int] = None,
+                 chunk: int = 0, position: Optional[str] = None, rotary_dim: int = 0, output_gate: bool = False):
         if num_heads % num_kv_heads:
             raise PartError(f"windowed_attention: {num_heads} heads are not a multiple of {num_kv_heads} KV heads")
         if not (1 <= head_dim <= 256 and 1 <= value_dim <= 256):
             raise PartError(f"windowed_attention: key width {head_dim} or value width {value_dim} is outside 1..256")
-        if qk_norm not in (None, "whole"):
-            raise PartError(f"windowed_attention: qk_norm {qk_norm!r} is not one of None, 'whole'")
+        if qk_norm not in (None, "whole", "unit"):
+            raise PartError(f"windowed_attention: qk_norm {qk_norm!r} is not one of None, 'whole', 'unit'")
+        if chunk < 0 or (chunk and (window or keep_first or not own_keys)):
+            raise PartError(f"windowed_attention: chunks of {chunk} places go without a window, kept first tokens and another layer's keys")
+        if head_gate and output_gate:
+            raise PartError("windowed_attention: a gate per head or one per output column")
+        self.chunk, self.output_gate = int(chunk), bool(output_gate)
+        self.position = position
+        self.rotary_dim = int(rotary_dim or 0) if position else 0
+        if self.rotary_dim % 2 or self.rotary_dim > head_dim:
+            raise PartError(f"windowed_attention: {rotary_dim} rotated dimensions of a head of {head_dim}")
+        if qk_norm == "whole" and self.rotary_dim:
+            raise PartError("windowed_attention: a norm over the whole projection goes without rotation")
+        self.rope = None
         if sink not in (None, "learned"):
             raise PartError(f"windowed_attention: sink {sink!r} is not one of None, 'learned'")
         if window < 0 or keep_first < 0 or score_cap < 0 or slope_exponent < 0:
@@ -207,6 +230,15 @@ class WindowedAttention(Mixer):
                                   self.cache_keep_first < self.keep_first):
             raise PartError("windowed_attention: the cache's mask must hold everything this layer's mask sees")
         self.w_in = self.w_o = self.q_norm = self.k_norm = self.sinks = self.slopes = None
+
+    def bind(self, shared):
+        if self.position is not None:
+            if self.position not in shared:
+                raise PartError(f"windowed_attention: the model has no position encoding named {self.position!r}")
+            self.rope = shared[self.position]
+            if getattr(self.rope, "rotary_dim", None) != self.rotary_dim or not hasattr(self.rope, "inv_freq"):
+                raise PartError(f"windowed_attention: position encoding {self.position!r} must give the frequencies of "
+                                f"{self.rotary_dim} rotated dimensions")
 
     # ---- sizes of its columns in the projection of its input ----
     @property
@@ -226,7 +258,13 @@ class WindowedAttention(Mixer):
         """Width of what ``mix`` leaves for the output projection."""
         return self.num_heads * self.value_dim
 
+    @property
+    def ng(self) -> int:
+        return self.mixed_size if self.output_gate else (self.num_heads if self.head_gate else 0)
+
     def cache_spec(self):
+        if self.chunk:
+            return ChunkedKVCacheSpec(self.num_kv_heads, self.head_dim, self.chunk, self.value_dim, self.chunk)
         if self.cache_window and self.cache_keep_first:
             return KeptFirstKVCacheSpec(self.num_kv_heads, self.head_dim, self.cache_window, self.value_dim, self.cache_keep_first)
         return KVCacheSpec(self.num_kv_heads, self.head_dim, self.cache_window, self.value_dim)
@@ -236,20 +274,20 @@ class WindowedAttention(Mixer):
         t = {"q": TensorReq((self.nq, h), MATRIX), "o": TensorReq((h, self.mixed_size), MATRIX)}
         if self.own_keys:
             t.update({"k": TensorReq((self.nk, h), MATRIX), "v": TensorReq((self.nv, h), MATRIX)})
-        if self.qk_norm:
+        if self.qk_norm == "whole":
             t["q.norm"] = TensorReq((self.nq,), NORM)
             if self.own_keys:
                 t["k.norm"] = TensorReq((self.nk,), NORM)
         if self.sink:
             t["sink"] = TensorReq((self.num_heads,), VECTOR)
-        if self.head_gate:
-            t["g"] = TensorReq((self.num_heads, h), MATRIX)
+        if self.ng:
+            t["g"] = TensorReq((self.ng, h), MATRIX)
         return t
 
     def input_rows(self, tensors) -> torch.Tensor:
         """The rows of the product of its input this mixer wants, [q | k | v | gate]; keeps its other tensors."""
-        rows = [tensors["q"]] + ([tensors["k"], tensors["v"]] if self.own_keys else []) + ([tensors["g"]] if self.head_gate else [])
-        if self.qk_norm:
+        rows = [tensors["q"]] + ([tensors["k"], tensors["v"]] if self.own_keys else []) + ([tensors["g"]] if self.ng else [])
+        if self.qk_norm == "whole":
             self.q_norm = tensors["q.norm"]
             self.k_norm = tensors["k.norm"] if self.own_keys else None
         self.sinks = tensors["sink"] if self.sink else None
@@ -271,14 +309,32 @@ class WindowedAttention(Mixer):
                             "reads another's")
         nh, nkv, hd, vd = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
         g = step.kv[cache.group]
-        q = K.qkv_prepare(p, off, off + self.nq, off + self.nq + self.nk, self.q_norm, self.k_norm,
-                          g.slots if write_cache else None, cache.k, cache.v, nh, nkv, hd, vd, self.norm_eps)
-        gate = p[:, off + self.nq + self.nk + self.nv: off + self.nq + self.nk + self.nv + nh] if self.head_gate else None
-        if not self.keep_first and self.slopes is None and gate is None and vd == hd and out is None and out_scale == 1.0:
+        k_off, v_off, g_off = off + self.nq, off + self.nq + self.nk, off + self.nq + self.nk + self.nv
+        slots = g.slots if write_cache else None
+        if self.rope is not None or self.qk_norm == "unit":
+            q = K.qkv_rope_prepare(p, off, k_off, v_off, self.rope.inv_freq if self.rope is not None else None, step.positions, slots, cache.k,
+                                   cache.v, nh, nkv, nkv, hd, vd, self.rotary_dim, True, unit_eps=self.norm_eps if self.qk_norm == "unit" else None)
+        else:
+            q = K.qkv_prepare(p, off, k_off, v_off, self.q_norm, self.k_norm, slots, cache.k, cache.v, nh, nkv, hd, vd, self.norm_eps)
+        gate = p[:, g_off: g_off + self.ng] if self.ng else None
+        if self.on_matrix_cores(q, cache, gate, out, out_scale):
+            return K.attention_wide(q, cache.k, cache.v, g, step, self.window, self.scale, self.sinks, out, self.chunk, gate)
+        if not self.keep_first and self.slopes is None and gate is None and not self.chunk and vd == hd and out is None and out_scale == 1.0:
             o = K.attention(q, cache.k, cache.v, g, step, self.window, self.scale, self.score_cap, sink=self.sinks)
             return o.view(o.shape[0], nh * vd)
         return K.attention_masked(q, cache.k, cache.v, g, step, self.window, self.keep_first, self.scale, self.score_cap,
-                                  self.slopes, self.sinks, gate, out, out_scale)
+                                  self.slopes, self.sinks, gate, out, out_scale, self.chunk)
+
+    def on_matrix_cores(self, q, cache, gate, out, out_scale) -> bool:
+        """Whether the matrix-core attention for any widths takes this step: chunks, a gate per output column, and widths the plain
+        matrix-core kernels do not have."""
+        hd, vd, page = self.head_dim, self.value_dim, cache.k.shape[2]
+        return (q.dtype == torch.bfloat16 and (self.chunk > 0 or self.output_gate or
+                                               (self.rotary_dim > 0 or self.qk_norm == "unit") and
+                                               not (hd == vd and K.mfma_attention_supported(hd, page)))
+                and K.attention_wide_supported(hd, vd, page) and self.scale > 0 and not self.keep_first and self.slopes is None
+                and not self.score_cap and (gate is None or self.output_gate) and out_scale == 1.0
+                and (out is None or (out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0)))
 
     def forward(self, x, step, cache, write_cache=True):
         p = K.linear(x, self.w_in)

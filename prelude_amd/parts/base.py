@@ -61,6 +61,7 @@ class PagedCacheSpec:
     PAGED = True
     window: int = 0
     keep_first: int = 0    # with a window: the first positions every later token still sees; their pages are never given back
+    chunk: int = 0         # with a window of as many places: a token sees back to the start of its own chunk of that many only
 
     def bytes_per_token(self, element_size: int) -> int:
         """Bytes a token takes in this mixer's storage, for an engine element of ``element_size`` bytes."""
@@ -251,8 +252,8 @@ class FeedForward(Part):
         """(new residual, forward(norm of residual + x)): what a block asks for behind a mixer.  A feed-forward whose
         first kernel can take the add and the norm in (it learns the norm's kind from ``norm.as_rms()``) does so
         here; this is the plain order."""
-        if not norm.TAKES_SLICE_SUMS:
-            from ..ops.kernels import as_tensor
+        from ..ops.kernels import NormedBranches, as_tensor
+        if not (norm.TAKES_BRANCHES if isinstance(x, NormedBranches) else norm.TAKES_SLICE_SUMS):
             x = as_tensor(x)
         residual, h = norm.forward_residual(x, residual)
         return residual, (self.forward(h, step=step) if self.NEEDS_STEP else self.forward(h))
@@ -274,6 +275,9 @@ class Norm(Part):
     # inner size (``ops.kernels.SliceSums``) in place of ``x``, adding the slices as it loads them; a block
     # hands other norms the finished tensor.
     TAKES_SLICE_SUMS = False
+    # True for a norm whose methods also take a mixer's members' outputs that are still to be brought to unit RMS and added
+    # up (``ops.kernels.NormedBranches``); only with a 32-bit residual.
+    TAKES_BRANCHES = False
 
     def as_rms(self):
         """(gain, eps) if this norm is exactly y = x * rsqrt(mean(x^2) + eps) * gain over the whole row with the

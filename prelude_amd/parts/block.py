@@ -17,6 +17,11 @@ from ..ops import kernels as K
 from .base import Block, PartError, register_part
 
 
+def as_norm_takes(norm, x):
+    """What waits for ``norm``, in a form it takes."""
+    return x if (norm.TAKES_BRANCHES if isinstance(x, K.NormedBranches) else norm.TAKES_SLICE_SUMS) else K.as_tensor(x)
+
+
 @register_part("block", "prenorm")
 class PreNormBlock(Block):
     GRAPH_SAFE_PORTIONS = True   # launches follow the step's shape alone; tokens, positions and pages are read on the device
@@ -27,10 +32,9 @@ class PreNormBlock(Block):
         self.input_norm, self.mixer, self.post_mixer_norm, self.ffn = input_norm, mixer, post_mixer_norm, ffn
 
     def forward(self, hidden, residual, step, cache, write_cache=True):
-        # a mixer's or feed-forward's last product may come as partial sums of slices (``K.SliceSums``): a norm
-        # that can adds them as it loads them, any other gets the finished tensor
-        if not self.input_norm.TAKES_SLICE_SUMS:
-            hidden = K.as_tensor(hidden)
+        # a mixer's or feed-forward's last product may come as partial sums of slices (``K.SliceSums``), or a mixer's members'
+        # outputs as they are (``K.NormedBranches``): a norm that can adds them as it loads them, any other gets the tensor
+        hidden = as_norm_takes(self.input_norm, hidden)
         residual, h = self.input_norm.forward_residual(hidden, residual)
         h = self.mixer.forward(h, step, cache, write_cache)
         if getattr(self.ffn, "NEEDS_STEP", False):
@@ -51,8 +55,7 @@ class PreNormMixerBlock(Block):
         self.input_norm, self.mixer = input_norm, mixer
 
     def forward(self, hidden, residual, step, cache, write_cache=True):
-        if not self.input_norm.TAKES_SLICE_SUMS:
-            hidden = K.as_tensor(hidden)
+        hidden = as_norm_takes(self.input_norm, hidden)
         residual, h = self.input_norm.forward_residual(hidden, residual)
         return self.mixer.forward(h, step, cache, write_cache), residual
 

@@ -54,7 +54,7 @@ class ConvInputMixer(Mixer):
     def forward(self, x, step, cache, write_cache=True):
         caches = list(cache) if isinstance(cache, tuple) else [cache]
         state = caches.pop(0).tensors["inputs"] if self.taps > 1 else None
-        x = K.time_conv_add(x, self.weight, state, step)
+        x = K.time_conv(x, self.weight, state, step, add_input=True)
         inner_spec = self.inner.cache_spec()
         if isinstance(inner_spec, (tuple, list)):
             inner_cache = tuple(caches)

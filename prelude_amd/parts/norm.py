@@ -21,6 +21,10 @@ class RMSNorm(Norm):
 
     TAKES_SLICE_SUMS = True
 
+    @property
+    def TAKES_BRANCHES(self):
+        return self.residual_float32
+
     def __init__(self, size: int, eps: float, weight_offset: float = 0.0, residual_float32: bool = False):
         """``weight_offset``: the stored weight lies around zero and the gain is ``offset + weight`` (added once,
         in 32-bit, when the weight is loaded).  ``residual_float32``: the residual stream this norm adds to is
@@ -30,6 +34,7 @@ class RMSNorm(Norm):
         self.weight_offset = float(weight_offset)
         self.residual_float32 = bool(residual_float32)
         self.weight: Optional[torch.Tensor] = None
+        self.dtype: Optional[torch.dtype] = None
 
     def tensors(self):
         # a weight stored around zero is drawn around zero in the random-weights mode too
@@ -38,6 +43,7 @@ class RMSNorm(Norm):
     def load(self, tensors, dtype, device):
         w = tensors["weight"]
         self.weight = (w + self.weight_offset).contiguous() if self.weight_offset else w
+        self.dtype = dtype
 
     def as_rms(self):
         return self.weight, self.eps
@@ -50,6 +56,9 @@ class RMSNorm(Norm):
         residual is updated in place with residual + x."""
         if residual is None:
             x = K.as_tensor(x)
+            if self.residual_float32 and x.dtype != self.dtype:
+                # the embedding came in 32-bit already: it is the stream
+                return x, K.rmsnorm_wide(None, self.weight, self.eps, residual=x, out_dtype=self.dtype)
             if self.residual_float32:
                 # the stream starts as a 32-bit copy of x (x itself when the engine's type is 32-bit already)
                 return K.to_f32(x), K.rmsnorm(x, self.weight, self.eps)
@@ -57,6 +66,8 @@ class RMSNorm(Norm):
         if self.residual_float32:
             if residual.dtype != torch.float32:
                 raise PartError("rms_norm: a norm with a 32-bit residual was handed one of another type")
+            if isinstance(x, K.NormedBranches):
+                return residual, K.branches_norm_step(x, residual, self.weight, self.eps)
             return residual, K.rmsnorm_wide(x, self.weight, self.eps, residual=residual)
         out = K.rmsnorm(x, self.weight, self.eps, residual=residual)
         return residual, out
@@ -67,6 +78,8 @@ class RMSNorm(Norm):
             if residual is None or residual.dtype != torch.float32:
                 raise PartError("rms_norm: the norm of the stream's rows alone needs a 32-bit stream")
             return K.rmsnorm_wide(None, self.weight, self.eps, residual=residual, rows=rows, out_dtype=out_dtype)
+        if isinstance(x, K.NormedBranches):
+            return K.branches_norm_step(x, residual, self.weight, self.eps, rows=rows)
         if self.residual_float32 and residual is not None:
             return K.rmsnorm_wide(x, self.weight, self.eps, residual=residual, rows=rows)
         return K.rmsnorm(x, self.weight, self.eps, residual=residual, rows=rows)
