@@ -232,6 +232,38 @@ def pugavik_record(args):
     return arch_record(args, "pugavik", (("pugavik", pugavik_shape(layers)), ("fazopel_beside", fazopel_beside_pugavik(layers))))
 
 
+# ``--arch pogorax``: a decoder of the Pogorax design at layer sizes of a real model of that kind, in periods of four layers:
+# Mamba-2 (no feed-forward); attention on rotated unit queries beside Griffin's recurrent block; Mamba-2; attention inside chunks of
+# 1,024 with a gate on its output beside mLSTM -- beside the closest existing design at equal size, a Tedalix decoder with retention
+# (no feed-forward) in Mamba-2's places and attention beside the gated delta rule in the others', the first of them without a
+# window and with feed-forwards of as many weights
+def pogorax_shape(layers=12, width=2048, vocab=65536):
+    dense = dict(kind="dense", ff=5504)
+    mamba = dict(heads=64, vdim=64, state=128, groups=8, conv=4, norm_groups=8)
+    attention = dict(heads=16, kv_heads=4, dim=128, vdim=128, scale=128 ** -0.5)
+    griffin = dict(left=dict(attention, rot=dict(base=1000000.0, dims=64)), right=dict(width=width, blocks=8, conv=4))
+    xlstm = dict(left=dict(attention, mask=dict(size=1024)), right=dict(heads=8, dim=128, vdim=256, gate_cap=15.0))
+    period = (("mamba2", mamba, None), ("parallel_2", griffin, dense), ("mamba2", mamba, None), ("parallel", xlstm, dense))
+    return dict(architecture="Pogorax", vocab=vocab, width=width, norm=dict(eps=1e-5), embedding=dict(scale=width ** 0.5),
+                layers=[dict(type=period[i % 4][0], mixer=period[i % 4][1], mlp=period[i % 4][2]) for i in range(layers)])
+
+
+def tedalix_beside_pogorax(layers=12):
+    raw = tedalix_shape(4)
+    parallel, retention = raw["layers"][1], raw["layers"][2]
+    left = {k: v for k, v in parallel["mixer"]["left"].items() if k != "mask"}
+    beside = {1: dict(parallel, mixer=dict(parallel["mixer"], left=left)),
+              3: dict(parallel, mixer=dict(parallel["mixer"], left=dict(left, mask=dict(size=1024))))}
+    raw["layers"] = [beside.get(i % 4, retention) for i in range(layers)]
+    return raw
+
+
+def pogorax_record(args):
+    """Prefill and decode throughput of the Pogorax shape and of a Tedalix shape beside it, same points."""
+    layers = args.layers or 12
+    return arch_record(args, "pogorax", (("pogorax", pogorax_shape(layers)), ("tedalix_beside", tedalix_beside_pogorax(layers))))
+
+
 def build_engine(raw, dtype, cache_tokens, seed=0, page_size=16, **cfg_overrides):
     """The engine in its random-weights mode: the product's own loader, tensors drawn on the device."""
     from prelude_amd.config import EngineConfig
@@ -467,8 +499,8 @@ def main() -> int:
     ap.add_argument("--layers", type=int, default=None, help="fewer layers than the configuration has (named in config)")
     ap.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
     ap.add_argument("--shape", default="4b", choices=sorted(SHAPES), help="layer sizes: Qwen3-4B (the default run), 0.6B, 8B or 32B")
-    ap.add_argument("--arch", default="qwen3", choices=["qwen3", "libodra", "fazopel", "tedalix", "nivasun", "pugavik"],
-                    help="libodra, fazopel, tedalix, nivasun, pugavik: prefill and decode of that design at a real model's layer sizes beside the closest other "
+    ap.add_argument("--arch", default="qwen3", choices=["qwen3", "libodra", "fazopel", "tedalix", "nivasun", "pugavik", "pogorax"],
+                    help="libodra, fazopel, tedalix, nivasun, pugavik, pogorax: prefill and decode of that design at a real model's layer sizes beside the closest other "
                          "decoder of equal size, as one record (the default run and its record are Qwen3's)")
     ap.add_argument("--prefill-tokens", type=int, default=2048)
     ap.add_argument("--no-points", action="store_true", help="skip the points at other batches and lengths")
@@ -506,6 +538,9 @@ def main() -> int:
         return 0
     if args.arch == "pugavik":
         print(json.dumps(pugavik_record(args)), flush=True)
+        return 0
+    if args.arch == "pogorax":
+        print(json.dumps(pogorax_record(args)), flush=True)
         return 0
     raw = dict(SHAPES[args.shape])
     name = f"Qwen3-{args.shape.upper()} shape"

@@ -44,6 +44,21 @@ template <typename T> __device__ __forceinline__ T from_f32(float v);
 template <> __device__ __forceinline__ float from_f32<float>(float v) { return v; }
 template <> __device__ __forceinline__ bf16 from_f32<bf16>(float v) { return static_cast<bf16>(v); }  // round to nearest even
 
+// sigmoid, SiLU and the gated activations for a result that is rounded to T: behind bfloat16 the hardware's exponential and
+// reciprocal serve (a few units of the 24th bit); GELU in its tanh form is x sigmoid(2 u), u = sqrt(2 / pi) (x + 0.044715 x^3).
+template <typename T>
+__device__ __forceinline__ float sigmoid_of(float z) {
+  if (sizeof(T) == 2) return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+  return 1.0f / (1.0f + expf(-z));
+}
+template <typename T>
+__device__ __forceinline__ float silu_of(float z) { return sizeof(T) == 2 ? z * sigmoid_of<T>(z) : z / (1.0f + expf(-z)); }
+template <typename T>
+__device__ __forceinline__ float gate_activation_of(float z, int act) {
+  if (sizeof(T) == 2) return z * sigmoid_of<T>(act == kActGeluTanh ? 1.5957691216057308f * (z + 0.044715f * z * z * z) : z);
+  return gate_activation(z, act);
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int m = kWave / 2; m > 0; m >>= 1) v += __shfl_xor(v, m, kWave);

@@ -74,35 +74,34 @@ __global__ __launch_bounds__(256) void ssd_gates_kernel(const T* __restrict__ p,
   la[i] = -expf(a_log[h]) * dt;
 }
 
-// A wavefront a (head, sequence of at least min_len tokens), 64 tokens at a time, a lane a token.  A token is the map
+// A workgroup a (head, sequence of at least min_len tokens), 1,024 tokens at a time, a thread a token.  A token is the map
 // m -> max(f + m, i), and maps compose: (f1, i1) and then (f2, i2) is (f1 + f2, max(i1 + f2, i2)).
+constexpr int kGateThreads = 1024;
+
 template <typename T>
-__global__ __launch_bounds__(kWave) void mlstm_gates_kernel(const T* __restrict__ p, size_t ld, int i_off, int f_off,
-                                                            const float* __restrict__ i_bias, const float* __restrict__ f_bias,
-                                                            float cap, float* __restrict__ m_state, int copies,
-                                                            const int* __restrict__ state_slots, const int* __restrict__ cu_q,
-                                                            float* __restrict__ la, float* __restrict__ b,
-                                                            float* __restrict__ floor_out, int heads, int min_len) {
-  const int h = blockIdx.x, seq = blockIdx.y, lane = threadIdx.x;
+__global__ __launch_bounds__(kGateThreads) void mlstm_gates_kernel(const T* __restrict__ p, size_t ld, int i_off, int f_off,
+                                                                   const float* __restrict__ i_bias, const float* __restrict__ f_bias,
+                                                                   float cap, float* __restrict__ m_state, int copies,
+                                                                   const int* __restrict__ state_slots, const int* __restrict__ cu_q,
+                                                                   float* __restrict__ la, float* __restrict__ b,
+                                                                   float* __restrict__ floor_out, int heads, int min_len) {
+  constexpr int kWaves = kGateThreads / kWave;
+  __shared__ float wave_f[2][kWaves], wave_i[2][kWaves];
+  const int h = blockIdx.x, seq = blockIdx.y, lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
   const int row0 = cu_q[seq], row1 = cu_q[seq + 1];
   const int slot = state_slots[seq];
-  if (slot < 0 || row1 - row0 < min_len || row1 <= row0) return;
+  if (slot < 0 || row1 - row0 < min_len || row1 <= row0) return;   // the same for the whole workgroup
   float* ms = m_state + ((size_t)slot * heads + h) * copies;
   float m = ms[0];
   const float ib = i_bias[h], fb = f_bias[h];
-  float zi = 0.f, zf = 0.f;
-  auto fetch = [&](int t) {
-    t = t < row1 ? t : row1 - 1;
-    zi = to_f32(p[(size_t)t * ld + i_off + h]);
-    zf = to_f32(p[(size_t)t * ld + f_off + h]);
-  };
-  fetch(row0 + lane);
-  for (int t0 = row0; t0 < row1; t0 += kWave) {
-    const int t = t0 + lane;
+  int buf = 0;
+  for (int t0 = row0; t0 < row1; t0 += kGateThreads, buf ^= 1) {
+    const int t = t0 + threadIdx.x;
     const bool live = t < row1;
+    const T* z = p + (size_t)(live ? t : row1 - 1) * ld + h;
+    const float zi = to_f32(z[i_off]), zf = to_f32(z[f_off]);
     const float ig = live ? scan_capped(zi + ib, cap) : -INFINITY;
     const float fg = live ? scan_log_sigmoid(scan_capped(zf + fb, cap)) : 0.f;
-    if (t0 + kWave < row1) fetch(t + kWave);
     float A = fg, B = ig;
 #pragma unroll
     for (int o = 1; o < kWave; o <<= 1) {
@@ -112,18 +111,28 @@ __global__ __launch_bounds__(kWave) void mlstm_gates_kernel(const T* __restrict_
         A += Ao;
       }
     }
-    const float mt = fmaxf(A + m, B);
+    if (lane == kWave - 1) {
+      wave_f[buf][wave] = A;
+      wave_i[buf][wave] = B;
+    }
+    __syncthreads();               // (two buffers: the next block's sums do not meet this one's readers)
+    float mine = m;                // the maximum in front of this wavefront's tokens, and behind the block's
+    for (int w = 0; w < kWaves; ++w) {
+      if (w == wave) mine = m;
+      m = fmaxf(wave_f[buf][w] + m, wave_i[buf][w]);
+    }
+    const float mt = fmaxf(A + mine, B);
     float before = __shfl_up(mt, 1, kWave);
-    if (lane == 0) before = m;
+    if (lane == 0) before = mine;
     if (live) {
       const size_t at = (size_t)t * heads + h;
       la[at] = fg + before - mt;
       b[at] = expf(ig - mt);
       floor_out[at] = expf(-mt);
     }
-    m = __shfl(mt, kWave - 1, kWave);
   }
-  for (int i = lane; i < copies; i += kWave) ms[i] = m;
+  __syncthreads();                 // every thread has read the slot
+  for (int i = threadIdx.x; i < copies; i += kGateThreads) ms[i] = m;
 }
 
 // ---- token by token ----------------------------------------------------------------------------------------------------
@@ -633,10 +642,10 @@ extern "C" int pa_mlstm_gates(void* stream, int dtype, const void* p, long ld, i
   hipStream_t st = (hipStream_t)stream;
   const int copies = pa_mlstm_max_copies(vdim);
   if (dtype == kF32)
-    hipLaunchKernelGGL(mlstm_gates_kernel<float>, dim3(heads, nseq), dim3(kWave), 0, st, (const float*)p, (size_t)ld, i_off, f_off, i_bias,
+    hipLaunchKernelGGL(mlstm_gates_kernel<float>, dim3(heads, nseq), dim3(kGateThreads), 0, st, (const float*)p, (size_t)ld, i_off, f_off, i_bias,
                        f_bias, cap, m, copies, state_slots, cu_q, la, b, floor_out, heads, min_len);
   else if (dtype == kBF16)
-    hipLaunchKernelGGL(mlstm_gates_kernel<bf16>, dim3(heads, nseq), dim3(kWave), 0, st, (const bf16*)p, (size_t)ld, i_off, f_off, i_bias,
+    hipLaunchKernelGGL(mlstm_gates_kernel<bf16>, dim3(heads, nseq), dim3(kGateThreads), 0, st, (const bf16*)p, (size_t)ld, i_off, f_off, i_bias,
                        f_bias, cap, m, copies, state_slots, cu_q, la, b, floor_out, heads, min_len);
   else
     return pa::fail("mlstm_gates: unknown element type code %d", dtype);

@@ -320,17 +320,6 @@ __global__ __launch_bounds__(256) void embed_scaled_kernel(const int* __restrict
   }
 }
 
-// GELU in its tanh form is x sigmoid(2 u), u = sqrt(2 / pi) (x + 0.044715 x^3): for bfloat16 results with the hardware's
-// exponential and reciprocal (the tanh's own code would take longer than the memory).
-template <typename T>
-__device__ __forceinline__ float activation_of(float x, int act) {
-  if (sizeof(T) == 2 && act == kActGeluTanh) {
-    const float u2 = 1.5957691216057308f * (x + 0.044715f * x * x * x);
-    return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * u2));
-  }
-  return gate_activation(x, act);
-}
-
 // V consecutive columns a thread.
 template <typename T, int V>
 __global__ __launch_bounds__(256) void activate_kernel(const T* __restrict__ x, size_t x_stride, T* __restrict__ out, size_t out_stride,
@@ -342,7 +331,7 @@ __global__ __launch_bounds__(256) void activate_kernel(const T* __restrict__ x, 
   const vec_t v = *reinterpret_cast<const vec_t*>(x + r * x_stride + c);
   vec_t o;
 #pragma unroll
-  for (int e = 0; e < V; ++e) o[e] = from_f32<T>(activation_of<T>(to_f32(v[e]), act) * scale);
+  for (int e = 0; e < V; ++e) o[e] = from_f32<T>(gate_activation_of<T>(to_f32(v[e]), act) * scale);
   *reinterpret_cast<vec_t*>(out + r * out_stride + c) = o;
 }
 

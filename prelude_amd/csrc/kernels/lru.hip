@@ -10,7 +10,7 @@
 //   pa_lru_gates   a and sqrt(1 - a^2) i u for every token; a sequence that brings one token is finished here (it is the only
 //                  reader of its slot).  bfloat16: the blocks' products on the matrix cores, a wavefront 16 channels of both
 //                  gates against up to 64 tokens, so that a lane holds both gates of its channels.
-//   pa_lru_scan    the sequences of several tokens.  Chunks of 64 tokens run side by side: (1) where a sequence has more than one,
+//   pa_lru_scan    the sequences of several tokens.  Chunks of 32 tokens run side by side: (1) where a sequence has more than one,
 //                  every chunk makes its product of decays and its end from zero; (2) every chunk folds the chunks before it
 //                  into the state it starts from, in order, and makes its outputs.
 #include "common.h"
@@ -19,15 +19,30 @@
 
 namespace pa {
 
-constexpr int kLruChunk = 64;
+constexpr int kLruChunk = 32;
+constexpr int kLruBatch = 16;    // tokens asked for together
 constexpr int kLruThreads = 256;
 
-__device__ __forceinline__ float lru_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+// 1 - e^-x for x >= 0: below a quarter as its series (an alternating one whose eighth term is below 2^-30 of the first), which
+// loses nothing where a is close to one
+__device__ __forceinline__ float lru_one_minus_exp(float x, float e) {
+  if (x > 0.25f) return 1.0f - e;
+  float p = 1.0f - x * (1.0f / 8.0f);
+  p = 1.0f - x * (1.0f / 7.0f) * p;
+  p = 1.0f - x * (1.0f / 6.0f) * p;
+  p = 1.0f - x * (1.0f / 5.0f) * p;
+  p = 1.0f - x * (1.0f / 4.0f) * p;
+  p = 1.0f - x * (1.0f / 3.0f) * p;
+  p = 1.0f - x * (1.0f / 2.0f) * p;
+  return x * p;
+}
 
 // a, and the factor of u
+template <typename T>
 __device__ __forceinline__ float2 lru_gate(float zr, float zi, float rate) {
-  const float log_a = -rate * lru_sigmoid(zr);
-  return float2{expf(log_a), sqrtf(-expm1f(2.0f * log_a)) * lru_sigmoid(zi)};
+  const float x = rate * sigmoid_of<T>(zr);
+  const float a = sizeof(T) == 2 ? __builtin_amdgcn_exp2f(-1.4426950408889634f * x) : expf(-x);
+  return float2{a, sqrtf(lru_one_minus_exp(2.0f * x, a * a)) * sigmoid_of<T>(zi)};
 }
 
 template <typename T>
@@ -49,23 +64,24 @@ struct LruArgs {
   int tokens, width;
   __device__ __forceinline__ T output(float s, size_t t, int c) const {
     const float z = to_f32(y[t * y_ld + c]) + (y_bias ? y_bias[c] : 0.f);
-    return from_f32<T>(s * gate_activation(z, act) * out_scale);
+    return from_f32<T>(s * gate_activation_of<T>(z, act) * out_scale);
   }
-  // what a (token, channel)'s gates lead to
-  __device__ __forceinline__ void finish(float zr, float zi, int t, int c, bool single, int slot) const {
+  // what a (token, channel)'s gates lead to; ut: the token's u; slot: of a sequence that brings this token alone, else -1
+  __device__ __forceinline__ void finish(float zr, float zi, float ut, int t, int c, int slot) const {
     const size_t at = (size_t)t * width + c;
-    const float2 g = lru_gate(zr, zi, rate[c]);
-    const float in = g.y * to_f32(u[at]);
-    if (!single) {
+    const float2 g = lru_gate<T>(zr, zi, rate[c]);
+    const float in = g.y * ut;
+    if (slot < 0) {
       a[at] = g.x;
       x[at] = in;
-    } else if (slot >= 0) {
+    } else {
       float* sp = state + (size_t)slot * width + c;
       const float s = fmaf(g.x, *sp, in);
       *sp = s;
       out[(size_t)t * out_ld + c] = output(s, t, c);
     }
   }
+  __device__ __forceinline__ int single_slot(int seq) const { return cu_q[seq + 1] - cu_q[seq] == 1 ? slots[seq] : -1; }
 };
 
 // A thread a (token, channel).
@@ -84,8 +100,7 @@ __global__ __launch_bounds__(kLruThreads) void lru_gates_kernel(LruArgs<T> p, co
     zr = fmaf(to_f32(r[k]), v, zr);
     zi = fmaf(to_f32(i[k]), v, zi);
   }
-  const int seq = seq_of_token[t];
-  p.finish(zr + br[c], zi + bi[c], t, c, p.cu_q[seq + 1] - p.cu_q[seq] == 1, p.slots[seq]);
+  p.finish(zr + br[c], zi + bi[c], to_f32(p.u[(size_t)t * p.width + c]), t, c, p.single_slot(seq_of_token[t]));
 }
 
 // Grid (runs of 16 * MT tokens, runs of 64 channels of a block, blocks); a wavefront 16 channels.
@@ -128,14 +143,23 @@ __global__ __launch_bounds__(kLruThreads) void lru_gates_mfma_kernel(LruArgs<bf1
   if (o0 + r >= size) return;
   const int c = base + o0 + r;
   const float b0 = br[c], b1 = bi[c];
+  // what the tokens' ends need is asked for before the first of them is written
+  int slot[MT][4];
+  bf16 ut[MT][4];
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = t0 + 16 * m + 4 * g + i < p.tokens ? t0 + 16 * m + 4 * g + i : p.tokens - 1;
+      slot[m][i] = p.single_slot(seq_of_token[t]);
+      ut[m][i] = p.u[(size_t)t * p.width + c];
+    }
 #pragma unroll
   for (int m = 0; m < MT; ++m)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int t = t0 + 16 * m + 4 * g + i;
-      if (t >= p.tokens) continue;
-      const int seq = seq_of_token[t];
-      p.finish(ar[m][i] + b0, ai[m][i] + b1, t, c, p.cu_q[seq + 1] - p.cu_q[seq] == 1, p.slots[seq]);
+      if (t < p.tokens) p.finish(ar[m][i] + b0, ai[m][i] + b1, (float)ut[m][i], t, c, slot[m][i]);
     }
 }
 
@@ -155,16 +179,16 @@ __global__ __launch_bounds__(kLruThreads) void lru_chunk_kernel(LruArgs<T> p, co
   if (j == 0) w0[(size_t)z * p.width + c] = p.state[(size_t)p.slots[seq] * p.width + c];
   const int t0 = row0 + j * kLruChunk, t1 = t0 + kLruChunk < row1 ? t0 + kLruChunk : row1;
   float A = 1.f, U = 0.f;
-  for (int t = t0; t < t1; t += 8) {
-    float av[8], xv[8];
+  for (int t = t0; t < t1; t += kLruBatch) {
+    float av[kLruBatch], xv[kLruBatch];
 #pragma unroll
-    for (int k = 0; k < 8; ++k) {
+    for (int k = 0; k < kLruBatch; ++k) {
       const size_t at = (size_t)(t + k < t1 ? t + k : t1 - 1) * p.width + c;
       av[k] = p.a[at];
       xv[k] = p.x[at];
     }
 #pragma unroll
-    for (int k = 0; k < 8; ++k)
+    for (int k = 0; k < kLruBatch; ++k)
       if (t + k < t1) {
         A *= av[k];
         U = fmaf(av[k], U, xv[k]);
@@ -189,24 +213,24 @@ __global__ __launch_bounds__(kLruThreads) void lru_out_kernel(LruArgs<T> p, cons
   // one chunk: its thread is the only one that touches the slot's place; several: they start from the copy (1) made
   float S = row1 - row0 <= kLruChunk ? *sp : w0[(size_t)z * p.width + c];
   const size_t first = lru_chunk_index(row0, z, 0) * p.width + c;
-  for (int k0 = 0; k0 < j; k0 += 8) {
-    float A[8], U[8];
+  for (int k0 = 0; k0 < j; k0 += kLruBatch) {
+    float A[kLruBatch], U[kLruBatch];
 #pragma unroll
-    for (int k = 0; k < 8; ++k) {
+    for (int k = 0; k < kLruBatch; ++k) {
       const size_t at = first + (size_t)(k0 + k < j ? k0 + k : j - 1) * p.width;
       A[k] = wa[at];
       U[k] = wu[at];
     }
 #pragma unroll
-    for (int k = 0; k < 8; ++k)
+    for (int k = 0; k < kLruBatch; ++k)
       if (k0 + k < j) S = fmaf(A[k], S, U[k]);
   }
   const int t0 = row0 + j * kLruChunk, t1 = t0 + kLruChunk < row1 ? t0 + kLruChunk : row1;
-  for (int t = t0; t < t1; t += 8) {
-    float av[8], xv[8];
-    T yv[8];
+  for (int t = t0; t < t1; t += kLruBatch) {
+    float av[kLruBatch], xv[kLruBatch];
+    T yv[kLruBatch];
 #pragma unroll
-    for (int k = 0; k < 8; ++k) {
+    for (int k = 0; k < kLruBatch; ++k) {
       const size_t tt = t + k < t1 ? t + k : t1 - 1;
       av[k] = p.a[tt * p.width + c];
       xv[k] = p.x[tt * p.width + c];
@@ -214,10 +238,10 @@ __global__ __launch_bounds__(kLruThreads) void lru_out_kernel(LruArgs<T> p, cons
     }
     const float yb = p.y_bias ? p.y_bias[c] : 0.f;
 #pragma unroll
-    for (int k = 0; k < 8; ++k)
+    for (int k = 0; k < kLruBatch; ++k)
       if (t + k < t1) {
         S = fmaf(av[k], S, xv[k]);
-        p.out[(size_t)(t + k) * p.out_ld + c] = from_f32<T>(S * gate_activation(to_f32(yv[k]) + yb, p.act) * p.out_scale);
+        p.out[(size_t)(t + k) * p.out_ld + c] = from_f32<T>(S * gate_activation_of<T>(to_f32(yv[k]) + yb, p.act) * p.out_scale);
       }
   }
   if (t1 == row1) *sp = S;

@@ -319,7 +319,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_vec_kernel(const float* 
       load8(w + c0 + 8 * piece, wv[v]);
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
-        u[v][i] *= zv[i] / (1.0f + expf(-zv[i]));
+        u[v][i] *= silu_of<T>(zv[i]);
         ss += u[v][i] * u[v][i];
       }
     }

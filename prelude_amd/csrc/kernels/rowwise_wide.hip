@@ -72,6 +72,82 @@ __global__ __launch_bounds__(256) void rmsnorm_wide_kernel(const T* __restrict__
   }
 }
 
+__device__ __forceinline__ void wide_load8(const float* p, float* v) {
+  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+  v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+}
+__device__ __forceinline__ void wide_load8(const bf16* p, float* v) {
+  const bf16x8 a = *reinterpret_cast<const bf16x8*>(p);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = (float)a[i];
+}
+__device__ __forceinline__ void wide_store8(float* p, const float* v) {
+  *reinterpret_cast<float4*>(p) = float4{v[0], v[1], v[2], v[3]};
+  *reinterpret_cast<float4*>(p + 4) = float4{v[4], v[5], v[6], v[7]};
+}
+__device__ __forceinline__ void wide_store8(bf16* p, const float* v) {
+  bf16x8 a;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) a[i] = (bf16)v[i];
+  *reinterpret_cast<bf16x8*>(p) = a;
+}
+
+// The same for rows of up to 8 * 256 * VPT elements in whole pieces of eight: everything a thread needs is asked for at once, in
+// 16-byte loads.
+template <typename T, int VPT>
+__global__ __launch_bounds__(256) void rmsnorm_wide_vec_kernel(const T* __restrict__ x, const float* __restrict__ parts, int slices,
+                                                              size_t slice_stride, float* __restrict__ residual,
+                                                              const float* __restrict__ w, T* __restrict__ out,
+                                                              const int* __restrict__ rows, int hidden, float eps) {
+  __shared__ float scratch[16];
+  const size_t r = blockIdx.x;
+  const size_t src = (rows ? (size_t)rows[r] : r) * hidden;
+  const int pieces = hidden / 8;
+  float v[VPT][8], wv[VPT][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int piece = k * 256 + threadIdx.x;
+    if (piece < pieces) {
+      const size_t at = src + 8 * piece;
+      float y[8];
+      wide_load8(w + 8 * piece, wv[k]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] = 0.f;
+      if (residual) wide_load8(residual + at, v[k]);
+      if (parts) {
+        wide_load8(parts + at, y);
+        for (int p = 1; p < slices; ++p) {
+          float u[8];
+          wide_load8(parts + (size_t)p * slice_stride + at, u);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) y[i] += u[i];
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[k][i] += y[i];
+      } else if (x) {
+        wide_load8(x + at, y);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[k][i] += y[i];
+      }
+      if (residual && !rows && (x || parts)) wide_store8(residual + at, v[k]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += v[k][i] * v[k][i];
+    }
+  }
+  const float inv = rsqrtf(block_sum(ss, scratch) / (float)hidden + eps);
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int piece = k * 256 + threadIdx.x;
+    if (piece < pieces) {
+      float o[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) o[i] = v[k][i] * inv * wv[k][i];
+      wide_store8(out + r * hidden + 8 * piece, o);
+    }
+  }
+}
+
 // gate_up [T, 2I] with columns alternating gate_j, up_j -> [T, I]
 template <typename T>
 __global__ void clamped_gate_kernel(const T* __restrict__ gate_up, T* __restrict__ out, size_t total, float limit,
@@ -234,6 +310,17 @@ static int launch_gated(hipStream_t st, const float* o, const T* gate, size_t ga
 template <typename T>
 static void launch_wide(hipStream_t st, const T* x, const float* parts, int slices, size_t slice_stride, float* residual,
                         const float* w, T* out, const int* rows, int nrows, int hidden, float eps) {
+  auto aligned = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (hidden % 8 == 0 && hidden <= 8 * 256 * 4 && slice_stride % 4 == 0 && aligned(x) && aligned(parts) && aligned(residual) && aligned(w) && aligned(out)) {
+#define PA_WIDE_VEC(V)                                                                                                      \
+  hipLaunchKernelGGL((rmsnorm_wide_vec_kernel<T, V>), dim3(nrows), dim3(256), 0, st, x, parts, slices, slice_stride, residual, \
+                     w, out, rows, hidden, eps)
+    if (hidden <= 8 * 256) PA_WIDE_VEC(1);
+    else if (hidden <= 8 * 256 * 2) PA_WIDE_VEC(2);
+    else PA_WIDE_VEC(4);
+#undef PA_WIDE_VEC
+    return;
+  }
 #define PA_WIDE(NV)                                                                                                  \
   hipLaunchKernelGGL((rmsnorm_wide_kernel<T, NV>), dim3(nrows), dim3(256), 0, st, x, parts, slices, slice_stride,    \
                      residual, w, out, rows, hidden, eps)

@@ -59,67 +59,161 @@ __global__ __launch_bounds__(256) void pair_embed_kernel(const int* __restrict__
 // itself; portions leave that to time_conv_carry_kernel, which runs behind this one.
 constexpr int kConvMaxTaps = 17;
 
-template <typename T, int V>
+// A run of TOK consecutive tokens a thread: a tap's weights are read once for all of them.
+template <typename T, int V, int TOK>
 __global__ __launch_bounds__(256) void time_conv_kernel(const T* __restrict__ h, size_t stride, const float* __restrict__ w,
                                                         const float* __restrict__ in_bias, const float* __restrict__ bias,
                                                         float* __restrict__ state, const int* __restrict__ seq_of_token,
                                                         const int* __restrict__ cu_q, const int* __restrict__ state_slots,
-                                                        T* __restrict__ out, size_t out_stride, int C, int taps, int act,
+                                                        T* __restrict__ out, size_t out_stride, int tokens, int C, int taps, int act,
                                                         int add_input) {
   typedef T vec_t __attribute__((ext_vector_type(V)));
-  const int t = blockIdx.x;
+  const int t0 = blockIdx.x * TOK;
   const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
   if (c >= C) return;
-  const int seq = seq_of_token[t];
-  const int begin = cu_q[seq];
-  const int rel = t - begin;
-  const bool single = cu_q[seq + 1] - begin == 1;
   const int keep = taps - 1;
-  float* st = keep > 0 ? state + (size_t)state_slots[seq] * keep * C : nullptr;
-  float x[V], acc[V], ib[V];
-  auto input = [&](int at, float* v) {
-    const vec_t pv = *reinterpret_cast<const vec_t*>(h + (size_t)at * stride + c);
+  float acc[TOK][V], ib[V];
+  int rel[TOK];                     // tokens of its sequence the step brings before this one
+  unsigned single = 0;              // the tokens that are all their sequence brings
 #pragma unroll
-    for (int e = 0; e < V; ++e) v[e] = to_f32(pv[e]) + ib[e];
-  };
+  for (int e = 0; e < V; ++e) ib[e] = in_bias ? in_bias[c + e] : 0.f;
 #pragma unroll
-  for (int e = 0; e < V; ++e) ib[e] = in_bias ? in_bias[c + e] : 0.f, acc[e] = bias ? bias[c + e] : 0.f;
-  input(t, x);
+  for (int k = 0; k < TOK; ++k) {
+    const int t = t0 + k < tokens ? t0 + k : tokens - 1;
+    const int seq = seq_of_token[t];
+    const int begin = cu_q[seq];
+    rel[k] = t - begin;
+    if (cu_q[seq + 1] - begin == 1) single |= 1u << k;
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[k][e] = bias ? bias[c + e] : 0.f;
+  }
+  auto carried = [&](int k) { return state + (size_t)state_slots[seq_of_token[t0 + k]] * keep * C + c; };
   for (int j = 0; j < taps; ++j) {
-    const int back = keep - j;   // the input `back` positions before this token
-    float v[V];
-    if (back == 0) {
+    const int back = keep - j;      // the input `back` positions before a token
+    float wv[V];
 #pragma unroll
-      for (int e = 0; e < V; ++e) v[e] = x[e];
-    } else if (rel - back >= 0) {
-      input(t - back, v);
-    } else {
-      const float* sp = st + (size_t)(rel - back + keep) * C + c;
+    for (int e = 0; e < V; ++e) wv[e] = w[(size_t)j * C + c + e];   // w [taps, C]: a tap's weights side by side
 #pragma unroll
-      for (int e = 0; e < V; ++e) v[e] = sp[e];
-      if (single && j > 0) {     // one token: the place before this one takes what this place held
-        float* dp = st + (size_t)(j - 1) * C + c;
+    for (int k = 0; k < TOK; ++k) {
+      if (t0 + k >= tokens) break;
+      float v[V];
+      if (rel[k] - back >= 0) {
+        const vec_t pv = *reinterpret_cast<const vec_t*>(h + (size_t)(t0 + k - back) * stride + c);
 #pragma unroll
-        for (int e = 0; e < V; ++e) dp[e] = v[e];
+        for (int e = 0; e < V; ++e) v[e] = to_f32(pv[e]) + ib[e];
+      } else {
+        float* st = carried(k);
+        const float* sp = st + (size_t)(rel[k] - back + keep) * C;
+#pragma unroll
+        for (int e = 0; e < V; ++e) v[e] = sp[e];
+        if ((single >> k & 1) && j > 0) {     // one token: the place before this one takes what this place held
+          float* dp = st + (size_t)(j - 1) * C;
+#pragma unroll
+          for (int e = 0; e < V; ++e) dp[e] = v[e];
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < V; ++e) acc[k][e] = fmaf(wv[e], v[e], acc[k][e]);
+      if (back == 0) {                        // the token's own input
+        if ((single >> k & 1) && keep > 0) {
+          float* dp = carried(k) + (size_t)(keep - 1) * C;
+#pragma unroll
+          for (int e = 0; e < V; ++e) dp[e] = v[e];
+        }
+        vec_t ov;
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          float y = acc[k][e];
+          if (act == 1) y = silu_of<T>(y);
+          if (add_input) y += v[e];
+          ov[e] = from_f32<T>(y);
+        }
+        *reinterpret_cast<vec_t*>(out + (size_t)(t0 + k) * out_stride + c) = ov;
       }
     }
-#pragma unroll
-    for (int e = 0; e < V; ++e) acc[e] = fmaf(w[(size_t)j * C + c + e], v[e], acc[e]);   // w [taps, C]: a tap's weights side by side
   }
-  if (single && keep > 0) {
-    float* dp = st + (size_t)(keep - 1) * C + c;
+}
+
+// The same for a number of taps known when this is compiled: everything a token's sum needs is asked for before any of it is used.
+// A run of tokens that lies inside one sequence, behind its first taps - 1 tokens of the step, reads every input once.
+template <typename T, int TAPS, int TOK>
+__global__ __launch_bounds__(256) void time_conv_taps_kernel(const T* __restrict__ h, size_t stride, const float* __restrict__ w,
+                                                             const float* __restrict__ in_bias, const float* __restrict__ bias,
+                                                             float* __restrict__ state, const int* __restrict__ seq_of_token,
+                                                             const int* __restrict__ cu_q, const int* __restrict__ state_slots,
+                                                             T* __restrict__ out, size_t out_stride, int tokens, int C, int act,
+                                                             int add_input) {
+  constexpr int V = 8, KEEP = TAPS - 1;
+  typedef T vec_t __attribute__((ext_vector_type(V)));
+  typedef float fvec_t __attribute__((ext_vector_type(V)));
+  const int t0 = blockIdx.x * TOK;
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * V;
+  if (c >= C) return;
+  fvec_t wv[TAPS], ib, bv;
 #pragma unroll
-    for (int e = 0; e < V; ++e) dp[e] = x[e];
-  }
-  vec_t ov;
+  for (int j = 0; j < TAPS; ++j) wv[j] = *reinterpret_cast<const fvec_t*>(w + (size_t)j * C + c);
 #pragma unroll
-  for (int e = 0; e < V; ++e) {
-    float y = acc[e];
-    if (act == 1) y = y / (1.0f + expf(-y));
-    if (add_input) y += x[e];
-    ov[e] = from_f32<T>(y);
+  for (int e = 0; e < V; ++e) ib[e] = in_bias ? in_bias[c + e] : 0.f, bv[e] = bias ? bias[c + e] : 0.f;
+  auto emit = [&](int t, const fvec_t* v) {        // v: the token's taps, the last one its own
+    vec_t ov;
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      float y = bv[e];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) y = fmaf(wv[j][e], v[j][e], y);
+      if (act == 1) y = silu_of<T>(y);
+      if (add_input) y += v[KEEP][e];
+      ov[e] = from_f32<T>(y);
+    }
+    *reinterpret_cast<vec_t*>(out + (size_t)t * out_stride + c) = ov;
+  };
+  auto widen = [&](const vec_t& x) {
+    fvec_t v;
+#pragma unroll
+    for (int e = 0; e < V; ++e) v[e] = to_f32(x[e]) + ib[e];
+    return v;
+  };
+  const int seq0 = seq_of_token[t0];
+  const int begin0 = cu_q[seq0];
+  if (TOK > 1 && t0 + TOK <= cu_q[seq0 + 1] && t0 - begin0 >= KEEP) {   // (the same for the whole workgroup)
+    vec_t x[TOK + KEEP];
+#pragma unroll
+    for (int i = 0; i < TOK + KEEP; ++i) x[i] = *reinterpret_cast<const vec_t*>(h + (size_t)(t0 - KEEP + i) * stride + c);
+#pragma unroll
+    for (int k = 0; k < TOK; ++k) {
+      fvec_t v[TAPS];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) v[j] = widen(x[k + j]);
+      emit(t0 + k, v);
+    }
+    return;
   }
-  *reinterpret_cast<vec_t*>(out + (size_t)t * out_stride + c) = ov;
+  for (int k = 0; k < TOK; ++k) {
+    const int t = t0 + k;
+    if (t >= tokens) return;
+    const int seq = seq_of_token[t];
+    const int begin = cu_q[seq], rel = t - begin;
+    fvec_t v[TAPS];
+    vec_t x[TAPS];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) x[j] = *reinterpret_cast<const vec_t*>(h + (size_t)(t - (KEEP - j <= rel ? KEEP - j : 0)) * stride + c);
+    if (rel < KEEP) {
+      float* st = state + (size_t)state_slots[seq] * KEEP * C + c;
+      fvec_t old[KEEP > 0 ? KEEP : 1];             // the carried input that stands in tap j's place: row rel + j
+#pragma unroll
+      for (int j = 0; j < KEEP; ++j) old[j] = *reinterpret_cast<const fvec_t*>(st + (size_t)(rel + j < KEEP ? rel + j : KEEP - 1) * C);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) v[j] = KEEP - j <= rel ? widen(x[j]) : old[j < KEEP ? j : 0];
+      if (cu_q[seq + 1] - begin == 1) {            // the only reader of its slot moves the inputs on
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) *reinterpret_cast<fvec_t*>(st + (size_t)j * C) = v[j + 1];
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) v[j] = widen(x[j]);
+    }
+    emit(t, v);
+  }
 }
 
 // A thread a (sequence, channel) of the sequences that bring more than one token: it reads all it needs before it writes.
@@ -315,15 +409,24 @@ extern "C" int pa_time_conv(void* stream, int dtype, const void* h, long stride,
   const bool wide = channels % 8 == 0 && stride % 8 == 0 && out_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(h) & 15) == 0 &&
                     (reinterpret_cast<uintptr_t>(out) & 15) == 0;
   const int per = wide ? 8 : 1;
-  dim3 grid(tokens, (channels / per + 255) / 256), cgrid(nseq, (channels + 255) / 256);
+  constexpr int kRun = 8;
+  const bool four = wide && taps == 4 && ((reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(state)) & 31) == 0;
+  const bool runs = wide && tokens >= 64 * kRun;
+  dim3 grid(runs ? (tokens + kRun - 1) / kRun : tokens, (channels / per + 255) / 256), cgrid(nseq, (channels + 255) / 256);
   const int threads = channels / per >= 256 ? 256 : 64 * ((channels / per + 63) / 64);
-#define PA_CONV_V(T, V)                                                                                                         \
-  hipLaunchKernelGGL((time_conv_kernel<T, V>), grid, dim3(threads), 0, st, (const T*)h, (size_t)stride, w, in_bias, bias, state, \
-                     seq_of_token, cu_q, state_slots, (T*)out, (size_t)out_stride, channels, taps, act, add_input)
+#define PA_CONV_V(T, V, N)                                                                                                      \
+  hipLaunchKernelGGL((time_conv_kernel<T, V, N>), grid, dim3(threads), 0, st, (const T*)h, (size_t)stride, w, in_bias, bias, state, \
+                     seq_of_token, cu_q, state_slots, (T*)out, (size_t)out_stride, tokens, channels, taps, act, add_input)
+#define PA_CONV_4(T, N)                                                                                                         \
+  hipLaunchKernelGGL((time_conv_taps_kernel<T, 4, N>), grid, dim3(threads), 0, st, (const T*)h, (size_t)stride, w, in_bias, bias, \
+                     state, seq_of_token, cu_q, state_slots, (T*)out, (size_t)out_stride, tokens, channels, act, add_input)
 #define PA_CONV(T)                                                                                                              \
   do {                                                                                                                          \
-    if (wide) PA_CONV_V(T, 8);                                                                                                  \
-    else PA_CONV_V(T, 1);                                                                                                       \
+    if (four && runs) PA_CONV_4(T, kRun);                                                                                       \
+    else if (four) PA_CONV_4(T, 1);                                                                                             \
+    else if (runs) PA_CONV_V(T, 8, kRun);                                                                                            \
+    else if (wide) PA_CONV_V(T, 8, 1);                                                                                          \
+    else PA_CONV_V(T, 1, 1);                                                                                                       \
     if (taps > 1 && !all_single)                                                                                                \
       hipLaunchKernelGGL(time_conv_carry_kernel<T>, cgrid, dim3(256), 0, st, (const T*)h, (size_t)stride, in_bias, state, cu_q,  \
                          state_slots, channels, taps);                                                                          \
@@ -332,6 +435,7 @@ extern "C" int pa_time_conv(void* stream, int dtype, const void* h, long stride,
   else if (dtype == kBF16) PA_CONV(bf16);
   else return pa::fail("time_conv: unknown element type code %d", dtype);
 #undef PA_CONV
+#undef PA_CONV_4
 #undef PA_CONV_V
   return check_launch("time_conv");
 }

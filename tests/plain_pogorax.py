@@ -224,7 +224,7 @@ def parallel_layer(heads=4, kv_heads=2, dim=16, vdim=24, chunk=20, scale=0.3, rh
                       "right": {"heads": rheads, "dim": rdim, "vdim": rvdim, "gate_cap": cap}}}
 
 
-def parallel2_layer(heads=4, kv_heads=2, dim=16, vdim=24, rot=8, base=10000.0, scale=2.0, width=48, blocks=3, conv=5, ff=40):
+def parallel2_layer(heads=4, kv_heads=2, dim=16, vdim=24, rot=8, base=10000.0, scale=0.5, width=48, blocks=3, conv=5, ff=40):
     return {"type": "parallel_2", "mlp": _mlp(ff),
             "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "rot": {"base": base, "dims": rot}},
                       "right": {"width": width, "blocks": blocks, "conv": conv}}}
@@ -243,9 +243,9 @@ def tiny_config_s():
 
 def tiny_config_u():
     """Sizes the matrix cores take; one KV head; states larger than a chunk of tokens is long; a block for the whole width."""
-    return model([parallel2_layer(heads=4, kv_heads=1, dim=64, vdim=64, rot=64, scale=0.5, width=64, blocks=1, conv=4),
+    return model([parallel2_layer(heads=4, kv_heads=1, dim=64, vdim=64, rot=64, scale=0.2, width=64, blocks=1, conv=4),
                   mamba2_layer(heads=4, vdim=64, state=128, groups=4, conv=4, norm_groups=1),
-                  parallel_layer(heads=4, kv_heads=1, dim=64, vdim=128, chunk=96, scale=0.125, rheads=2, rdim=64, rvdim=128, cap=20.0),
+                  parallel_layer(heads=4, kv_heads=1, dim=64, vdim=128, chunk=80, scale=0.125, rheads=2, rdim=64, rvdim=128, cap=20.0),
                   parallel_layer(heads=8, kv_heads=4, dim=32, vdim=32, chunk=65, scale=0.2, rheads=4, rdim=128, rvdim=32)],
                  width=64, vocab=120, scale=1.5)
 
@@ -305,8 +305,6 @@ def random_weights(cfg, seed):
             x = 1.0 + 0.2 * n
         elif name.endswith(".f.b"):
             x = 3.0 + n
-        elif name.endswith((".i", ".f")):
-            x = 2.0 * n / math.sqrt(shape[-1])
         elif last == "dt_bias":
             x = n - 2.0
         elif last == "A_log":
@@ -320,8 +318,20 @@ def random_weights(cfg, seed):
         elif last == "conv":
             x = n / math.sqrt(shape[-1])
         elif last == "embed":
-            x = 0.4 * n
+            x = n
         else:
             x = n / math.sqrt(shape[-1])
         w[name] = x.to(torch.bfloat16).to(torch.float64).numpy()
     return w
+
+
+def movement(cfg, w, toks, seeds=2, size=2.0 ** -9):
+    """How far every position's logits move, in units of their spread, when every weight is off by a random part of its last
+    bfloat16 place: the largest over a few draws.  What rounding to bfloat16 does to a model is of this size."""
+    ref = forward(cfg, w, toks)
+    out = np.zeros(len(toks))
+    for s in range(seeds):
+        g = np.random.default_rng(s)
+        moved = forward(cfg, {k: v * (1.0 + size * g.standard_normal(v.shape)) for k, v in w.items()}, toks)
+        out = np.maximum(out, np.abs(moved - ref).max(axis=1) / ref.std())
+    return out
