@@ -468,7 +468,7 @@ __global__ __launch_bounds__(256) void scan_chunk_carry_kernel(ScanArgs<bf16> a,
 // (3) Grid as (1).  Every wavefront makes the weights of one tile of 16 keys against the queries of the chunk, then all of
 // them the outputs of their tiles of columns.
 template <int DP>
-__global__ __launch_bounds__(kScanThreads) void scan_chunk_out_kernel(ScanArgs<bf16> a, const int* __restrict__ seq_ids,
+__global__ __launch_bounds__(kScanThreads, DP <= 64 ? 3 : 1) void scan_chunk_out_kernel(ScanArgs<bf16> a, const int* __restrict__ seq_ids,
                                                                       const float* __restrict__ work, int max_chunks, int et_per) {
   constexpr int KS = DP / 32;
   extern __shared__ __align__(16) unsigned char scan_lds[];
@@ -544,6 +544,7 @@ __global__ __launch_bounds__(kScanThreads) void scan_chunk_out_kernel(ScanArgs<b
   __syncthreads();
   const float* wp = work + (idx * a.heads + h) * (size_t)(16 * tiles) * dpad;
   const float skip = a.skip ? a.skip[h] : 0.f;
+#pragma unroll 1
   for (int et = wave; et < etn; et += kScanThreads / kWave) {
     const int e = 16 * (et0 + et) + r;
     f32x4 acc[4];
@@ -581,20 +582,20 @@ __global__ __launch_bounds__(kScanThreads) void scan_chunk_out_kernel(ScanArgs<b
         acc[it] = mfma16(scan_piece(wh, 16 * it + r, 32 * ks + 8 * g), v, acc[it]);
       }
     }
+    // a column of S, or n's: from one base, a token a step
+    const bool is_n = e == a.vdim && a.den;
+    if (e >= a.vdim && !is_n) continue;
+    const int step = is_n ? a.heads : a.heads * a.vdim;
+    float* dst = is_n ? a.den + (size_t)row0 * a.heads + h : a.out + ((size_t)row0 * a.heads + h) * a.vdim + e;
 #pragma unroll
     for (int it = 0; it < 4; ++it)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int t = 16 * it + 4 * g + i;
         if (t >= n) continue;
-        const size_t at = (size_t)(row0 + t) * a.heads + h;
-        if (e < a.vdim) {
-          float o = acc[it][i];
-          if (a.skip) o = fmaf(skip, (float)vt[scan_at(16 * et + r, t)], o);
-          a.out[at * a.vdim + e] = o;
-        } else if (e == a.vdim && a.den) {
-          a.den[at] = acc[it][i];
-        }
+        float o = acc[it][i];
+        if (a.skip && !is_n) o = fmaf(skip, (float)vt[scan_at(16 * et + r, t)], o);
+        dst[(size_t)t * step] = o;
       }
   }
 }

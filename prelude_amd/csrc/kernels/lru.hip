@@ -103,21 +103,32 @@ __global__ __launch_bounds__(kLruThreads) void lru_gates_kernel(LruArgs<T> p, co
   p.finish(zr + br[c], zi + bi[c], to_f32(p.u[(size_t)t * p.width + c]), t, c, p.single_slot(seq_of_token[t]));
 }
 
-// Grid (runs of 16 * MT tokens, runs of 64 channels of a block, blocks); a wavefront 16 channels.
+// Grid (runs of 16 * MT tokens, runs of 64 channels of a block, blocks); a wavefront 16 channels, of which a lane holds four
+// neighbouring ones of one token.  MT = 4: the tokens' u go through LDS, 128 channels of the block at a time.
+constexpr int kLruPanel = 128;
+
 template <int MT>
 __global__ __launch_bounds__(kLruThreads) void lru_gates_mfma_kernel(LruArgs<bf16> p, const bf16* __restrict__ wr,
                                                                      const bf16* __restrict__ wi, const float* __restrict__ br,
                                                                      const float* __restrict__ bi, const int* __restrict__ seq_of_token,
                                                                      int size) {
+  constexpr bool STAGED = MT == 4;
+  constexpr int kRow = kLruPanel + 8;           // 16-byte reads of sixteen rows fall into different banks
+  constexpr int kPieces = 16 * MT * kLruPanel / 8 / kLruThreads;
+  __shared__ __align__(16) bf16 us[STAGED ? 16 * MT * kRow : 8];
+  __shared__ int slot_of[16 * MT];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
   const int g = lane / 16, r = lane % 16;
   const int t0 = blockIdx.x * 16 * MT;
-  const int o0 = blockIdx.y * 64 + 16 * wave;
-  if (o0 >= size) return;                       // (no barrier in this kernel)
+  const int o0 = blockIdx.y * 64 + 16 * wave;   // may lie past the block's end: such a wavefront only helps to stage
   const int base = blockIdx.z * size;
   const int o = o0 + r < size ? o0 + r : size - 1;
   const bf16* rr = wr + (size_t)(base + o) * size;
   const bf16* ri = wi + (size_t)(base + o) * size;
+  if ((int)threadIdx.x < 16 * MT) {
+    const int t = t0 + threadIdx.x;
+    slot_of[threadIdx.x] = t < p.tokens ? p.single_slot(seq_of_token[t]) : -1;
+  }
   const bf16* ur[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) {
@@ -127,40 +138,91 @@ __global__ __launch_bounds__(kLruThreads) void lru_gates_mfma_kernel(LruArgs<bf1
   f32x4 ar[MT], ai[MT];
 #pragma unroll
   for (int m = 0; m < MT; ++m) ar[m] = ai[m] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int k0 = 0; k0 < size; k0 += 32) {
-    const bool in = k0 + 8 * g < size;          // (a multiple of 8: a piece lies inside or outside whole)
-    const int k = in ? k0 + 8 * g : 0;
-    const bf16x8 fr = *reinterpret_cast<const bf16x8*>(rr + k), fi = *reinterpret_cast<const bf16x8*>(ri + k);
+  if (STAGED) {
+    bf16x8 raw[kPieces > 0 ? kPieces : 1];
+    auto fetch = [&](int k0) {
 #pragma unroll
-    for (int m = 0; m < MT; ++m) {
-      const bf16x8 v = *reinterpret_cast<const bf16x8*>(ur[m] + k);
-      const bf16x8 f = in ? v : zero8();
-      ar[m] = mfma16(f, fr, ar[m]);
-      ai[m] = mfma16(f, fi, ai[m]);
+      for (int i = 0; i < kPieces; ++i) {
+        const int piece = i * kLruThreads + threadIdx.x;
+        const int row = piece / (kLruPanel / 8), k = k0 + 8 * (piece % (kLruPanel / 8));
+        const int t = t0 + row < p.tokens ? t0 + row : p.tokens - 1;
+        const bf16x8 v = *reinterpret_cast<const bf16x8*>(p.u + (size_t)t * p.width + base + (k < size ? k : 0));
+        raw[i] = k < size ? v : zero8();        // (a multiple of 8: a piece lies inside or outside whole)
+      }
+    };
+    fetch(0);
+    for (int k0 = 0; k0 < size; k0 += kLruPanel) {
+      bf16x8 fr[kLruPanel / 32], fi[kLruPanel / 32];
+#pragma unroll
+      for (int ks = 0; ks < kLruPanel / 32; ++ks) {
+        const int k = k0 + 32 * ks + 8 * g < size ? k0 + 32 * ks + 8 * g : 0;
+        fr[ks] = *reinterpret_cast<const bf16x8*>(rr + k);
+        fi[ks] = *reinterpret_cast<const bf16x8*>(ri + k);
+      }
+      __syncthreads();
+#pragma unroll
+      for (int i = 0; i < kPieces; ++i) {
+        const int piece = i * kLruThreads + threadIdx.x;
+        *reinterpret_cast<bf16x8*>(us + (piece / (kLruPanel / 8)) * kRow + 8 * (piece % (kLruPanel / 8))) = raw[i];
+      }
+      __syncthreads();
+      if (k0 + kLruPanel < size) fetch(k0 + kLruPanel);
+#pragma unroll
+      for (int ks = 0; ks < kLruPanel / 32; ++ks)
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+          const bf16x8 f = *reinterpret_cast<const bf16x8*>(us + (16 * m + r) * kRow + 32 * ks + 8 * g);
+          ar[m] = mfma16(fr[ks], f, ar[m]);
+          ai[m] = mfma16(fi[ks], f, ai[m]);
+        }
+    }
+  } else {
+#pragma unroll 4
+    for (int k0 = 0; k0 < size; k0 += 32) {
+      const bool in = k0 + 8 * g < size;
+      const int k = in ? k0 + 8 * g : 0;
+      const bf16x8 fr = *reinterpret_cast<const bf16x8*>(rr + k), fi = *reinterpret_cast<const bf16x8*>(ri + k);
+#pragma unroll
+      for (int m = 0; m < MT; ++m) {
+        const bf16x8 v = *reinterpret_cast<const bf16x8*>(ur[m] + k);
+        const bf16x8 f = in ? v : zero8();
+        ar[m] = mfma16(fr, f, ar[m]);
+        ai[m] = mfma16(fi, f, ai[m]);
+      }
+    }
+    __syncthreads();                            // slot_of
+  }
+  if (o0 + 4 * g >= size) return;
+  const int c = base + o0 + 4 * g;
+  const f32x4 b0 = *reinterpret_cast<const f32x4*>(br + c), b1 = *reinterpret_cast<const f32x4*>(bi + c);
+  const f32x4 rate = *reinterpret_cast<const f32x4*>(p.rate + c);
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int t = t0 + 16 * m + r;
+    if (t >= p.tokens) continue;
+    const size_t at = (size_t)t * p.width + c;
+    const bf16x4 ut = *reinterpret_cast<const bf16x4*>(p.u + at);
+    f32x4 a4, x4;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float2 f = lru_gate<bf16>(ar[m][i] + b0[i], ai[m][i] + b1[i], rate[i]);
+      a4[i] = f.x;
+      x4[i] = f.y * (float)ut[i];
+    }
+    const int slot = slot_of[16 * m + r];
+    if (slot < 0) {
+      *reinterpret_cast<f32x4*>(p.a + at) = a4;
+      *reinterpret_cast<f32x4*>(p.x + at) = x4;
+    } else {
+      f32x4* sp = reinterpret_cast<f32x4*>(p.state + (size_t)slot * p.width + c);
+      f32x4 s4 = *sp;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) s4[i] = fmaf(a4[i], s4[i], x4[i]);
+      *sp = s4;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) p.out[(size_t)t * p.out_ld + c + i] = p.output(s4[i], t, c + i);
     }
   }
-  if (o0 + r >= size) return;
-  const int c = base + o0 + r;
-  const float b0 = br[c], b1 = bi[c];
-  // what the tokens' ends need is asked for before the first of them is written
-  int slot[MT][4];
-  bf16 ut[MT][4];
-#pragma unroll
-  for (int m = 0; m < MT; ++m)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = t0 + 16 * m + 4 * g + i < p.tokens ? t0 + 16 * m + 4 * g + i : p.tokens - 1;
-      slot[m][i] = p.single_slot(seq_of_token[t]);
-      ut[m][i] = p.u[(size_t)t * p.width + c];
-    }
-#pragma unroll
-  for (int m = 0; m < MT; ++m)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = t0 + 16 * m + 4 * g + i;
-      if (t < p.tokens) p.finish(ar[m][i] + b0, ai[m][i] + b1, (float)ut[m][i], t, c, slot[m][i]);
-    }
 }
 
 // Where chunk j of the z-th listed sequence keeps its sums (a different place for every chunk of the launch).
@@ -280,7 +342,10 @@ extern "C" int pa_lru_gates(void* stream, int dtype, const void* u, const void* 
   } else if (dtype == kBF16) {
     LruArgs<bf16> p;
     if (int rc = lru_args("lru_gates", p, u, rate, state, state_slots, cu_q, y, y_ld, y_bias, act, a, x, out, out_ld, out_scale, tokens, width)) return rc;
-    const bool pieces = size % 8 == 0 && ((reinterpret_cast<uintptr_t>(u) | reinterpret_cast<uintptr_t>(wr) | reinterpret_cast<uintptr_t>(wi)) & 15) == 0;
+    const uintptr_t all = reinterpret_cast<uintptr_t>(u) | reinterpret_cast<uintptr_t>(wr) | reinterpret_cast<uintptr_t>(wi) | reinterpret_cast<uintptr_t>(br) |
+                          reinterpret_cast<uintptr_t>(bi) | reinterpret_cast<uintptr_t>(rate) | reinterpret_cast<uintptr_t>(state) |
+                          reinterpret_cast<uintptr_t>(a) | reinterpret_cast<uintptr_t>(x);
+    const bool pieces = size % 8 == 0 && (all & 15) == 0;
     if (!pieces)
       hipLaunchKernelGGL(lru_gates_kernel<bf16>, dim3(tokens, (width + 255) / 256), dim3(kLruThreads), 0, st, p, (const bf16*)wr,
                          (const bf16*)wi, br, bi, seq_of_token, size);
